@@ -4,6 +4,7 @@ from .zederax import ZederaxConfig
 from .nakurax import NakuraxConfig
 from .tativik import TativikConfig
 from .kegetar import KegetarConfig
+from .lelatar import LelatarConfig
 from .engine_config import InferenceEngineConfig
 
-__all__ = ["ConfigError", "LmConfig", "Gpt2Config", "ZederaxConfig", "NakuraxConfig", "TativikConfig", "KegetarConfig", "InferenceEngineConfig"]
+__all__ = ["ConfigError", "LmConfig", "Gpt2Config", "ZederaxConfig", "NakuraxConfig", "TativikConfig", "KegetarConfig", "LelatarConfig", "InferenceEngineConfig"]

@@ -7,6 +7,7 @@
 //   write:  x <- x + mult * gn(y * sigmoid(gate), post_w)     the result y of the sublayer before (float32 [T][D]), gated element by
 //                                                              element by the sigmoid of gate (float32 or compute dtype, row stride
 //                                                              gate_stride; null: not gated), normalised and added to the residual
+//   sum:    x <- x + part[0] + .. + part[S-1] + part_bias       what a product into the stream has left undone (its K ranges [S][T][D], S = 0: none)
 //   read:   h = gn(x, w)                                       for the next sublayer, into h_out (compute dtype or float32; may be x
 //                                                              itself when there is no write); w == null: h = x as it is, only
 //                                                              rounded to h_out's type (a sublayer that reads the stream itself)
@@ -41,7 +42,8 @@ template <typename TG, typename TO, int PER>
 __global__ void __launch_bounds__(GN_NT)
 group_norm_step_kernel(float* __restrict__ x, const float* __restrict__ y, const TG* __restrict__ gate, long gate_stride,
                        const float* __restrict__ post_w, float mult, const float* __restrict__ w, TO* __restrict__ h_out,
-                       const int* __restrict__ rows, int D, int G, float eps) {
+                       const int* __restrict__ rows, int D, int G, float eps, const float* __restrict__ ranges, int n_ranges, size_t range_stride,
+                       const float* __restrict__ range_bias) {
   __shared__ float part[4 * GN_MAX_GROUPS], total[GN_MAX_GROUPS];
   const int tid = threadIdx.x;
   const int r = blockIdx.x, row = rows ? rows[r] : r;
@@ -61,6 +63,20 @@ group_norm_step_kernel(float* __restrict__ x, const float* __restrict__ y, const
     if (gate != nullptr) z[i] = z[i] / (1.0f + expf(-gt));
     if (e >= D) xv[i] = 0.f, z[i] = 0.f;
     gid[i] = e < D ? e / group_size : -1;
+  }
+  if (n_ranges > 0) {
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int e = tid + GN_NT * i, ec = min(e, D - 1);
+      float sum = 0.f;
+#pragma unroll 8
+      for (int r2 = 0; r2 < n_ranges; ++r2) sum += ranges[(size_t)r2 * range_stride + (size_t)row * D + ec];
+      if (range_bias != nullptr) sum += range_bias[ec];
+      if (e < D) {
+        xv[i] = sum + xv[i];
+        if (rows == nullptr && y == nullptr) x[(size_t)row * D + e] = xv[i];
+      }
+    }
   }
   if (y != nullptr) {
     group_inverse_rms<PER>(z, gid, G, inv_n, eps, part, total);
@@ -94,9 +110,11 @@ group_norm_step_kernel(float* __restrict__ x, const float* __restrict__ y, const
 
 template <typename TG, typename TO>
 static void group_norm_launch(float* x, const float* y, const void* gate, long gate_stride, const float* post_w, float mult, const float* w,
-                              void* h_out, const int* rows, int n, int D, int G, float eps, hipStream_t stream) {
+                              void* h_out, const int* rows, int n, int D, int G, float eps, const float* ranges, int n_ranges, size_t range_stride,
+                              const float* range_bias, hipStream_t stream) {
 #define GN_CASE(PER)                                                                                                                       \
-  group_norm_step_kernel<TG, TO, PER><<<n, GN_NT, 0, stream>>>(x, y, (const TG*)gate, gate_stride, post_w, mult, w, (TO*)h_out, rows, D, G, eps)
+  group_norm_step_kernel<TG, TO, PER><<<n, GN_NT, 0, stream>>>(x, y, (const TG*)gate, gate_stride, post_w, mult, w, (TO*)h_out, rows, D, G, eps, ranges, \
+                                                         n_ranges, range_stride, range_bias)
   if (D <= GN_NT) GN_CASE(1);
   else if (D <= GN_NT * 2) GN_CASE(2);
   else if (D <= GN_NT * 4) GN_CASE(4);
@@ -107,19 +125,21 @@ static void group_norm_launch(float* x, const float* y, const void* gate, long g
 }
 
 extern "C" int lev_group_norm_step(float* x, const float* y, const void* gate, long gate_stride, int gate_dtype, const float* post_w, float mult,
-                                   const float* w, void* h_out, int out_dtype, const int* rows, int n, int D, int G, float eps,
-                                   hipStream_t stream) {
+                                   const float* w, void* h_out, int out_dtype, const int* rows, int n, int D, int G, float eps, const float* ranges,
+                                   int n_ranges, int T, const float* range_bias, hipStream_t stream) {
   LEV_REQUIRE(n >= 0 && D > 0 && D <= GN_NT * GN_MAX_PER, "group norm: a row of %d numbers (at most %d)", D, GN_NT * GN_MAX_PER);
   LEV_REQUIRE(G > 0 && G <= GN_MAX_GROUPS && D % G == 0, "group norm: %d numbers do not split into %d equal groups (at most %d)", D, G, GN_MAX_GROUPS);
   LEV_REQUIRE(x != nullptr && (y == nullptr || post_w != nullptr), "group norm: a tensor is missing");
-  LEV_REQUIRE(y != nullptr || h_out != nullptr, "group norm: nothing to do");
+  LEV_REQUIRE(y != nullptr || h_out != nullptr || n_ranges > 0, "group norm: nothing to do");
+  LEV_REQUIRE(n_ranges >= 0 && (n_ranges == 0 || (ranges != nullptr && T > 0 && (void*)h_out != (void*)x)), "group norm: an unfinished sum needs its ranges");
+  const size_t range_stride = (size_t)T * D;
   LEV_REQUIRE(gate == nullptr || (y != nullptr && gate_stride >= D), "group norm: a gate needs a result to gate and rows of at least %d", D);
   LEV_REQUIRE((gate_dtype == LEV_F32 || gate_dtype == LEV_BF16) && (out_dtype == LEV_F32 || out_dtype == LEV_BF16), "group norm: unknown dtype");
   LEV_REQUIRE((void*)h_out != (void*)x || (y == nullptr && rows == nullptr && out_dtype == LEV_F32), "group norm: the output may be the input only without a write");
   if (n == 0) return 0;
-  if (gate_dtype == LEV_F32 && out_dtype == LEV_F32) group_norm_launch<float, float>(x, y, gate, gate_stride, post_w, mult, w, h_out, rows, n, D, G, eps, stream);
-  else if (gate_dtype == LEV_F32) group_norm_launch<float, bf16_t>(x, y, gate, gate_stride, post_w, mult, w, h_out, rows, n, D, G, eps, stream);
-  else if (out_dtype == LEV_F32) group_norm_launch<bf16_t, float>(x, y, gate, gate_stride, post_w, mult, w, h_out, rows, n, D, G, eps, stream);
-  else group_norm_launch<bf16_t, bf16_t>(x, y, gate, gate_stride, post_w, mult, w, h_out, rows, n, D, G, eps, stream);
+  if (gate_dtype == LEV_F32 && out_dtype == LEV_F32) group_norm_launch<float, float>(x, y, gate, gate_stride, post_w, mult, w, h_out, rows, n, D, G, eps, ranges, n_ranges, range_stride, range_bias, stream);
+  else if (gate_dtype == LEV_F32) group_norm_launch<float, bf16_t>(x, y, gate, gate_stride, post_w, mult, w, h_out, rows, n, D, G, eps, ranges, n_ranges, range_stride, range_bias, stream);
+  else if (out_dtype == LEV_F32) group_norm_launch<bf16_t, float>(x, y, gate, gate_stride, post_w, mult, w, h_out, rows, n, D, G, eps, ranges, n_ranges, range_stride, range_bias, stream);
+  else group_norm_launch<bf16_t, bf16_t>(x, y, gate, gate_stride, post_w, mult, w, h_out, rows, n, D, G, eps, ranges, n_ranges, range_stride, range_bias, stream);
   return lev_check_launch("group_norm_step");
 }

@@ -696,10 +696,11 @@ extern "C" int lev_glu_activate(const void* z, long z_stride, void* out, long o_
 
 // ------------------------------------------------------------------------------------------
 // The sum of two branches that each pass an RMS norm of their own first: y = sa * a / rms(a) * wa + sb * b / rms(b) * wb over rows
-// of D float32 numbers, rms(v) = sqrt(mean(v^2) + eps). One workgroup per row; `y` may be `a` or `b`.
+// of D float32 numbers, rms(v) = sqrt(mean(v^2) + eps). One workgroup per row; `y` may be `a` or `b`. accumulate: the sum is added to
+// what y holds.
 __global__ void __launch_bounds__(256)
 norm_sum2_kernel(const float* __restrict__ a, const float* __restrict__ b, const float* __restrict__ wa, const float* __restrict__ wb, float sa,
-                 float sb, float eps, float* __restrict__ y, int D) {
+                 float sb, float eps, float* __restrict__ y, int D, int accumulate) {
   __shared__ float red[8];
   const size_t row = (size_t)blockIdx.x * D;
   float ssa = 0.f, ssb = 0.f;
@@ -711,13 +712,117 @@ norm_sum2_kernel(const float* __restrict__ a, const float* __restrict__ b, const
   ssa = block_sum<256>(ssa, red);
   ssb = block_sum<256>(ssb, red);
   const float ra = sa / sqrtf(ssa / (float)D + eps), rb = sb / sqrtf(ssb / (float)D + eps);
-  for (int d = threadIdx.x; d < D; d += 256) y[row + d] = a[row + d] * ra * wa[d] + b[row + d] * rb * wb[d];
+  for (int d = threadIdx.x; d < D; d += 256) {
+    const float sum = a[row + d] * ra * wa[d] + b[row + d] * rb * wb[d];
+    y[row + d] = accumulate ? y[row + d] + sum : sum;
+  }
 }
 
 extern "C" int lev_norm_sum2(const float* a, const float* b, const float* wa, const float* wb, float sa, float sb, float eps, float* y, int T, int D,
-                             hipStream_t stream) {
+                             int accumulate, hipStream_t stream) {
   LEV_REQUIRE(T >= 0 && D > 0 && a && b && wa && wb && y, "norm_sum2: a tensor is missing or bad sizes T=%d D=%d", T, D);
   if (T == 0) return 0;
-  norm_sum2_kernel<<<T, 256, 0, stream>>>(a, b, wa, wb, sa, sb, eps, y, D);
+  norm_sum2_kernel<<<T, 256, 0, stream>>>(a, b, wa, wb, sa, sb, eps, y, D, accumulate);
   return lev_check_launch("norm_sum2");
+}
+
+// ------------------------------------------------------------------------------------------
+// A token's row of a table as a further input of a layer: out[t][i] = gelu_tanh(z[t][i]) * table[tokens[t]][i]. z is float32 (a product's
+// 32-bit sums), the table and the output are of the compute dtype.
+template <typename T>
+__global__ void __launch_bounds__(256)
+token_gate_kernel(const float* __restrict__ z, long z_stride, const int* __restrict__ tokens, const T* __restrict__ table, T* __restrict__ out,
+                  int Tn, int D) {
+  const long idx = (long)blockIdx.x * 256 + threadIdx.x;
+  if (idx >= (long)Tn * D) return;
+  const int t = (int)(idx / D), i = (int)(idx - (long)t * D);
+  out[idx] = from_float<T>(lev_activate(z[(size_t)t * z_stride + i], LEV_ACT_GELU_TANH) * to_float<T>(table[(size_t)tokens[t] * D + i]));
+}
+
+extern "C" int lev_token_gate(const float* z, long z_stride, const int* tokens, const void* table, void* out, int T, int D, int dtype, hipStream_t stream) {
+  LEV_REQUIRE(T >= 0 && D > 0 && z && tokens && table && out && z_stride >= D, "token_gate: a tensor is missing or bad sizes T=%d D=%d", T, D);
+  LEV_REQUIRE(dtype == LEV_F32 || dtype == LEV_BF16, "token_gate: unknown dtype %d", dtype);
+  if (T == 0) return 0;
+  const unsigned blocks = (unsigned)(((long)T * D + 255) / 256);
+  if (dtype == LEV_F32) token_gate_kernel<float><<<blocks, 256, 0, stream>>>(z, z_stride, tokens, (const float*)table, (float*)out, T, D);
+  else token_gate_kernel<bf16_t><<<blocks, 256, 0, stream>>>(z, z_stride, tokens, (const bf16_t*)table, (bf16_t*)out, T, D);
+  return lev_check_launch("token_gate");
+}
+
+// ------------------------------------------------------------------------------------------
+// Queries and keys normed over their whole projections (all heads of a token at once, with a weight as wide as the projection), then
+// rotated, in one kernel with 32-bit numbers between the two: one workgroup per (token, queries | keys | values). `half`: dimension i of a
+// head is paired with i + n_pairs, else 2i with 2i + 1; i < n_pairs, the rest of a head passes unrotated. Queries change in place. With
+// pages (steps of single tokens) keys and values go into them at dest[t] and stay as they are in k and v; without, keys change in place
+// and values are not touched. The arithmetic is the same either way. norm_dim_*: the projections' true sizes (heads may carry zeros).
+template <typename T>
+__global__ void __launch_bounds__(256)
+projection_norm_rotate_kernel(T* __restrict__ q, long q_stride, int H, T* __restrict__ k, long k_stride, int G, int hd, const T* __restrict__ v,
+                              long v_stride, int vd, float eps, int norm_dim_q, int norm_dim_k, const float* __restrict__ wq,
+                              const float* __restrict__ wk, const float* __restrict__ freqs, int n_pairs, int half, const int* __restrict__ positions,
+                              T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ dest, int PS) {
+  __shared__ float red[4];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int dst = k_pages ? dest[t] : 0, page = max(dst, 0) / max(PS, 1), off = k_pages ? max(dst, 0) % PS : 0;
+  if (blockIdx.y == 2) {  // values: single tokens only
+    if (dst < 0) return;
+    for (int e = tid; e < G * vd; e += 256) v_pages[((size_t)page * G * vd + e) * PS + off] = v[(size_t)t * v_stride + e];
+    return;
+  }
+  const bool is_q = blockIdx.y == 0;
+  const int heads = is_q ? H : G, n = heads * hd;
+  T* row = is_q ? q + (size_t)t * q_stride : k + (size_t)t * k_stride;
+  const float* w = is_q ? wq : wk;
+  float ss = 0.f;
+  for (int d = tid; d < n; d += 256) {
+    const float x = to_float<T>(row[d]);
+    ss = fmaf(x, x, ss);
+  }
+  ss = block_sum<256>(ss, red);
+  const float r = 1.0f / sqrtf(ss / (float)(is_q ? norm_dim_q : norm_dim_k) + eps);
+  if (!is_q && dst < 0) return;
+  const float pos = n_pairs ? (float)positions[t] : 0.f;
+  T* kd = is_q || !k_pages ? nullptr : k_pages + (size_t)page * G * hd * PS;
+  auto put = [&](int head, int d, float val) {
+    if (kd) kd[(size_t)head * hd * PS + ((size_t)(d >> 3) * PS + off) * 8 + (d & 7)] = from_float<T>(val);
+    else row[head * hd + d] = from_float<T>(val);
+  };
+  const int items = hd - n_pairs;  // of a head: its pairs, then the dimensions that do not turn
+  for (int it = tid; it < heads * items; it += 256) {
+    const int head = it / items, i = it - head * items;
+    if (i < n_pairs) {
+      const int d0 = half ? i : 2 * i, d1 = half ? i + n_pairs : 2 * i + 1;
+      const float a = to_float<T>(row[head * hd + d0]) * r * w[head * hd + d0], b = to_float<T>(row[head * hd + d1]) * r * w[head * hd + d1];
+      float sn, cs;
+      sincosf(pos * freqs[i], &sn, &cs);
+      put(head, d0, a * cs - b * sn);
+      put(head, d1, b * cs + a * sn);
+    } else {
+      const int d = i + n_pairs;
+      put(head, d, to_float<T>(row[head * hd + d]) * r * w[head * hd + d]);
+    }
+  }
+}
+
+extern "C" int lev_projection_norm_rotate(void* q, long q_stride, int H, void* k, long k_stride, int G, int hd, const void* v, long v_stride, int vd,
+                                          float eps, int norm_dim_q, int norm_dim_k, const float* wq, const float* wk, const float* freqs, int n_pairs,
+                                          int half, const int* positions, void* k_pages, void* v_pages, const int* dest, int PS, int T, int dtype,
+                                          hipStream_t stream) {
+  LEV_REQUIRE(T >= 0 && H > 0 && G > 0 && hd > 0 && hd % 8 == 0, "projection_norm_rotate: bad sizes T=%d heads=%d/%d size=%d", T, H, G, hd);
+  LEV_REQUIRE(q && k && wq && wk && norm_dim_q > 0 && norm_dim_q <= H * hd && norm_dim_k > 0 && norm_dim_k <= G * hd, "projection_norm_rotate: a tensor is missing or bad divisors");
+  LEV_REQUIRE(q_stride >= (long)H * hd && k_stride >= (long)G * hd, "projection_norm_rotate: row strides are smaller than the heads");
+  LEV_REQUIRE(n_pairs >= 0 && 2 * n_pairs <= hd && (n_pairs == 0 || (freqs && positions)), "projection_norm_rotate: %d rotated pairs need frequencies, positions and a head of at least twice their number", n_pairs);
+  LEV_REQUIRE(!k_pages || (v && v_pages && dest && vd > 0 && PS > 0 && PS % 16 == 0 && v_stride >= (long)G * vd), "projection_norm_rotate: pages need values, destinations and a page size that is a multiple of 16");
+  LEV_REQUIRE(dtype == LEV_F32 || dtype == LEV_BF16, "projection_norm_rotate: unknown dtype %d", dtype);
+  if (T == 0) return 0;
+  const dim3 grid(T, k_pages ? 3 : 2);
+  if (dtype == LEV_F32)
+    projection_norm_rotate_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, H, (float*)k, k_stride, G, hd, (const float*)v, v_stride, vd, eps,
+                                                                  norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, half, positions, (float*)k_pages,
+                                                                  (float*)v_pages, dest, PS);
+  else
+    projection_norm_rotate_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)q, q_stride, H, (bf16_t*)k, k_stride, G, hd, (const bf16_t*)v, v_stride, vd, eps,
+                                                                   norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, half, positions, (bf16_t*)k_pages,
+                                                                   (bf16_t*)v_pages, dest, PS);
+  return lev_check_launch("projection_norm_rotate");
 }

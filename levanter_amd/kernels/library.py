@@ -534,6 +534,37 @@ class HipKernels:
                                                   _ptr(k_norm_weight), _ptr(rotary_freqs) if n_pairs else None, n_pairs, _ptr(positions) if n_pairs else None,
                                                   float(rotary_magnitude), T, _DT[dt], self._s()))
 
+    def projection_norm_rotate(self, q, k, n_heads: int, n_kv_heads: int, head_dim: int, eps: float, q_weight, k_weight, q_norm_dim: Optional[int] = None,
+                               k_norm_dim: Optional[int] = None, freqs=None, positions=None, half: bool = False, v=None, value_dim: int = 0, k_pages=None,
+                               v_pages=None, dest=None, page_size: int = 0) -> None:
+        """Queries and keys (``[T, heads*head_dim]``) divided by the root mean square of their whole rows (mean over ``*_norm_dim``; the rows may
+        carry zeros) and multiplied by float32 weights as wide as the rows, then rotated by ``positions[t] * freqs[i]`` (``freqs`` None: not at all):
+        dimension ``i`` of a head with ``i + len(freqs)`` (``half``) or ``2i`` with ``2i + 1``. Queries in place; keys in place, or, with pages, into
+        them at ``dest`` together with the values (``kv_write``). One kernel, the same arithmetic either way."""
+        _dev(q, k, q_weight, k_weight, freqs, positions, v, k_pages, v_pages, dest)
+        T, dt = q.shape[0], q.dtype
+        _req(dt in _DT and k.dtype == dt and q.shape == (T, n_heads * head_dim) and k.shape == (T, n_kv_heads * head_dim), "projection_norm_rotate: q and k must be [T, heads*head_dim] of one compute dtype")
+        for w, n in ((q_weight, n_heads), (k_weight, n_kv_heads)):
+            _req(w.dtype == torch.float32 and w.numel() == n * head_dim and w.is_contiguous(), "projection_norm_rotate: the norms' weights must be float32 and as wide as the projections")
+        n_pairs = 0
+        if freqs is not None and freqs.numel():
+            _req(freqs.dtype == torch.float32 and freqs.is_contiguous() and 2 * freqs.numel() <= head_dim, "projection_norm_rotate: float32 frequencies, at most head_dim / 2")
+            _req(positions is not None and positions.dtype == torch.int32 and positions.numel() == T, "projection_norm_rotate: one int32 position per token")
+            n_pairs = freqs.numel()
+        vs = 0
+        if k_pages is not None:
+            _req(dt == k_pages.dtype == v_pages.dtype == v.dtype and v.shape == (T, n_kv_heads * value_dim), "projection_norm_rotate: values must be [T, kv_heads*value_dim] of the pages' dtype")
+            _req(dest.dtype == torch.int32 and dest.numel() == T, "projection_norm_rotate: one int32 destination per token")
+            n = k_pages.numel()
+            _req(k_pages.is_contiguous() and v_pages.is_contiguous() and n % (n_kv_heads * head_dim * page_size) == 0 and n * value_dim == v_pages.numel() * head_dim,
+                 "projection_norm_rotate: page tensors must be contiguous and fit the sizes")
+            vs = _rows(v, "projection_norm_rotate: v")
+        self._check(self.lib.lev_projection_norm_rotate(
+            _ptr(q), _rows(q, "projection_norm_rotate: q"), int(n_heads), _ptr(k), _rows(k, "projection_norm_rotate: k"), int(n_kv_heads), int(head_dim),
+            _ptr(v) if k_pages is not None else None, vs, int(value_dim), float(eps), int(q_norm_dim or n_heads * head_dim), int(k_norm_dim or n_kv_heads * head_dim),
+            _ptr(q_weight), _ptr(k_weight), _ptr(freqs) if n_pairs else None, n_pairs, int(bool(half)), _ptr(positions) if n_pairs else None, _ptr(k_pages),
+            _ptr(v_pages), _ptr(dest) if k_pages is not None else None, int(page_size), T, _DT[dt], self._s()))
+
     def norm_write_latent(self, c, weight, eps: float, norm_dim: int, k_pages, v_pages, dest, page_size: int) -> None:
         """``c`` ``[T, R]`` (one key/value head that all query heads share) becomes its RMS norm with ``weight`` (float32 ``[R]``;
         the mean of squares is over ``norm_dim``), in place, and goes into the key and the value pages at ``dest``: what
@@ -837,8 +868,14 @@ class HipKernels:
         (compute dtype or float32; ``plain_read``: ``h_out = x`` as it is, only rounded to ``h_out``'s type, for a sublayer that reads the
         stream itself). ``rows``: only these rows, into ``h_out [len(rows), D]``; ``x`` is not stored then.
         ``defer``: nothing is launched; the write comes back as a ``PendingGatedNorm`` for the next call (``pending=``) or
-        ``finish``. ``pending``: the write of an earlier call, done in this pass."""
-        if pending is not None:
+        ``finish``. ``pending``: the write of an earlier call, or a product into ``x`` that has left its K ranges undone (a
+        ``PendingSum``; added before anything else), done in this pass."""
+        part = part_bias = None
+        n_ranges = 0
+        if isinstance(pending, PendingSum):
+            _req(pending.out is x and pending.ldo == x.shape[1] and h_out is not x, "group norm: the unfinished product belongs to another tensor")
+            part, n_ranges, part_bias = pending.workspace, pending.n_ranges, pending.bias
+        elif pending is not None:
             _req(pending.out is x and y is None and pending.groups == groups and pending.eps == eps, "group norm: the unfinished sublayer belongs to another tensor or norm")
             y, gate, post_weight, mult = pending.y, pending.gate, pending.post_weight, pending.mult
         if defer:
@@ -862,7 +899,7 @@ class HipKernels:
             _req((weight is not None) != bool(plain_read) and h_out.dtype in _DT and h_out.is_contiguous() and tuple(h_out.shape) == (n, D), "group norm: bad normalised output")
             odt = h_out.dtype
         self._check(self.lib.lev_group_norm_step(_ptr(x), _ptr(y), _ptr(gate), gs, _DT[gdt], _ptr(post_weight), float(mult), _ptr(weight), _ptr(h_out),
-                                                 _DT[odt], _ptr(rows), n, D, int(groups), float(eps), self._s()))
+                                                 _DT[odt], _ptr(rows), n, D, int(groups), float(eps), _ptr(part), int(n_ranges), T, _ptr(part_bias), self._s()))
         return None
 
     # ---- rotation, "rotate half" layout --------------------------------------------------------
@@ -947,6 +984,49 @@ class HipKernels:
             return
         self._check(self.lib.lev_gla_tokens(*head, T, *tail))
 
+    # ---- a matrix state per head with one decay a token, behind a short convolution (state-space duality, gated delta rule) -------
+    STATE_RULES = {"ssd": 0, "delta": 1}
+
+    def state_recurrence(self, rule: str, x, taps, conv_bias, a, b, a_bias, rate, skip, gate, norm_weight, state, token_slots, positions, out, *, n_heads: int,
+                         n_groups: int, key_dim: int, value_dim: int, q_offset: int, k_offset: int, v_offset: int, norm_groups: int, norm_eps: float,
+                         key_eps: float = 0.0, q_scale: float = 1.0, max_runs: Optional[int] = None) -> None:
+        """From a mixer's projections to what its output projection reads, in 32-bit. ``x`` ``[T, C]`` (compute dtype, rows may be strided)
+        passes a causal convolution per channel (``taps`` float32 ``[C, K]``, the last column is the current token's; ``conv_bias`` or None) and
+        silu; queries, keys (``n_groups`` of ``key_dim``) and values (``n_heads`` of ``value_dim``) are the channels from ``*_offset`` on; head h
+        reads group ``h // (n_heads / n_groups)``. With ``sp = softplus(a + a_bias)`` (``a`` ``[T, H]``) and the decay ``d = exp(-rate * sp)``:
+
+        * rule "ssd": ``S <- d S + sp k v^T``, ``y = (S^T q + skip v) * silu(gate)``, ``out = y / rms(y) * norm_weight`` with the root mean square over
+          ``norm_groups`` equal parts of the row ``[H * dv]``;
+        * rule "delta": q and k become unit vectors (``key_eps``), q times ``q_scale``; ``S <- d S``, ``S <- S + k (sigmoid(b) (v - S^T k))^T``, ``o = S^T q``,
+          ``out = o / rms(o) * norm_weight * silu(gate)`` per head.
+
+        ``state`` float32 ``[slots, K * C + H * dk * dv]``: the convolution's inputs by position mod K, then S; read and stored. ``token_slots``:
+        -1 for a token of nobody (zeros). ``max_runs`` (at most this many runs of consecutive tokens of one slot): the step has runs longer than
+        one token; None: every token is a run of its own."""
+        _dev(x, taps, conv_bias, a, b, a_bias, rate, skip, gate, norm_weight, state, token_slots, positions, out)
+        T, C = x.shape
+        dt = x.dtype
+        H, G, dk, dv = int(n_heads), int(n_groups), int(key_dim), int(value_dim)
+        K = taps.shape[1]
+        _req(rule in self.STATE_RULES, f"state recurrence: unknown rule {rule!r}")
+        _req(dt in _DT and a.dtype == gate.dtype == out.dtype == dt and (b is None or b.dtype == dt), "state recurrence: x, a, b, gate and out must share a compute dtype")
+        _req(tuple(a.shape) == (T, H) and (b is None or tuple(b.shape) == (T, H)), "state recurrence: a and b must be [T, heads]")
+        _req(tuple(gate.shape) == tuple(out.shape) == (T, H * dv), "state recurrence: gate and out must be [T, heads*value_dim]")
+        _req(taps.dtype == torch.float32 and tuple(taps.shape) == (C, K) and taps.is_contiguous(), "state recurrence: taps must be float32 [C, K]")
+        for name, w, n in (("conv_bias", conv_bias, C), ("a_bias", a_bias, H), ("rate", rate, H), ("skip", skip, H), ("norm_weight", norm_weight, H * dv)):
+            _req(w is None or (w.dtype == torch.float32 and w.numel() == n and w.is_contiguous()), f"state recurrence: {name} must be float32 with {n} entries")
+        _req(state.dtype == torch.float32 and state.dim() == 2 and state.is_contiguous() and state.shape[1] >= K * C + H * dk * dv, "state recurrence: state must be float32 [slots, K*C + heads*dk*dv]")
+        for t in (token_slots, positions):
+            _req(t.dtype == torch.int32 and t.numel() == T, "state recurrence: one int32 slot and position per token")
+        runs = 0 if max_runs is None else max(1, min(int(max_runs), T))
+        ws = torch.empty(self.lib.lev_state_recurrence_workspace(T, H, G, dv, C, int(runs > 0), _DT[dt]), dtype=torch.uint8, device=x.device)
+        self._check(self.lib.lev_state_recurrence(
+            self.STATE_RULES[rule], _ptr(x), _rows(x, "state recurrence: x"), _ptr(taps), _ptr(conv_bias), _ptr(a), _rows(a, "state recurrence: a"), _ptr(b),
+            _rows(b, "state recurrence: b") if b is not None else H, _ptr(a_bias), _ptr(rate), _ptr(skip), _ptr(gate), _rows(gate, "state recurrence: gate"),
+            _ptr(norm_weight), _ptr(state), state.shape[1], _ptr(token_slots), _ptr(positions), _ptr(out), _rows(out, "state recurrence: out"), _ptr(ws), T,
+            runs if T else 0, H, G, dk, dv, C, K, int(q_offset), int(k_offset), int(v_offset), int(norm_groups), float(norm_eps), float(key_eps), float(q_scale),
+            _DT[dt], self._s()))
+
     # ---- row kernels of gated feed-forwards and of branches with norms of their own ---------------
     def glu_activate(self, z, out, activation: str, limit: float = 0.0, up_shift: float = 0.0) -> None:
         """``z`` ``[T, 2F]`` (gate sums, then up sums; rows may be strided) -> ``out`` ``[T, F]`` (may be ``z[:, :F]``):
@@ -958,16 +1038,26 @@ class HipKernels:
         self._check(self.lib.lev_glu_activate(_ptr(z), _rows(z, "glu_activate: z"), _ptr(out), _rows(out, "glu_activate: out"), T, F2 // 2,
                                               ACTIVATIONS[activation], float(limit), float(up_shift), _DT[z.dtype], self._s()))
 
-    def norm_sum2(self, a, b, weight_a, weight_b, scale_a: float, scale_b: float, eps: float, y) -> None:
+    def norm_sum2(self, a, b, weight_a, weight_b, scale_a: float, scale_b: float, eps: float, y, accumulate: bool = False) -> None:
         """``y = scale_a * a / rms(a) * weight_a + scale_b * b / rms(b) * weight_b`` over rows, ``rms(v) = sqrt(mean(v^2) + eps)``; all
-        float32, ``y`` may be ``a`` or ``b``."""
+        float32, ``y`` may be ``a`` or ``b``. ``accumulate``: added to what ``y`` holds."""
         _dev(a, b, weight_a, weight_b, y)
         T, D = a.shape
         for t in (a, b, y):
             _req(t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (T, D), "norm_sum2: contiguous float32 [T, D] tensors")
         for w in (weight_a, weight_b):
             _req(w.dtype == torch.float32 and w.is_contiguous() and w.numel() == D, "norm_sum2: the weights must be float32 [D]")
-        self._check(self.lib.lev_norm_sum2(_ptr(a), _ptr(b), _ptr(weight_a), _ptr(weight_b), float(scale_a), float(scale_b), float(eps), _ptr(y), T, D, self._s()))
+        self._check(self.lib.lev_norm_sum2(_ptr(a), _ptr(b), _ptr(weight_a), _ptr(weight_b), float(scale_a), float(scale_b), float(eps), _ptr(y), T, D, int(bool(accumulate)), self._s()))
+
+    def token_gate(self, z, tokens, table, out) -> None:
+        """``out[t] = gelu_tanh(z[t]) * table[tokens[t]]``: ``z`` float32 ``[T, D]`` (rows may be strided), ``table`` ``[vocab, D]`` and ``out``
+        ``[T, D]`` of one compute dtype. Token ids are trusted (the step checks them)."""
+        _dev(z, tokens, table, out)
+        T, D = out.shape
+        _req(z.dtype == torch.float32 and tuple(z.shape) == (T, D), "token_gate: z must be float32 [T, D]")
+        _req(tokens.dtype == torch.int32 and tokens.numel() == T, "token_gate: one int32 token per row")
+        _req(table.dtype == out.dtype and table.dtype in _DT and table.is_contiguous() and out.is_contiguous() and table.dim() == 2 and table.shape[1] == D, "token_gate: table [vocab, D] and out [T, D] must be contiguous and of one compute dtype")
+        self._check(self.lib.lev_token_gate(_ptr(z), _rows(z, "token_gate: z"), _ptr(tokens), _ptr(table), _ptr(out), T, D, _DT[out.dtype], self._s()))
 
     # ---- mixture of experts --------------------------------------------------------------------
     def moe_route(self, z, correction, chosen, weights, *, n_groups: int = 1, keep: int = 1, group_top: int = 2, renormalize: bool = False,

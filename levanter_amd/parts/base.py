@@ -220,6 +220,18 @@ class StreamMix(Part):
         raise NotImplementedError
 
 
+class StreamEntry(Part):
+    """Changes the residual stream ``x`` (float32 ``[T, dim]``) in place right before a plan entry that names it, for instance where a pass of
+    a loop over layers begins. ``begin(x, ctx)`` is called once a step, with the embedding's output; ``enter_run(x, run, ctx)`` before the
+    entry, with the number the entry gives (what is unfinished about ``x`` is in ``ctx.pending``). What it keeps lives in ``ctx.shared``."""
+
+    def begin(self, x: torch.Tensor, ctx: StepContext) -> None:
+        return None
+
+    def enter_run(self, x: torch.Tensor, run: int, ctx: StepContext) -> None:
+        raise NotImplementedError
+
+
 class Block:
     """Arranges the parts of a layer around the residual stream. Built from ``parts``: role -> built part, with the
     roles its description names; ``roles`` lists the ones this block cannot do without. One plan entry has one

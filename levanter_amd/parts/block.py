@@ -1,5 +1,6 @@
 """Blocks: how the parts of a layer are arranged around the residual stream.
-Pre-norm (src/levanter/models/gpt2.py:237-248): x += mixer(norm1(x)); x += feed_forward(norm2(x))."""
+Pre-norm (src/levanter/models/gpt2.py:237-248): x += mixer(norm1(x)); x += feed_forward(norm2(x)). A layer may have no
+feed-forward, and may end with a part that adds to the stream as a function of the stream and the token ids (``token_input``)."""
 from __future__ import annotations
 
 from typing import Dict
@@ -13,21 +14,30 @@ from .registry import BLOCKS
 
 @BLOCKS.register("pre_norm")
 class PreNormBlock(Block):
-    roles = ("norm1", "mixer", "norm2", "feed_forward")
-    defers_residual = True
+    roles = ("norm1", "mixer")
+    defers_residual = True  # x is read through the norms and the parts only
 
     def __init__(self, parts: Dict[str, Part]):
         super().__init__(parts)
-        self.norm1, self.mixer, self.norm2, self.feed_forward = (parts[r] for r in self.roles)
+        unknown = [r for r in parts if r not in ("norm1", "mixer", "norm2", "feed_forward", "token_input")]
+        if unknown:
+            raise ValueError(f"block 'pre_norm' has no role {', '.join(unknown)}")
+        self.norm1, self.mixer = parts["norm1"], parts["mixer"]
+        self.norm2, self.feed_forward, self.token_input = (parts.get(r) for r in ("norm2", "feed_forward", "token_input"))
+        if (self.norm2 is None) != (self.feed_forward is None):
+            raise ValueError("block 'pre_norm': norm2 and feed_forward come together or not at all")
 
     def forward(self, x: torch.Tensor, ctx: StepContext, unit: CacheUnitView, writes_cache: bool) -> None:
         # a product that the part before has left unfinished is folded into the norm that follows it, or finished first
         if not self.norm1.folds_pending:
             ctx.settle()
         self.mixer.forward(self.norm1(x, ctx), x, ctx, unit, writes_cache)
-        if not self.norm2.folds_pending:
-            ctx.settle()
-        self.feed_forward.forward(self.norm2(x, ctx), x, ctx)
+        if self.feed_forward is not None:
+            if not self.norm2.folds_pending:
+                ctx.settle()
+            self.feed_forward.forward(self.norm2(x, ctx), x, ctx)
+        if self.token_input is not None:
+            self.token_input.add(x, ctx)
 
 
 @BLOCKS.register("parallel")

@@ -31,6 +31,7 @@ class DecoderLm:
         self.embedding = build(spec.embedding, "embedding")
         self.blocks = [BLOCKS.get(layer.block)({role: build(part) for role, part in layer.parts.items()}) for layer in spec.layers]
         self.plan = list(spec.plan)
+        self.stream_entries = [build(part, "stream_mix") for part in spec.stream_entries]
         self.final_norm = build(spec.final_norm, "norm")
         self.head = build(spec.head, "head")
         self.head.bind(self.embedding)
@@ -41,6 +42,8 @@ class DecoderLm:
         for i, e in enumerate(self.plan):
             if not 0 <= e.layer < len(self.blocks):
                 raise ValueError(f"plan entry {i} names layer {e.layer}, the model has {len(self.blocks)}")
+            if e.enters is not None and not 0 <= e.enters[0] < len(self.stream_entries):
+                raise ValueError(f"plan entry {i} names stream entry {e.enters[0]}, the model has {len(self.stream_entries)}")
             if e.writes_cache:
                 if e.cache in owners:
                     raise ValueError(f"plan entries {owners[e.cache]} and {i} both write cache unit {e.cache}")
@@ -57,7 +60,7 @@ class DecoderLm:
     @property
     def graph_safe(self) -> bool:
         """Every part agrees to be replayed from a HIP graph (a block answers for its members)."""
-        return all(getattr(p, "graph_safe", False) for p in (self.embedding, *self.blocks, self.final_norm, self.head))
+        return all(getattr(p, "graph_safe", False) for p in (self.embedding, *self.blocks, *self.stream_entries, self.final_norm, self.head))
 
     @property
     def max_positions(self) -> Optional[int]:
@@ -89,8 +92,12 @@ class DecoderLm:
 
     def _forward(self, ctx: StepContext, logit_rows: torch.Tensor) -> torch.Tensor:
         x = self.embedding(ctx)
+        for s in self.stream_entries:
+            s.begin(x, ctx)
         for e in self.plan:
             block = self.blocks[e.layer]
+            if e.enters is not None:
+                self.stream_entries[e.enters[0]].enter_run(x, e.enters[1], ctx)
             ctx.may_defer = bool(block.defers_residual)
             if not ctx.may_defer:
                 ctx.settle()  # this block may read the residual stream in ways of its own

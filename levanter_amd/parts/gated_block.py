@@ -16,17 +16,38 @@ from typing import Dict, Optional
 
 import torch
 
-from levanter_amd.kernels.library import PendingGatedNorm
+from levanter_amd.kernels.library import PendingGatedNorm, PendingProduct, PendingSum
 from .base import Block, BuildEnv, CacheUnitView, Norm, Part, StepContext
 from .linear import Linear
 from .registry import BLOCKS, NORMS, STREAM_MIXES
 from .spec import PartSpec
 
 
+def take_foldable(x: torch.Tensor, ctx: StepContext, groups: int, eps: float):
+    """What is unfinished about the stream ``x`` and can be done inside a ``group_norm_step`` of this grouping (a gated write of the same
+    norm, a product that has left its K ranges); anything else is finished here. None: nothing is left to do."""
+    pending = ctx.take_pending(x)
+    if pending is None:
+        return None
+    same_norm = isinstance(pending, PendingGatedNorm) and pending.groups == groups and pending.eps == eps
+    if same_norm or (isinstance(pending, PendingSum) and not isinstance(pending, PendingProduct) and pending.ldo == x.shape[1]):
+        return pending
+    ctx.kernels.finish(pending)
+    return None
+
+
+def read_stream(x: torch.Tensor, ctx: StepContext, groups: int = 1, eps: float = 1e-6) -> torch.Tensor:
+    """The residual stream itself as a product's input, rounded to the compute dtype by a pass that also does what is unfinished about it."""
+    pending = take_foldable(x, ctx, groups, eps)
+    h = ctx.empty(x.shape[0], x.shape[1])
+    ctx.kernels.group_norm_step(x, groups=groups, eps=eps, h_out=h, pending=pending, plain_read=True)
+    return h
+
+
 @NORMS.register("group_rmsnorm")
 class GroupRmsNorm(Norm):
     """params: ``dim``, ``groups``, ``eps``, ``weight_offset`` (0; 1 for a weight that is stored as its distance from one); tensor
-    ``weight`` ``[dim]``. Folds a pending gated write of the same grouping into its pass."""
+    ``weight`` ``[dim]``. Folds a pending gated write of the same grouping, or a product's unfinished sum, into its pass."""
 
     graph_safe = True
     folds_pending = True
@@ -43,10 +64,7 @@ class GroupRmsNorm(Norm):
     def __call__(self, x: torch.Tensor, ctx: StepContext, rows: Optional[torch.Tensor] = None, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
         n = x.shape[0] if rows is None else rows.numel()
         out = ctx.empty(n, self.dim, out_dtype)
-        pending = ctx.take_pending(x)
-        if pending is not None and not (isinstance(pending, PendingGatedNorm) and pending.groups == self.groups and pending.eps == self.eps):
-            ctx.kernels.finish(pending)
-            pending = None
+        pending = take_foldable(x, ctx, self.groups, self.eps)
         ctx.kernels.group_norm_step(x, groups=self.groups, eps=self.eps, weight=self.weight, h_out=out, rows=rows, pending=pending)
         return out
 
@@ -193,20 +211,9 @@ class PostNormBlock(Block):
         if self.feed_forward is not None and self.connect2 is None:
             raise ValueError("block 'post_norm': a feed-forward needs connect2")
 
-    @staticmethod
-    def _read(connect, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
-        """The stream as a sublayer's input; the write that the sublayer before has left pending is done in the same pass."""
-        pending = ctx.take_pending(x)
-        if pending is not None and not (isinstance(pending, PendingGatedNorm) and pending.groups == connect.groups and pending.eps == connect.eps):
-            ctx.kernels.finish(pending)
-            pending = None
-        h = ctx.empty(x.shape[0], x.shape[1])
-        ctx.kernels.group_norm_step(x, groups=connect.groups, eps=connect.eps, h_out=h, pending=pending, plain_read=True)
-        return h
-
     def _sublayer(self, connect, run, x: torch.Tensor, ctx: StepContext) -> None:
         may_defer = ctx.may_defer
-        h = self._read(connect, x, ctx)
+        h = read_stream(x, ctx, connect.groups, connect.eps)  # the write that the sublayer before has left pending is done in the same pass
         y = torch.empty_like(x)
         ctx.may_defer = False  # a sublayer's result is complete before it is normed
         run(h, y)

@@ -78,21 +78,20 @@ class ParallelMixers(Mixer):
         reqs = tuple(r for r in (b.cache_requirement() for b in self.branches) if r is not None)
         return reqs[0] if len(reqs) == 1 else (Combined(reqs) if reqs else None)
 
-    def _normed_sum(self, h: torch.Tensor, y: torch.Tensor, ctx: StepContext, unit: CacheUnitView, writes_cache: bool) -> None:
-        """``y`` = the weighted sum of the branches' results, each through its norm."""
+    def _normed_sum(self, h: torch.Tensor, y: torch.Tensor, ctx: StepContext, unit: CacheUnitView, writes_cache: bool, residual: bool = False) -> None:
+        """``y`` = (``residual``: plus) the weighted sum of the branches' results, each through its norm."""
         a = ctx.empty(h.shape[0], sum(self.out_cols))
         self.attend(self.proj(h, ctx), ctx, unit, writes_cache, a, h=h)
         n_left = self.out_cols[0]
         left = self.outs[0](a[:, :n_left], ctx, out_dtype=torch.float32)
-        self.outs[1](a[:, n_left:], ctx, out=y)
-        ctx.kernels.norm_sum2(left, y, self.norm_weights[0], self.norm_weights[1], self.scales[0], self.scales[1], self.branch_norm_eps, y)
+        right = self.outs[1](a[:, n_left:], ctx, out=None if residual else y, out_dtype=torch.float32)
+        ctx.kernels.norm_sum2(left, right, self.norm_weights[0], self.norm_weights[1], self.scales[0], self.scales[1], self.branch_norm_eps, y,
+                              **({"accumulate": True} if residual else {}))
 
     def forward(self, h: torch.Tensor, x: torch.Tensor, ctx: StepContext, unit: CacheUnitView, writes_cache: bool) -> None:
         if self.branch_norm_eps is not None:
-            y = torch.empty_like(x)
-            self._normed_sum(h, y, ctx, unit, writes_cache)
             ctx.settle()
-            x.add_(y)
+            self._normed_sum(h, x, ctx, unit, writes_cache, residual=True)
             return
         a = ctx.empty(h.shape[0], self.out.n_in)
         self.attend(self.proj(h, ctx), ctx, unit, writes_cache, a, h=h)

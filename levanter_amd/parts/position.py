@@ -84,6 +84,7 @@ class RotaryPairs(PositionEncoding):
     cosine and sine alike; 1 by default). Angles are 32-bit."""
 
     graph_safe = True
+    layout = "pairs"
 
     def __init__(self, spec: PartSpec, tensors: Dict[str, torch.Tensor], env: BuildEnv):
         super().__init__(spec, tensors, env)
@@ -100,3 +101,25 @@ class RotaryPairs(PositionEncoding):
                 ctx.kernels.rotary_pairs(q, k, self.head_dim, self.freqs, ctx.attention.positions)
             else:
                 ctx.kernels.rotary_pairs(q, k, self.head_dim, self.freqs, ctx.attention.positions, magnitude=self.magnitude)
+
+
+@POSITION_ENCODINGS.register("rotary_half")
+class RotaryHalf(PositionEncoding):
+    """The same rotation in the "rotate half" layout: dimension i of every query and key head is paired with dimension i + dims/2,
+    i < dims/2; dimensions from ``dims`` on pass unchanged. params: ``head_dim`` (the size of a head as the mixer stores it), ``dims``,
+    ``base``, ``scaling`` (see ``rotary_frequencies``). Angles are 32-bit."""
+
+    graph_safe = True
+    layout = "half"
+
+    def __init__(self, spec: PartSpec, tensors: Dict[str, torch.Tensor], env: BuildEnv):
+        super().__init__(spec, tensors, env)
+        p = spec.params
+        self.head_dim, self.dims = int(p["head_dim"]), int(p["dims"])
+        if self.dims % 2 or not 0 <= self.dims <= self.head_dim:
+            raise ValueError(f"rotary_half: {self.dims} rotated dimensions must be even and fit a head of {self.head_dim}")
+        self.freqs = torch.tensor(rotary_frequencies(self.dims, p["base"], p.get("scaling")), dtype=torch.float64).to(torch.float32).to(env.device)
+
+    def rotate(self, q: torch.Tensor, k: torch.Tensor, ctx: StepContext) -> None:
+        for t in (q, k):
+            ctx.kernels.rotary_half(t, t.shape[1] // self.head_dim, self.head_dim, 0, self.freqs, ctx.attention.positions)

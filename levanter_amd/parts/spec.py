@@ -73,6 +73,8 @@ class PlanEntry:
     """Cache unit this entry's mixer reads. Entries with ``writes_cache`` own their unit."""
     writes_cache: bool = True
     """False: the mixer only reads the unit, which an earlier entry has written in this step."""
+    enters: Optional[Tuple[int, int]] = None
+    """(index into ``ModelSpec.stream_entries``, a number for it): what is done to the residual stream right before this entry."""
 
 
 @dataclass
@@ -97,6 +99,8 @@ class ModelSpec:
     """Checkpoint tensors that may be present as a second copy of a parameter (a stored tied head): name -> the tensor
     it must equal. A copy that differs is an error: the model would not compute what the file's author computed."""
     init_std: float = 0.02
+    stream_entries: List[PartSpec] = field(default_factory=list)
+    """Parts of the family "stream_mix" with ``begin`` and ``enter_run`` that plan entries name in ``enters``."""
 
     def all_tensors(self) -> Dict[str, TensorSpec]:
         out: Dict[str, TensorSpec] = {}
@@ -115,6 +119,8 @@ class ModelSpec:
         for layer in self.layers:
             for part in layer.parts.values():
                 add(part)
+        for part in self.stream_entries:
+            add(part)
         add(self.final_norm)
         add(self.head)
         return out

@@ -7,6 +7,7 @@
 * no value projection (``values_from_keys``): the keys as projected, before any norm, are the values;
 * a soft cap on the scaled score, then a term per head that grows with the distance, ``- slope[h] * (i - j)``;
 * a rotation of queries and keys by their positions before the keys are cached (``rotary``: a position encoding);
+* a sink per head: exp(sink_h) in the softmax's denominator, with no key and no value (the tensor ``sinks``);
 * a window of the last ``window`` keys whose first ``keep_first`` positions stay in sight whatever the window, and/or chunks: a query sees only the keys of its own ``chunk`` positions, counted
   from the start of the sequence;
 * the softmax weights mixed over the heads after the softmax, ``w'_h = sum_g talk[h, g] w_g``, each head applying its
@@ -48,7 +49,7 @@ class TalkingHeadsAttention(Mixer):
     ``rotate``, or None), ``out_scale`` (1 by default), ``qk_norm`` (None, "head" or "projection") with ``qk_norm_eps`` and the tensors
     ``q_norm.weight`` / ``k_norm.weight`` (``[head_dim]``, or the whole projection's size), ``keep_first`` (0), ``gate_kind`` ("head" or
     "element": ``gate.weight`` ``[heads * value_dim, dim]``), ``values_from_keys`` (False; True: no ``v.weight``). All tensors but the four matrices are optional. Tensors: ``q.weight``, ``k.weight``, ``v.weight``, ``out.weight`` (``[out, in]``), their
-    optional ``.bias``, optional ``gate.weight`` ``[heads, dim]``, ``talk`` ``[heads, heads]``, ``value_mix.weight`` (one number)."""
+    optional ``.bias``, optional ``gate.weight`` ``[heads, dim]``, ``talk`` ``[heads, heads]``, ``value_mix.weight`` (one number), ``sinks`` ``[heads]``."""
 
     graph_safe = True
 
@@ -97,6 +98,10 @@ class TalkingHeadsAttention(Mixer):
         self.blend = None
         if self.value_mix == "blend":
             self.blend = tensors["value_mix.weight"].to(env.device, torch.float32).reshape(1).contiguous()
+        sinks = tensors.get("sinks")
+        self.sinks = None if sinks is None else sinks.to(env.device, torch.float32).reshape(-1).contiguous()
+        if self.sinks is not None and self.sinks.numel() != self.n_heads:
+            raise ValueError(f"attention: {self.sinks.numel()} sinks for {self.n_heads} heads")
         talk = tensors.get("talk")
         self.talk = None if talk is None else talk.to(env.device, torch.float32).contiguous()
         if self.talk is not None and tuple(self.talk.shape) != (self.n_heads, self.n_heads):
@@ -188,13 +193,26 @@ class TalkingHeadsAttention(Mixer):
         single = writes_cache and ctx.attention.n_prefill_tiles == 0
         fused_rotation = {}
         fused_norm = {}
-        if self.qk_norm == "projection":  # one statistic over all heads of a token: a pass of its own, ahead of everything else
-            K.head_prepare(q, 1, self.q_cols, self.qk_norm_eps, norm_dim=self.n_heads * self.true_head_dim, norm_weight=self.q_norm_weight)
-            K.head_prepare(k, 1, self.k_cols, self.qk_norm_eps, norm_dim=self.n_kv_heads * self.true_head_dim, norm_weight=self.k_norm_weight)
-        elif self.qk_norm == "head":
+        rot_known = self.rotary is not None and getattr(self.rotary, "freqs", None) is not None and getattr(self.rotary, "head_dim", None) == self.head_dim
+        rot_here = rot_known and getattr(self.rotary, "layout", "pairs") == "pairs"
+        g = unit.group
+        written = False
+        if self.qk_norm == "projection":
+            # one statistic over all heads of a token; the rotation behind it and, for single tokens, the write into the pages are the same kernel
+            turns = rot_known and getattr(self.rotary, "magnitude", 1.0) == 1.0
+            rot = {"freqs": self.rotary.freqs, "positions": ctx.attention.positions, "half": self.rotary.layout == "half"} if turns else {}
+            written = single and self.value_mix is None and (turns or self.rotary is None)
+            pages = {"v": v, "value_dim": self.value_dim, "k_pages": unit.k_pages, "v_pages": unit.v_pages, "dest": g.dest, "page_size": g.page_size} if written else {}
+            K.projection_norm_rotate(q, k, self.n_heads, self.n_kv_heads, self.head_dim, self.qk_norm_eps, self.q_norm_weight, self.k_norm_weight,
+                                     q_norm_dim=self.n_heads * self.true_head_dim, k_norm_dim=self.n_kv_heads * self.true_head_dim, **rot, **pages)
+            if self.rotary is not None and not turns:
+                self.rotary.rotate(q, k, ctx)
+            rot_done = True
+        else:
+            rot_done = self.rotary is None
+        if self.qk_norm == "head":
             fused_norm = {"q_norm_weight": self.q_norm_weight, "k_norm_weight": self.k_norm_weight}
-        rot_here = self.rotary is not None and getattr(self.rotary, "freqs", None) is not None and getattr(self.rotary, "head_dim", None) == self.head_dim
-        if self.rotary is not None and rot_here and (single or fused_norm):
+        if not rot_done and rot_here and (single or fused_norm):
             # a step of single tokens: the rotation happens inside the kernel that writes the pages; with a weighted norm ahead of it,
             # a step with longer runs does both in one kernel of the same arithmetic (a norm with a weight does not commute with the rotation)
             fused_rotation = {"rotary_freqs": self.rotary.freqs, "positions": ctx.attention.positions} if self.rotary.freqs.numel() else {}
@@ -205,7 +223,7 @@ class TalkingHeadsAttention(Mixer):
             if self.rotary is not None and not rot_here:  # a rotation of another kind: behind the norm
                 self.rotary.rotate(q, k, ctx)
             fused_norm, fused_rotation = {}, {}  # both are done: what writes the pages only writes
-        elif self.rotary is not None and not (single and rot_here):
+        elif not rot_done and not (single and rot_here):
             self.rotary.rotate(q, k, ctx)
         v_first = None
         if self.value_mix == "source":
@@ -214,8 +232,9 @@ class TalkingHeadsAttention(Mixer):
             v_first = ctx.shared.get(self.value_mix_key)
             if v_first is None or v_first.shape != v.shape:
                 raise RuntimeError("attention: no layer before this one has left values of this shape to blend with")
-        g = unit.group
-        if single:
+        if written:
+            pass
+        elif single:
             # a step of single tokens: unit norms, the rotation, the blend and the write into the pages are one kernel
             K.head_prepare_write(q, k, v, unit.k_pages, unit.v_pages, g.dest, self.n_heads, self.n_kv_heads, self.head_dim, self.value_dim,
                                  g.page_size, self.qk_norm_eps if fused_norm else self.unit_norm_eps, v_first=v_first, blend=self.blend,
@@ -234,6 +253,6 @@ class TalkingHeadsAttention(Mixer):
                            head_dim=self.head_dim, value_dim=self.value_dim, all_value_heads=self.talk is not None,
                            page_size=g.page_size, scale=self.scale, window=self.window, block_tables=g.block_tables,
                            softcap=self.softcap, slopes=self.slopes, **({"chunk": self.chunk} if self.chunk else {}),
-                           **({"keep_first": self.keep_first} if self.keep_first else {}))
+                           **({"keep_first": self.keep_first} if self.keep_first else {}), **({} if self.sinks is None else {"sinks": self.sinks}))
         K.head_talk(w, self.talk, gate, a, self.n_heads, self.n_kv_heads, self.value_dim, **({"out_scale": self.out_scale} if self.out_scale != 1.0 else {}),
                     **({"gate_elements": True} if self.gate_elements and gate is not None else {}))

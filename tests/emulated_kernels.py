@@ -292,11 +292,67 @@ class EmulatedKernels:
             gt, up = gt.clamp(max=limit), up.clamp(-limit, limit)
         out.copy_((_act(activation)(gt) * (up + up_shift)).to(out.dtype))
 
-    def norm_sum2(self, a, b, weight_a, weight_b, scale_a, scale_b, eps, y) -> None:
+    # ---- a matrix state per head with one decay a token, behind a short convolution
+    def state_recurrence(self, rule, x, taps, conv_bias, a, b, a_bias, rate, skip, gate, norm_weight, state, token_slots, positions, out, *, n_heads, n_groups,
+                         key_dim, value_dim, q_offset, k_offset, v_offset, norm_groups, norm_eps, key_eps=0.0, q_scale=1.0, max_runs=None) -> None:
+        T, C = x.shape
+        H, G, dk, dv, K = n_heads, n_groups, key_dim, value_dim, taps.shape[1]
+        own = torch.arange(H) // (H // G)
+        for t in range(T):
+            slot, pos = int(token_slots[t]), int(positions[t])
+            if slot < 0:
+                out[t] = 0
+                continue
+            ring = state[slot, :K * C].view(K, C)
+            S = state[slot, K * C:K * C + H * dk * dv].view(H, dk, dv)
+            ring[pos % K] = x[t].float()
+            acc = torch.zeros(C) if conv_bias is None else conv_bias.clone()
+            for k in range(min(K, pos + 1)):
+                acc = acc + taps[:, K - 1 - k] * ring[(pos - k) % K]
+            u = F.silu(acc).to(x.dtype).float()
+            q, kk = (u[o:o + G * dk].view(G, dk) for o in (q_offset, k_offset))
+            v = u[v_offset:v_offset + H * dv].view(H, dv)
+            sp = F.softplus(a[t].float() + a_bias)
+            d = torch.exp(-rate * sp)
+            if rule == "ssd":
+                S.copy_(d[:, None, None] * S + (sp[:, None] * kk[own])[:, :, None] * v[:, None, :])
+                y = torch.einsum("hij,hi->hj", S, q[own]) + skip[:, None] * v
+                y = (y.reshape(-1) * F.silu(gate[t].float())).view(norm_groups, -1)
+                y = y / torch.sqrt((y * y).mean(-1, keepdim=True) + norm_eps)
+                out[t] = (y.reshape(-1) * norm_weight).to(out.dtype)
+            else:
+                q = q / torch.sqrt((q * q).sum(-1, keepdim=True) + key_eps) * q_scale
+                kk = kk / torch.sqrt((kk * kk).sum(-1, keepdim=True) + key_eps)
+                S.copy_(d[:, None, None] * S)
+                w = torch.sigmoid(b[t].float())[:, None] * (v - torch.einsum("hij,hi->hj", S, kk[own]))
+                S.copy_(S + kk[own][:, :, None] * w[:, None, :])
+                o = torch.einsum("hij,hi->hj", S, q[own])
+                o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + norm_eps)
+                out[t] = (o.reshape(-1) * norm_weight * F.silu(gate[t].float())).to(out.dtype)
+
+    def token_gate(self, z, tokens, table, out) -> None:
+        out.copy_((F.gelu(z.float(), approximate="tanh") * table[tokens.long()].float()).to(out.dtype))
+
+    def projection_norm_rotate(self, q, k, n_heads, n_kv_heads, head_dim, eps, q_weight, k_weight, q_norm_dim=None, k_norm_dim=None, freqs=None, positions=None,
+                               half=False, v=None, value_dim=0, k_pages=None, v_pages=None, dest=None, page_size=0) -> None:
+        kk = k.clone() if k_pages is not None else k
+        for t, n, w in ((q, q_norm_dim, q_weight), (kk, k_norm_dim, k_weight)):
+            self.head_prepare(t, 1, t.shape[1], eps, norm_dim=n, norm_weight=w)
+        if freqs is not None and freqs.numel():
+            if half:
+                self.rotary_half(q, n_heads, head_dim, 0, freqs, positions)
+                self.rotary_half(kk, n_kv_heads, head_dim, 0, freqs, positions)
+            else:
+                self.rotary_pairs(q, kk, head_dim, freqs, positions)
+        if k_pages is not None:
+            self.kv_write(kk, v, k_pages, v_pages, dest, n_kv_heads, head_dim, page_size, value_dim=value_dim)
+
+    def norm_sum2(self, a, b, weight_a, weight_b, scale_a, scale_b, eps, y, accumulate=False) -> None:
         def n(v, w):
             return v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * w
 
-        y.copy_(scale_a * n(a, weight_a) + scale_b * n(b, weight_b))
+        s = scale_a * n(a, weight_a) + scale_b * n(b, weight_b)
+        y.copy_(y + s if accumulate else s)
 
     # ---- mixture of experts
     def moe_route(self, z, correction, chosen, weights, *, n_groups=1, keep=1, group_top=2, renormalize=False, softmax=False) -> None:
