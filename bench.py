@@ -55,18 +55,20 @@ def main() -> int:
     ap.add_argument("--shape", default="7b", choices=["7b", "xl", "20b"],
                     help="layer sizes of the decode workload: 7b is the headline's; xl and 20b measure the same step at the other "
                          "sizes of the reference's configurations (use --no-points: the prefill point is 2,048 tokens)")
-    ap.add_argument("--workload", default="decode", choices=["decode", "xl_mix", "20b", "zederax", "nakurax", "tativik", "kegetar"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "xl_mix", "20b", "zederax", "nakurax", "tativik", "kegetar", "lelatar"],
                     help="decode: the workload described above. xl_mix / 20b: continuous-batching workloads at the gpt2_xl and gpt2_20b sizes "
                          "through InferenceEngine.generate; they print their own line. zederax: prefill and decode rates of Zederax "
                          "layers at a few sizes beside GPT-2 layers of the same width, heads and inner width; its own line. nakurax: the same for "
                          "Nakurax layers (latent attention and attention beside a recurrence, in turn) beside Zederax and GPT-2 layers. tativik: Tativik "
                          "layers (windowed latent attention with a rotated key part and a generalized delta rule, in turn, routed experts) beside Nakurax layers. "
                          "kegetar: Kegetar layers (windowed attention that keeps the first positions beside gated linear attention, and attention whose "
-                         "keys are its values, in turn; dense and routed feed-forwards in turn) beside Tativik layers")
+                         "keys are its values, in turn; dense and routed feed-forwards in turn) beside Tativik layers. lelatar: Lelatar layers (attention with sinks "
+                         "beside a gated delta rule with a dense feed-forward, and state-space duality, in turn, two layers looped, a token input a layer) beside "
+                         "Kegetar layers")
     ap.add_argument("--sizes", default="1k,2k,4k", help="with --workload zederax / nakurax: which of the sizes 1k, 2k, 4k to run")
     ap.add_argument("--batches", default="1,8,64", help="with --workload zederax: decode batch sizes to time ('' for none)")
     ap.add_argument("--no-prefill", action="store_true", help="with --workload zederax: skip the 2,048-token prompt")
-    ap.add_argument("--arch", default="both", choices=["both", "zederax", "gpt2", "nakurax", "tativik", "kegetar"],
+    ap.add_argument("--arch", default="both", choices=["both", "zederax", "gpt2", "nakurax", "tativik", "kegetar", "lelatar"],
                     help="with --workload zederax / nakurax: one architecture only (for profiling)")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -78,7 +80,7 @@ def main() -> int:
     from levanter_amd.config import InferenceEngineConfig, LmConfig
     from levanter_amd.engine import InferenceEngine, Request
 
-    if args.workload in ("zederax", "nakurax", "tativik", "kegetar"):
+    if args.workload in ("zederax", "nakurax", "tativik", "kegetar", "lelatar"):
         return zederax_workload(args)
     if args.workload != "decode":
         return serving_workload(args)
@@ -388,6 +390,25 @@ def kegetar_config(z):
             "embedding": {"bigram": {"buckets": 65521, "mul_prev": 1009, "mul_cur": 13}}, "layers": layers}
 
 
+def lelatar_config(z):
+    """Layers of a causal rotary attention with sinks beside a gated delta rule, with a dense gated feed-forward of two thirds of the size's
+    inner width (three matrices hold what the size's two hold), and layers of state-space duality (twice the width inside, heads of 64
+    over a state of 128, no feed-forward), in turn; the heads and head sizes of the size. Two layers in the middle run twice, so that the
+    layer runs are the size's layer count; every layer ends with a token input of a 16th of the width."""
+    import math
+
+    left = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["vdim"], "scale": 1.0 / math.sqrt(z["dim"]),
+            "rot": {"dims": z["dim"] // 2, "base": 500000.0}}
+    right = {"heads": z["heads"], "kv_heads": z["heads"] // 2, "dim": z["dim"], "vdim": z["vdim"], "conv": 4}
+    mamba = {"heads": z["width"] // 32, "vdim": 64, "state": 128, "groups": 4, "norm_groups": 4, "conv": 4}
+    n = z["layers"] - 2
+    layers = [{"type": "parallel", "mixer": json.loads(json.dumps({"left": left, "right": right})), "mlp": {"kind": "dense", "ff": z["ff"] * 2 // 3 // 256 * 256}}
+              if i % 2 == 0 else {"type": "mamba2", "mixer": dict(mamba), "mlp": None} for i in range(n)]
+    start = max(0, n // 2 - 1)
+    return {"architecture": "Lelatar", "vocab": ZEDERAX_VOCAB, "width": z["width"], "norm": {"eps": 1e-6}, "layers": layers,
+            "loop": {"start": start, "stop": start + 2, "times": 2}, "token_side": {"dim": z["width"] // 16}}
+
+
 def zederax_workload(args) -> int:
     """Prefill (one 2,048-token prompt) and decode (batch 1, 8, 64 after 512-token prompts) through the engine, for Zederax
     (or, with --workload nakurax, Nakurax and Zederax) and for GPT-2 at equal sizes. One JSON line."""
@@ -463,11 +484,14 @@ def zederax_workload(args) -> int:
             archs = [("tativik", tativik_config(z)), ("nakurax", nakurax_config(z))]
         if args.workload == "kegetar":  # beside the closest model: Tativik's windowed attention, matrix-state recurrence and experts
             archs = [("kegetar", kegetar_config(z)), ("tativik", tativik_config(z))]
+        if args.workload == "lelatar":  # beside the closest model: Kegetar's attention beside a recurrence with a matrix state, gated feed-forwards
+            archs = [("lelatar", lelatar_config(z)), ("kegetar", kegetar_config(z))]
         for arch, raw in archs:
             if args.arch in ("both", arch):
                 print(f"[bench] {arch} at size {name} ...", file=sys.stderr, flush=True)
                 results[name][arch] = measure(raw)
-    print(json.dumps({"metric": ("prefill and decode tok/s of Kegetar layers beside Tativik layers of equal width, heads and head sizes" if args.workload == "kegetar" else
+    print(json.dumps({"metric": ("prefill and decode tok/s of Lelatar layers beside Kegetar layers of equal width, heads and head sizes" if args.workload == "lelatar" else
+                                 "prefill and decode tok/s of Kegetar layers beside Tativik layers of equal width, heads and head sizes" if args.workload == "kegetar" else
                                  f"prefill and decode tok/s of Tativik layers beside Nakurax layers of equal width, heads and (per token) inner width" if args.workload == "tativik" else
                                  f"prefill and decode tok/s of {args.workload.capitalize()} layers beside {'Zederax and ' if args.workload == 'nakurax' else ''}GPT-2 layers of equal width, heads and inner width"),
                       "unit": "tok/s", "n_gpus": 1, "steps": steps, "warmup": warmup, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",

@@ -17,26 +17,9 @@
 // Steps of single tokens: one kernel per (token, head) does convolution, recurrence and (DELTA) norm and gate. A row of the ring of
 // inputs is written by the token of its position and read by the K - 1 tokens after it, so the workgroups of a token that share
 // channels need no order among them. Steps with runs: convolution; decays, step sizes, key norms and the ring (written by a
-// kernel behind the one that reads it); the recurrence; norm and gate.
-#include "common.h"
-
-#define SR_SSD 0
-#define SR_DELTA 1
-
-__device__ __forceinline__ float sr_softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
-__device__ __forceinline__ float sr_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
-__device__ __forceinline__ float sr_silu(float x) { return x / (1.0f + expf(-x)); }
-
-// sizes and places, the same for every kernel of the file
-struct SrShape {
-  int Tn, H, G, dk, dv, C, K;
-  int q_off, k_off, v_off;  // first channel of the queries, keys and values among the C
-  long x_stride;            // row stride of the convolution's inputs
-  long a_stride, b_stride;  // of the decay's and the write rate's sums
-  long gate_stride, o_stride;
-  long slot_stride;         // floats of a slot
-  float key_eps, q_scale, norm_eps;
-};
+// kernel behind the one that reads it); the recurrence (bfloat16: in chunks on the matrix cores, state_chunks.hip; float32, or without the
+// matrix cores: token by token); norm and gate.
+#include "state_recurrence.h"
 
 // ---- the convolution of a step with runs ----------------------------------------------------------------------------------
 // A thread takes SR_CT tokens of one channel; with K <= 4 their inputs and the three before them are held in registers.
@@ -126,42 +109,6 @@ sr_prepare_kernel(const T* __restrict__ x, const T* __restrict__ u, const T* __r
     }
     if (lane == 0) sc[2 * H + g] = r;
   }
-}
-
-// ---- the run-th run of a step: its first token, the token behind its last, its slot; false: there are fewer ------------------
-// A token starts a run if it has a slot and the token before it has another. Each thread counts the starts of its stretch of
-// tokens; the thread whose stretch holds the run-th one finds it. `tmp`: NT + 2 ints of LDS.
-template <int NT>
-__device__ __forceinline__ bool sr_find_run(int run, const int* __restrict__ token_slots, int Tn, int* tmp, int& t0, int& t_end, int& slot) {
-  const int tid = threadIdx.x;
-  const int per = (Tn + NT - 1) / NT, lo = min(Tn, tid * per), hi = min(Tn, lo + per);
-  int mine = 0;
-  for (int t = lo; t < hi; ++t) mine += (token_slots[t] >= 0 && (t == 0 || token_slots[t - 1] != token_slots[t])) ? 1 : 0;
-  tmp[tid] = mine;
-  if (tid == 0) tmp[NT] = -1, tmp[NT + 1] = Tn;
-  __syncthreads();
-  int before = 0;
-  for (int i = 0; i < tid; ++i) before += tmp[i];
-  if (run >= before && run < before + mine) {
-    int seen = before;
-    for (int t = lo; t < hi; ++t)
-      if (token_slots[t] >= 0 && (t == 0 || token_slots[t - 1] != token_slots[t])) {
-        if (seen == run) tmp[NT] = t;
-        ++seen;
-      }
-  }
-  __syncthreads();
-  t0 = tmp[NT];
-  if (t0 < 0) return false;  // the whole workgroup
-  slot = token_slots[t0];
-  for (int t = max(lo, t0 + 1); t < hi; ++t)
-    if (token_slots[t] != slot) {
-      atomicMin(&tmp[NT + 1], t);
-      break;
-    }
-  __syncthreads();
-  t_end = tmp[NT + 1];
-  return true;
 }
 
 // ---- the recurrence of a step with runs, token by token ------------------------------------------------------------------------
@@ -487,17 +434,24 @@ static int sr_tokens_launch(const T* x, const float* taps, const float* conv_bia
   return 0;
 }
 
+static long sr_pad4(long n) { return (n + 3) / 4 * 4; }  // parts of the scratch memory start at 16-byte boundaries
+
 template <typename T, int RULE>
 static int sr_runs_launch(const T* x, const float* taps, const float* conv_bias, const T* a, const T* b, const float* a_bias, const float* rate,
                           const float* skip, const T* gate, const float* norm_w, float* state, const int* token_slots, const int* positions,
-                          float* ws, T* out, int norm_groups, int max_runs, const SrShape& s, hipStream_t stream) {
+                          float* ws, T* out, int norm_groups, int max_runs, int use_mfma, const SrShape& s, hipStream_t stream) {
   float* o = ws;
-  float* scal = o + (size_t)s.Tn * s.H * s.dv;
-  T* u = reinterpret_cast<T*>(scal + (size_t)s.Tn * (2 * s.H + 2 * s.G));
+  float* scal = o + sr_pad4((long)s.Tn * s.H * s.dv);
+  T* u = reinterpret_cast<T*>(scal + sr_pad4((long)s.Tn * (2 * s.H + 2 * s.G)));
   sr_conv_kernel<T><<<dim3((s.Tn + SR_CT - 1) / SR_CT, (s.C + 255) / 256), 256, 0, stream>>>(x, taps, conv_bias, state, token_slots, positions, u, s);
   if (lev_check_launch("state recurrence (convolution)")) return -1;
   sr_prepare_kernel<T, RULE><<<s.Tn, 256, 0, stream>>>(x, u, a, b, a_bias, rate, state, token_slots, positions, scal, s);
   if (lev_check_launch("state recurrence (prepare)")) return -1;
+  if (sizeof(T) == 2 && use_mfma) {
+    if (sr_chunks_launch(RULE, (const bf16_t*)(const void*)u, scal, state, token_slots, o, max_runs, s, stream)) return -1;
+    sr_finish_launch<T, RULE>(o, u, skip, gate, norm_w, token_slots, out, norm_groups, s, stream);
+    return lev_check_launch("state recurrence (norm)");
+  }
   const dim3 walk(max_runs, s.H, (s.dv + SR_WC - 1) / SR_WC);
   if (s.dk <= 64) sr_walk_kernel<T, 64, RULE><<<walk, 256, 0, stream>>>(u, scal, state, token_slots, o, s);
   else if (s.dk <= 128) sr_walk_kernel<T, 128, RULE><<<walk, 256, 0, stream>>>(u, scal, state, token_slots, o, s);
@@ -509,8 +463,8 @@ static int sr_runs_launch(const T* x, const float* taps, const float* conv_bias,
 
 // scratch memory in bytes. Steps with runs: o [Tn][H][dv], the scalars, the convolution's output; steps of single tokens: o of the rule SSD
 extern "C" long lev_state_recurrence_workspace(int Tn, int H, int G, int dv, int C, int runs, int dtype) {
-  const long o = (long)Tn * H * dv * 4;
-  return runs ? o + (long)Tn * (2L * H + 2L * G) * 4 + (long)Tn * C * (dtype == LEV_F32 ? 4 : 2) : o;
+  const long o = sr_pad4((long)Tn * H * dv) * 4;
+  return runs ? o + sr_pad4((long)Tn * (2L * H + 2L * G)) * 4 + (long)Tn * C * (dtype == LEV_F32 ? 4 : 2) : o;
 }
 
 extern "C" int lev_state_recurrence(int rule, const void* x, long x_stride, const float* taps, const float* conv_bias, const void* a, long a_stride,
@@ -518,7 +472,7 @@ extern "C" int lev_state_recurrence(int rule, const void* x, long x_stride, cons
                                     long gate_stride, const float* norm_w, float* state, long slot_stride, const int* token_slots,
                                     const int* positions, void* out, long o_stride, float* workspace, int T, int max_runs, int H, int G, int dk,
                                     int dv, int C, int K, int q_off, int k_off, int v_off, int norm_groups, float norm_eps, float key_eps,
-                                    float q_scale, int dtype, hipStream_t stream) {
+                                    float q_scale, int use_mfma, int dtype, hipStream_t stream) {
   SrShape s{T, H, G, dk, dv, C, K, q_off, k_off, v_off, x_stride, a_stride, b_stride, gate_stride, o_stride, slot_stride, key_eps, q_scale, norm_eps};
   if (sr_check(s, rule, norm_groups, dtype)) return -1;
   LEV_REQUIRE(x && taps && a && a_bias && rate && gate && norm_w && state && token_slots && positions && out && workspace, "state recurrence: a tensor is missing");
@@ -527,7 +481,7 @@ extern "C" int lev_state_recurrence(int rule, const void* x, long x_stride, cons
   if (T == 0) return 0;
 #define SR_GO(TT, RULE)                                                                                                                              \
   (max_runs ? sr_runs_launch<TT, RULE>((const TT*)x, taps, conv_bias, (const TT*)a, (const TT*)b, a_bias, rate, skip, (const TT*)gate, norm_w, state,   \
-                                       token_slots, positions, workspace, (TT*)out, norm_groups, max_runs, s, stream)                                \
+                                       token_slots, positions, workspace, (TT*)out, norm_groups, max_runs, use_mfma, s, stream)                              \
             : sr_tokens_launch<TT, RULE>((const TT*)x, taps, conv_bias, (const TT*)a, (const TT*)b, a_bias, rate, skip, (const TT*)gate, norm_w, state, \
                                          token_slots, positions, workspace, (TT*)out, norm_groups, s, stream))
   if (dtype == LEV_F32) return rule == SR_SSD ? SR_GO(float, SR_SSD) : SR_GO(float, SR_DELTA);

@@ -272,7 +272,7 @@ _P, _I, _L, _F = ctypes.c_void_p, ctypes.c_int, ctypes.c_long, ctypes.c_float
 
 register_unit("core", ["errors.hip", "elementwise.hip", "layer_ops.hip", "gemm_simple.hip", "attention_simple.hip", "attention_values.hip",
                        "attention_common.hip", "stream_ops.hip", "rotary.hip", "block_linear.hip", "recurrent_ops.hip", "group_norm.hip", "delta_rule.hip",
-                       "moe_ops.hip", "linear_attention.hip", "state_recurrence.hip"], signatures={
+                       "moe_ops.hip", "linear_attention.hip", "state_recurrence.hip", "state_chunks.hip"], signatures={
     "lev_embed": [_P] * 5 + [_I, _I, _I, _F, _P],
     "lev_pair_embed_add": [_P] * 6 + [_I, _I, _I, _L, _L, _I, _P],
     "lev_streams_step": [_P, _I, _I, _I, _P, _P, _P, _P, _P, _P, _F, _P, _P, _P, _I, _I, _P, _I, _P, _P],
@@ -308,7 +308,7 @@ register_unit("core", ["errors.hip", "elementwise.hip", "layer_ops.hip", "gemm_s
     "lev_norm_sum2": [_P, _P, _P, _P, _F, _F, _F, _P, _I, _I, _I, _P],
     "lev_token_gate": [_P, _L, _P, _P, _P, _I, _I, _I, _P],
     "lev_projection_norm_rotate": [_P, _L, _I, _P, _L, _I, _I, _P, _L, _I, _F, _I, _I, _P, _P, _P, _I, _I, _P, _P, _P, _P, _I, _I, _I, _P],
-    "lev_state_recurrence": [_I, _P, _L, _P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _P, _P, _L, _P, _P, _P, _L, _P] + [_I] * 12 + [_F, _F, _F, _I, _P],
+    "lev_state_recurrence": [_I, _P, _L, _P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _P, _P, _L, _P, _P, _P, _L, _P] + [_I] * 12 + [_F, _F, _F, _I, _I, _P],
     "lev_state_recurrence_workspace": [_I] * 7,
     "lev_gla_tokens": [_P, _P, _L, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _I, _I, _I, _I, _F, _F, _F, _I, _I, _P],
     "lev_gla_scan": [_P, _P, _L, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _P, _I, _I, _I, _I, _I, _F, _F, _F, _I, _I, _P],
@@ -341,5 +341,5 @@ for _hd in MFMA_ATTENTION_HEAD_DIMS:
         "lev_attention_mfma": [_P, _L, _P, _L, _P, _P, _P, _P, _P, _I, _P, _I, _P, _I, _P, _P, _L, _P, _P] + [_I] * 5 + [_F, _I, _F, _P, _I, _P],
     })
 # key / value head sizes of the attention with separate sizes that are built ahead; any other pair is built at its first use
-for _hd, _vd in ((32, 16), (16, 32), (48, 32), (64, 64), (128, 64), (128, 128), (256, 256), (32, 32), (16, 16), (64, 48), (64, 32), (80, 64), (224, 192), (256, 224)):
+for _hd, _vd in ((32, 16), (16, 32), (48, 32), (64, 64), (128, 64), (128, 128), (256, 256), (32, 32), (16, 16), (64, 48), (64, 32), (80, 64), (224, 192), (256, 224), (128, 32)):
     attention_values_unit(_hd, _vd)

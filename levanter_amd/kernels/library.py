@@ -1025,7 +1025,7 @@ class HipKernels:
             _rows(b, "state recurrence: b") if b is not None else H, _ptr(a_bias), _ptr(rate), _ptr(skip), _ptr(gate), _rows(gate, "state recurrence: gate"),
             _ptr(norm_weight), _ptr(state), state.shape[1], _ptr(token_slots), _ptr(positions), _ptr(out), _rows(out, "state recurrence: out"), _ptr(ws), T,
             runs if T else 0, H, G, dk, dv, C, K, int(q_offset), int(k_offset), int(v_offset), int(norm_groups), float(norm_eps), float(key_eps), float(q_scale),
-            _DT[dt], self._s()))
+            int(self.use_mfma), _DT[dt], self._s()))
 
     # ---- row kernels of gated feed-forwards and of branches with norms of their own ---------------
     def glu_activate(self, z, out, activation: str, limit: float = 0.0, up_shift: float = 0.0) -> None:

@@ -5,14 +5,34 @@ Notation: x the residual stream ``[T, D]``, h a sublayer's input, positions coun
 """
 from __future__ import annotations
 
+import contextlib
 import math
-from typing import Dict, List, Optional, Tuple
+from typing import Callable, Dict, List, Optional, Tuple
 
 import torch
 
 F64 = torch.float64
 
 KEY_EPS = 1e-6  # inside the root of the unit norms of the delta rule's queries and keys
+
+_ROUND: Callable[[torch.Tensor], torch.Tensor] = lambda t: t
+
+
+@contextlib.contextmanager
+def rounded_products():
+    """Inside it every linear map's input and result (and the convolutions' results) are rounded to bfloat16: how far rounding alone moves
+    a model's logits."""
+    global _ROUND
+    was, _ROUND = _ROUND, lambda t: t.float().to(torch.bfloat16).double()
+    try:
+        yield
+    finally:
+        _ROUND = was
+
+
+def lin(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """w x for every row of x (weights are stored [out, in])."""
+    return _ROUND(_ROUND(x) @ w.T)
 
 
 # ---- norms and activations ----------------------------------------------------------------------------------------
@@ -69,14 +89,14 @@ def mamba2(h: torch.Tensor, W: Dict[str, torch.Tensor], p: str, m: dict, eps: fl
     T = h.shape[0]
     H, P, N, G = m["heads"], m["vdim"], m["state"], m["groups"]
     inner = H * P
-    z, xbc, dt = torch.split(h @ W[f"{p}.in"].T, [inner, inner + 2 * G * N, H], dim=1)
-    xbc = silu(causal_conv(xbc, W[f"{p}.conv"], W[f"{p}.conv.b"]))
+    z, xbc, dt = torch.split(lin(h, W[f"{p}.in"]), [inner, inner + 2 * G * N, H], dim=1)
+    xbc = _ROUND(silu(causal_conv(xbc, W[f"{p}.conv"], W[f"{p}.conv.b"])))
     x, B, C = torch.split(xbc, [inner, G * N, G * N], dim=1)
     dt = softplus(dt + W[f"{p}.dt_bias"])
     y, _ = ssd_scan(x.view(T, H, P), B.view(T, G, N), C.view(T, G, N), dt, torch.exp(W[f"{p}.A_log"]), W[f"{p}.D"])
     y = y.reshape(T, inner) * silu(z)
     y = rms_norm(y.view(T, m["norm_groups"], -1), None, eps).reshape(T, inner) * W[f"{p}.norm"]
-    return y @ W[f"{p}.o"].T
+    return lin(y, W[f"{p}.o"])
 
 
 # ---- attention ------------------------------------------------------------------------------------------------------
@@ -115,14 +135,14 @@ def sink_attention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, scale: flo
 def rotary_sink_attention(h: torch.Tensor, W: Dict[str, torch.Tensor], p: str, m: dict, eps: float) -> torch.Tensor:
     T = h.shape[0]
     H, G, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    q = rms_norm(h @ W[f"{p}.q"].T, W[f"{p}.q.norm"], eps).view(T, H, d)
-    k = rms_norm(h @ W[f"{p}.k"].T, W[f"{p}.k.norm"], eps).view(T, G, d)
-    v = (h @ W[f"{p}.v"].T).view(T, G, dv)
+    q = rms_norm(lin(h, W[f"{p}.q"]), W[f"{p}.q.norm"], eps).view(T, H, d)
+    k = rms_norm(lin(h, W[f"{p}.k"]), W[f"{p}.k.norm"], eps).view(T, G, d)
+    v = lin(h, W[f"{p}.v"]).view(T, G, dv)
     rot = m.get("rot") or {"dims": 0, "base": 1.0}
     pos = torch.arange(T)
     q, k = rotate_half(q, pos, rot["dims"], rot["base"]), rotate_half(k, pos, rot["dims"], rot["base"])
     o = sink_attention(q, k, v, m["scale"], W[f"{p}.sink"])
-    return o.reshape(T, H * dv) @ W[f"{p}.o"].T
+    return lin(o.reshape(T, H * dv), W[f"{p}.o"])
 
 
 # ---- gated delta rule -----------------------------------------------------------------------------------------------
@@ -151,13 +171,13 @@ def unit(x: torch.Tensor) -> torch.Tensor:
 def gated_delta_rule(h: torch.Tensor, W: Dict[str, torch.Tensor], p: str, m: dict, eps: float) -> torch.Tensor:
     T = h.shape[0]
     H, G, d, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    q, k, v = (silu(causal_conv(h @ W[f"{p}.{n}"].T, W[f"{p}.{n}.conv"])) for n in ("q", "k", "v"))
+    q, k, v = (_ROUND(silu(causal_conv(lin(h, W[f"{p}.{n}"]), W[f"{p}.{n}.conv"]))) for n in ("q", "k", "v"))
     q, k = unit(q.view(T, G, d)) * d ** -0.5, unit(k.view(T, G, d))
-    beta = torch.sigmoid(h @ W[f"{p}.b"].T)
-    g = torch.exp(-torch.exp(W[f"{p}.A_log"]) * softplus(h @ W[f"{p}.a"].T + W[f"{p}.dt_bias"]))
+    beta = torch.sigmoid(lin(h, W[f"{p}.b"]))
+    g = torch.exp(-torch.exp(W[f"{p}.A_log"]) * softplus(lin(h, W[f"{p}.a"]) + W[f"{p}.dt_bias"]))
     o, _ = delta_scan(q, k, v.view(T, H, dv), g, beta)
-    o = rms_norm(o, W[f"{p}.norm"], eps).reshape(T, H * dv) * silu(h @ W[f"{p}.g"].T)
-    return o @ W[f"{p}.o"].T
+    o = rms_norm(o, W[f"{p}.norm"], eps).reshape(T, H * dv) * silu(lin(h, W[f"{p}.g"]))
+    return lin(o, W[f"{p}.o"])
 
 
 def parallel_mixer(h: torch.Tensor, W: Dict[str, torch.Tensor], p: str, m: dict, eps: float) -> torch.Tensor:
@@ -169,20 +189,20 @@ def parallel_mixer(h: torch.Tensor, W: Dict[str, torch.Tensor], p: str, m: dict,
 
 # ---- feed-forward, token input, loop ----------------------------------------------------------------------------------
 def dense_feed_forward(h: torch.Tensor, W: Dict[str, torch.Tensor], p: str) -> torch.Tensor:
-    return (silu(h @ W[f"{p}.gate"].T) * (h @ W[f"{p}.up"].T)) @ W[f"{p}.down"].T
+    return lin(silu(lin(h, W[f"{p}.gate"])) * lin(h, W[f"{p}.up"]), W[f"{p}.down"])
 
 
 def token_input(x: torch.Tensor, tokens: List[int], W: Dict[str, torch.Tensor], layer: int, dim: int, eps: float) -> torch.Tensor:
     """What layer ``layer`` adds to the stream for each token: the layer's part of the token's row of a second table, gated by
     the stream, projected to the width and normed."""
     e = W["side.embed"][torch.tensor(tokens)][:, layer * dim:(layer + 1) * dim]
-    y = (gelu_tanh(x @ W[f"l{layer}.side.gate"].T) * e) @ W[f"l{layer}.side.proj"].T
+    y = lin(gelu_tanh(lin(x, W[f"l{layer}.side.gate"])) * e, W[f"l{layer}.side.proj"])
     return rms_norm(y, W[f"l{layer}.side.norm"], eps)
 
 
 def loop_entry(x: torch.Tensor, x0: torch.Tensor, W: Dict[str, torch.Tensor], run: int) -> torch.Tensor:
     """The stream as the loop's pass number ``run`` starts on it: a product of [x; x0] plus the pass's vector."""
-    return torch.cat([x, x0], 1) @ W["loop.in"].T + W["loop.step"][run]
+    return lin(torch.cat([x, x0], 1), W["loop.in"]) + W["loop.step"][run]
 
 
 def layer_order(cfg: dict) -> List[Tuple[int, Optional[int]]]:
@@ -217,7 +237,7 @@ def forward(tokens: List[int], weights: Dict[str, torch.Tensor], cfg: dict) -> T
         if side:
             x = x + token_input(x, tokens, weights, i, side["dim"], eps)
         streams.append(x.clone())
-    return one_plus_norm(x, weights["final.norm"], eps) @ weights["head"].T, streams
+    return lin(one_plus_norm(x, weights["final.norm"], eps), weights["head"]), streams
 
 
 def plain_logits(W: Dict[str, torch.Tensor], cfg: dict, tokens) -> torch.Tensor:

@@ -1,0 +1,574 @@
+"""Lelatar on the GPU: every kernel it brought against the plain function of its mechanism, whole models through ``bin/trace_run`` in every
+cutting, generation through the engine and the command line."""
+import math
+import os
+
+import pytest
+import torch
+
+import plain_lelatar as P
+import traces as TR
+from helpers import make_meta, random_block_tables
+from lelatar_configs import LEL
+
+pytestmark = pytest.mark.gpu
+
+DEV = "cuda:0"
+DTYPES = [torch.float32, torch.bfloat16]
+
+
+def K():
+    from levanter_amd.kernels import get_kernels
+
+    return get_kernels()
+
+
+def tol(dtype, f32=2e-5, bf16=2e-2):
+    return dict(rtol=f32, atol=f32) if dtype == torch.float32 else dict(rtol=bf16, atol=bf16)
+
+
+def bfn(x):
+    """Numbers that bfloat16 holds exactly, as float64."""
+    return x.to(torch.bfloat16).double()
+
+
+def dev(x, dtype=torch.float32):
+    return x.to(dtype).to(DEV)
+
+
+def ints(x):
+    return torch.tensor(x, dtype=torch.int32, device=DEV)
+
+
+# ---- the recurrences with a state per head ------------------------------------------------------------------------------------
+class Case:
+    """Sizes, constants and one or more sequences of inputs of ``state_recurrence``, with the plain results."""
+
+    def __init__(self, rule, H, G, dk, dv, taps, lengths, seed, dtype, norm_groups=1, rate_std=1.0, bias=True, eps=1e-5):
+        g = torch.Generator().manual_seed(seed)
+        self.rule, self.H, self.G, self.dk, self.dv, self.taps, self.dtype, self.eps = rule, H, G, dk, dv, taps, dtype, eps
+        self.norm_groups = norm_groups if rule == "ssd" else H
+        C = self.C = H * dv + 2 * G * dk
+        self.off = {"v": 0, "k": H * dv, "q": H * dv + G * dk} if rule == "ssd" else {"q": 0, "k": G * dk, "v": 2 * G * dk}
+        rn = lambda *shape, std=1.0, mean=0.0: bfn(torch.randn(*shape, generator=g) * std + mean)
+        self.w = rn(C, taps, std=0.7)
+        self.conv_bias = rn(C, std=0.2) if bias else None
+        self.a_bias, self.rate = rn(H, mean=-1.0), torch.exp(rn(H, std=rate_std))
+        self.skip = rn(H, mean=0.5) if rule == "ssd" else None
+        self.nw = rn(H * dv, mean=1.0, std=0.2)
+        self.seqs = []
+        for n in lengths:
+            # one product's output: [x | gap | gate | a | b], as the mixers lay it out
+            self.seqs.append({"x": rn(n, C), "gate": rn(n, H * dv), "a": rn(n, H), "b": rn(n, H)})
+        self.cols = {"x": 0, "gate": C + 3, "a": C + 3 + H * dv, "b": C + 3 + H * dv + H}
+
+    def rows(self, seq):
+        n = seq["x"].shape[0]
+        return dev(torch.cat([seq["x"], torch.zeros(n, 3).double(), seq["gate"], seq["a"], seq["b"]], 1), self.dtype)
+
+    def plain(self, seq, S=None, history=None):
+        """Output ``[n, H * dv]`` and last state, the convolution's output rounded to the compute dtype as the kernels do. ``history``: inputs of
+        the tokens before (their convolution reaches in)."""
+        H, G, dk, dv = self.H, self.G, self.dk, self.dv
+        n = seq["x"].shape[0]
+        x = seq["x"] if history is None else torch.cat([history, seq["x"]])
+        u = P.silu(P.causal_conv(x, self.w, self.conv_bias))[-n:]
+        if self.dtype == torch.bfloat16:
+            u = u.float().to(torch.bfloat16).double()
+        q, k = (u[:, self.off[i]:self.off[i] + G * dk].reshape(n, G, dk) for i in "qk")
+        v = u[:, self.off["v"]:self.off["v"] + H * dv].reshape(n, H, dv)
+        sp = P.softplus(seq["a"] + self.a_bias)
+        if self.rule == "ssd":
+            y, S = P.ssd_scan(v, k, q, sp, self.rate, self.skip, S)
+            y = (y.reshape(n, -1) * P.silu(seq["gate"])).view(n, self.norm_groups, -1)
+            return P.rms_norm(y, None, self.eps).reshape(n, -1) * self.nw, S
+        o, S = P.delta_scan(P.unit(q) * 0.3, P.unit(k), v, torch.exp(-self.rate * sp), torch.sigmoid(seq["b"]), S)
+        return P.rms_norm(o, None, self.eps).reshape(n, -1) * self.nw * P.silu(seq["gate"]), S
+
+    def state(self, slots):
+        return torch.zeros(slots, self.taps * self.C + self.H * self.dk * self.dv, device=DEV)
+
+    def matrices(self, state, slot):
+        return state[slot, self.taps * self.C:].view(self.H, self.dk, self.dv)
+
+    def run(self, rows, slots, positions, state, max_runs):
+        kern = K()
+        c, H = self.cols, self.H
+        out = torch.full((rows.shape[0], H * self.dv), float("nan"), dtype=self.dtype, device=DEV)
+        kern.state_recurrence(self.rule, rows[:, :self.C], dev(self.w), None if self.conv_bias is None else dev(self.conv_bias), rows[:, c["a"]:c["a"] + H],
+                              rows[:, c["b"]:c["b"] + H] if self.rule == "delta" else None, dev(self.a_bias), dev(self.rate),
+                              None if self.skip is None else dev(self.skip), rows[:, c["gate"]:c["gate"] + H * self.dv], dev(self.nw), state, ints(slots),
+                              ints(positions), out, n_heads=H, n_groups=self.G, key_dim=self.dk, value_dim=self.dv, q_offset=self.off["q"],
+                              k_offset=self.off["k"], v_offset=self.off["v"], norm_groups=self.norm_groups, norm_eps=self.eps, key_eps=P.KEY_EPS,
+                              q_scale=0.3, max_runs=max_runs)
+        return out.cpu().double()
+
+
+def check_rows(got, want, dtype, f32=2e-4, bf16=2e-2):
+    """Equal within the limit, relative to a row's size; one row in fifty may miss it tenfold: where a token's read-out nearly cancels, its
+    norm multiplies the rounding of the convolution's output."""
+    limit = f32 if dtype == torch.float32 else bf16
+    err = (got - want).abs().amax(-1) / want.abs().amax(-1).clamp(min=1.0)
+    assert torch.isfinite(got).all()
+    over = (err > limit).sum().item()
+    assert err.max().item() < 10 * limit and over <= max(1, got.shape[0] // 50), f"largest error {err.max().item():.2e}, {over} of {got.shape[0]} rows over {limit}"
+
+
+SIZES = [("ssd", 4, 2, 16, 8, 4, 2), ("ssd", 3, 1, 10, 20, 2, 1), ("ssd", 6, 6, 64, 64, 4, 3), ("ssd", 2, 1, 128, 64, 4, 1), ("ssd", 1, 1, 1, 1, 1, 1), ("ssd", 5, 1, 70, 24, 6, 5),
+         ("ssd", 1, 1, 200, 72, 3, 1), ("ssd", 2, 2, 256, 256, 4, 1), ("ssd", 8, 2, 33, 17, 3, 8),
+         ("delta", 4, 2, 16, 8, 4, 0), ("delta", 3, 3, 10, 20, 2, 0), ("delta", 6, 2, 64, 64, 4, 0), ("delta", 2, 1, 128, 128, 4, 0), ("delta", 1, 1, 1, 1, 1, 0),
+         ("delta", 5, 1, 70, 24, 6, 0), ("delta", 1, 1, 200, 72, 3, 0), ("delta", 2, 2, 256, 256, 4, 0), ("delta", 8, 2, 33, 17, 3, 0)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("rule,H,G,dk,dv,taps,ng", SIZES)
+def test_the_recurrence_carries_state_and_inputs_through_any_cutting(dtype, rule, H, G, dk, dv, taps, ng):
+    """Two requests whose tokens come in steps of every size beside each other and beside a token of nobody, steps of single tokens among
+    them; the states of other slots stay as they are."""
+    case = Case(rule, H, G, dk, dv, taps, (97, 80), H * 1000 + dk + dv, dtype, max(ng, 1), bias=dk % 2 == 0)
+    (a, b), (wa, Sa), (wb, Sb) = case.seqs, case.plain(case.seqs[0]), case.plain(case.seqs[1])
+    ra, rb = case.rows(a), case.rows(b)
+    state = case.state(5)
+    state[1] = 5.0
+    state[2, :taps * case.C] = 7.0  # inputs that the slot's last user has left: never read at positions before 0
+    state[0, :taps * case.C] = -7.0
+    got_a, got_b = [], []
+    ia = ib = 0
+    for na, nb in ((1, 1), (7, 2), (1, 0), (1, 1), (16, 9), (0, 1), (2, 1), (66, 64), (1, 1), (2, 0)):
+        rows = torch.cat([ra[ia:ia + na], ra[:1], rb[ib:ib + nb]])
+        slots, pos = [2] * na + [-1] + [0] * nb, list(range(ia, ia + na)) + [0] + list(range(ib, ib + nb))
+        out = case.run(rows, slots, pos, state, 3 if max(na, nb) > 1 else None)
+        got_a.append(out[:na]); got_b.append(out[na + 1:])
+        assert float(out[na].abs().max()) == 0.0
+        ia += na; ib += nb
+    assert (ia, ib) == (97, 80)
+    check_rows(torch.cat(got_a), wa, dtype)
+    check_rows(torch.cat(got_b), wb, dtype)
+    for slot, S in ((2, Sa), (0, Sb)):
+        err = (case.matrices(state, slot).cpu().double() - S).abs().max() / S.abs().max()
+        assert float(err) < (1e-4 if dtype == torch.float32 else 1e-2), float(err)
+    assert float((state[1] - 5.0).abs().max()) == 0.0 and float(state[3:].abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("dtype,mfma", [(torch.float32, True), (torch.bfloat16, True), (torch.bfloat16, False)])
+@pytest.mark.parametrize("rule,H,G,dk,dv,taps,ng", [s for s in SIZES if s[3] in (16, 64, 128, 70, 256)])
+def test_long_runs_from_states_that_are_not_zero(dtype, mfma, rule, H, G, dk, dv, taps, ng, monkeypatch):
+    """Three runs of unequal length in one step (one ends inside a chunk of 64 tokens, one at its edge, one is a single token), each from a
+    state and inputs of its own."""
+    monkeypatch.setattr(K(), "use_mfma", mfma)
+    lengths, before = (300, 128, 1), 9
+    case = Case(rule, H, G, dk, dv, taps, [n + before for n in lengths], dk + dv, dtype, max(ng, 1))
+    state = case.state(3)
+    g = torch.Generator().manual_seed(3)
+    want, rows, slots, pos, last = [], [], [], [], []
+    for i, (seq, n) in enumerate(zip(case.seqs, lengths)):
+        S0 = torch.randn(H, dk, dv, generator=g).double()
+        hist = seq["x"][:before]
+        ring = state[2 - i, :taps * case.C].view(taps, case.C)
+        for p in range(max(0, before - taps + 1), before):
+            ring[p % taps] = dev(seq["x"][p])
+        case.matrices(state, 2 - i).copy_(dev(S0))
+        w, S = case.plain({k: v[before:] for k, v in seq.items()}, S0.float().double(), hist)
+        want.append(w); last.append(S)
+        rows.append(case.rows(seq)[before:]); slots += [2 - i] * n; pos += list(range(before, before + n))
+    out = case.run(torch.cat(rows), slots, pos, state, 4)
+    check_rows(out, torch.cat(want), dtype, f32=3e-4)
+    for i, S in enumerate(last):
+        err = (case.matrices(state, 2 - i).cpu().double() - S).abs().max() / S.abs().max()
+        assert float(err) < (1e-4 if dtype == torch.float32 else 1e-2), float(err)
+
+
+@pytest.mark.parametrize("rule", ["ssd", "delta"])
+@pytest.mark.parametrize("mfma", [True, False])
+def test_a_fast_decay_inside_a_chunk_does_not_cost_the_digits_of_the_slow_ones_behind_it(rule, mfma, monkeypatch):
+    """Sums of step sizes whose logarithms of decay reach thousands at a few tokens and stay near zero at the others, in 16-bit inputs with
+    32-bit arithmetic: the state is exact to 32 bits' rounding (conv of one tap, so its output is the same on both sides)."""
+    monkeypatch.setattr(K(), "use_mfma", mfma)
+    case = Case(rule, 2, 1, 64, 32, 1, (200,), 5, torch.bfloat16)
+    seq = case.seqs[0]
+    case.rate = torch.tensor([30.0, 0.01], dtype=torch.float64)
+    case.a_bias[:] = 0.0
+    seq["a"][:] = -9.0
+    seq["a"][[20, 70, 71, 150]] = 120.0
+    want, S = case.plain(seq)
+    state = case.state(1)
+    out = case.run(case.rows(seq), [0] * 200, list(range(200)), state, 1)
+    check_rows(out, want, torch.bfloat16, bf16=1.5e-2)
+    S_got = case.matrices(state, 0).cpu().double()
+    for h in range(2):  # the convolution's output may round the other way at a tie: a few entries in a thousand
+        rel = (S_got[h] - S[h]).abs() / S[h].abs().max()
+        assert float(rel.median()) < 1e-5 and float(rel.max()) < 1e-2, (float(rel.median()), float(rel.max()))
+
+
+@pytest.mark.parametrize("rule", ["ssd", "delta"])
+def test_repeated_keys_with_full_write_rates_in_a_chunk(rule):
+    """The same key in every token and a write rate near one: the system that a chunk of the delta rule solves is as far from diagonal as
+    it gets; a state-space head piles its writes up."""
+    case = Case(rule, 2, 1, 64, 32, 2, (150,), 8, torch.bfloat16)
+    seq = case.seqs[0]
+    seq["x"][:, case.off["k"]:case.off["k"] + 64] = seq["x"][:1, case.off["k"]:case.off["k"] + 64]
+    seq["b"][:] = 12.0
+    seq["a"][:] = -6.0
+    want, S = case.plain(seq)
+    state = case.state(1)
+    out = case.run(case.rows(seq), [0] * 150, list(range(150)), state, 1)
+    check_rows(out, want, torch.bfloat16)
+    assert float((case.matrices(state, 0).cpu().double() - S).abs().max() / S.abs().max()) < 1e-2
+
+
+@pytest.mark.parametrize("rule", ["ssd", "delta"])
+def test_a_far_write_is_still_there_hundreds_of_tokens_later(rule):
+    """One token writes a value far from all others along a key that only the last token asks for; a decay near one keeps it."""
+    for dtype in DTYPES:
+        for single in (True, False):
+            n = 500
+            g = torch.Generator().manual_seed(4)
+            case = Case(rule, 2, 1, 64, 32, 1, (n,), 21, dtype, bias=False)
+            seq = case.seqs[0]
+            case.rate[:] = 1e-4
+            case.w[:] = 1.0
+            seq["b"][:] = 3.0
+            ko, qo, vo = case.off["k"], case.off["q"], case.off["v"]
+            for o in (ko, qo):
+                seq["x"][:, o:o + 64] = -8.0  # silu leaves next to nothing
+                seq["x"][:, o + 8:o + 64] = seq["x"][:, o + 8:o + 64].abs() * bfn(torch.rand(n, 56, generator=g))
+            seq["x"][13, ko:ko + 64], seq["x"][n - 1, qo:qo + 64] = -8.0, -8.0
+            seq["x"][13, ko + 3], seq["x"][n - 1, qo + 3] = 6.0, 6.0
+            seq["x"][13, vo:vo + 64] = 40.0
+            want, S = case.plain(seq)
+            state = case.state(1)
+            rows = case.rows(seq)
+            cut = n - 1 if single else n - 30
+            case.run(rows[:cut], [0] * cut, list(range(cut)), state, 1)
+            out = case.run(rows[cut:], [0] * (n - cut), list(range(cut, n)), state, None if single else 1)
+            check_rows(out, want[cut:], dtype)
+            assert float(S[:, 3].abs().min()) > 10 and float(case.matrices(state, 0)[:, 3].abs().min()) > 10
+
+
+@pytest.mark.parametrize("rule", ["ssd", "delta"])
+def test_long_decoding_keeps_its_digits(rule):
+    """400 single tokens in 32-bit, with a decay within 1e-4 of one in one head and one that forgets at once in the other."""
+    case = Case(rule, 2, 2, 16, 8, 4, (400,), 3, torch.float32)
+    case.rate = torch.tensor([1e-4, 60.0], dtype=torch.float64)
+    seq = case.seqs[0]
+    want, S = case.plain(seq)
+    state = case.state(1)
+    rows = case.rows(seq)
+    out = torch.cat([case.run(rows[t:t + 1], [0], [t], state, None) for t in range(400)])
+    check_rows(out, want, torch.float32, f32=3e-4)
+    torch.testing.assert_close(case.matrices(state, 0).cpu().double(), S, rtol=1e-3, atol=1e-4)
+
+
+# ---- row kernels ----------------------------------------------------------------------------------------------------------------
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,hd,true,vd,n_pairs,half", [(4, 2, 16, 16, 8, 4, True), (2, 2, 32, 32, 32, 16, True), (6, 1, 64, 64, 16, 10, True), (3, 3, 16, 12, 24, 3, True),
+                                                          (1, 1, 8, 8, 8, 0, True), (2, 1, 128, 128, 64, 64, True), (4, 2, 16, 16, 16, 8, False), (2, 1, 160, 160, 16, 1, True)])
+def test_norm_over_the_projection_rotation_and_write_in_one_kernel(dtype, H, G, hd, true, vd, n_pairs, half):
+    """Against the plain norm and rotation; a key is the same bits whether it goes into the pages at once (single tokens) or by way of
+    kv_write (runs); heads that carry zeros behind their true size keep them."""
+    g = torch.Generator().manual_seed(hd + vd + H)
+    T, ps = 6, 16
+    eps = 1e-5
+    q, k = (bfn(torch.randn(T, n, hd, generator=g) * 2) for n in (H, G))
+    wq, wk = 1.5 + torch.randn(H, hd, generator=g).double() * 0.3, 1.5 + torch.randn(G, hd, generator=g).double() * 0.3
+    for t in (q, k):
+        t[:, :, true:] = 0.0
+    v = torch.randn(T, G * vd, generator=g).to(dtype).to(DEV)
+    base = 700.0
+    freqs = torch.tensor([base ** (-i / max(n_pairs, 1)) for i in range(n_pairs)], dtype=torch.float64)
+    pos = [3, 0, 700, 15, 16, 4000]
+    dest = ints([5, 17, 33, 40, 3 * ps + 15, 0])
+
+    def plain(x, w, heads):
+        y = P.rms_norm(x[:, :, :true].reshape(T, -1), w[:, :true].reshape(-1), eps).view(T, heads, true)
+        if half:
+            return P.rotate_half(y, torch.tensor(pos), 2 * n_pairs, base)
+        out = y.clone()
+        a = torch.tensor(pos, dtype=torch.float64)[:, None] * freqs[None, :]
+        c, s = torch.cos(a)[:, None, :], torch.sin(a)[:, None, :]
+        u, z = y[..., 0:2 * n_pairs:2], y[..., 1:2 * n_pairs:2]
+        out[..., 0:2 * n_pairs:2], out[..., 1:2 * n_pairs:2] = u * c - z * s, z * c + u * s
+        return out
+
+    args = dict(q_norm_dim=H * true, k_norm_dim=G * true, half=half, **({"freqs": dev(freqs), "positions": ints(pos)} if n_pairs else {}))
+    q1, k1 = dev(q.reshape(T, -1), dtype), dev(k.reshape(T, -1), dtype)
+    K().projection_norm_rotate(q1, k1, H, G, hd, eps, dev(wq.reshape(-1)), dev(wk.reshape(-1)), **args)
+    t = dict(rtol=2e-3, atol=2e-3) if dtype == torch.float32 else dict(rtol=2e-2, atol=2e-2)  # angles are 32-bit: at position 4,000 known to 4000 * 2^-24
+    torch.testing.assert_close(q1.cpu().double().view(T, H, hd)[:, :, :true], plain(q, wq, H), **t)
+    torch.testing.assert_close(k1.cpu().double().view(T, G, hd)[:, :, :true], plain(k, wk, G), **t)
+    assert float(q1.view(T, H, hd)[:, :, true:].abs().sum()) == 0.0
+    kp1, vp1 = torch.zeros(4, G * hd * ps, dtype=dtype, device=DEV), torch.zeros(4, G * vd * ps, dtype=dtype, device=DEV)
+    kp2, vp2 = torch.zeros_like(kp1), torch.zeros_like(vp1)
+    K().kv_write(k1, v, kp1, vp1, dest, G, hd, ps, value_dim=vd)
+    q2, k2 = dev(q.reshape(T, -1), dtype), dev(k.reshape(T, -1), dtype)
+    K().projection_norm_rotate(q2, k2, H, G, hd, eps, dev(wq.reshape(-1)), dev(wk.reshape(-1)), v=v, value_dim=vd, k_pages=kp2, v_pages=vp2, dest=dest, page_size=ps, **args)
+    assert torch.equal(q1.cpu(), q2.cpu()) and torch.equal(kp1.cpu(), kp2.cpu()) and torch.equal(vp1.cpu(), vp2.cpu())
+    assert torch.equal(k2.cpu(), dev(k.reshape(T, -1), dtype).cpu())  # with pages the projection stays as it is
+    gone = ints([-1] * T)  # tokens that are written nowhere
+    before = kp2.clone()
+    K().projection_norm_rotate(q2, k2, H, G, hd, eps, dev(wq.reshape(-1)), dev(wk.reshape(-1)), v=v, value_dim=vd, k_pages=kp2, v_pages=vp2, dest=gone, page_size=ps, **args)
+    assert torch.equal(before, kp2)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,D", [(5, 16), (1, 8), (300, 256)])
+def test_the_token_tables_gate(dtype, T, D):
+    g = torch.Generator().manual_seed(T)
+    z, table = torch.randn(T, D + 3, generator=g) * 2, bfn(torch.randn(40, D, generator=g))
+    tokens = torch.randint(0, 40, (T,), generator=g)
+    out = torch.empty(T, D, dtype=dtype, device=DEV)
+    K().token_gate(dev(z)[:, :D], ints(tokens.tolist()), dev(table, dtype), out)
+    torch.testing.assert_close(out.cpu().double(), P.gelu_tanh(z[:, :D].double()) * table[tokens], **tol(dtype, f32=1e-5, bf16=1e-2))
+
+
+@pytest.mark.parametrize("T,D", [(5, 64), (3, 1000), (1, 7)])
+def test_the_sum_of_two_normed_branches_is_added_to_the_stream(T, D):
+    g = torch.Generator().manual_seed(D)
+    a, b, x = (torch.randn(T, D, generator=g).double() * s for s in (4.0, 0.01, 1.0))
+    wa, wb = 1 + torch.randn(D, generator=g).double() * 0.2, 1 + torch.randn(D, generator=g).double() * 0.2
+    y = dev(x)
+    K().norm_sum2(dev(a), dev(b), dev(wa), dev(wb), 0.5, 0.25, 1e-6, y, accumulate=True)
+    torch.testing.assert_close(y.cpu().double(), x + 0.5 * P.rms_norm(a, wa, 1e-6) + 0.25 * P.rms_norm(b, wb, 1e-6), rtol=2e-5, atol=2e-5)
+
+
+@pytest.mark.parametrize("M,N,Kd", [(3, 512, 4096), (1, 2048, 4096), (40, 264, 1024)])
+@pytest.mark.parametrize("plain_read", [True, False])
+def test_the_streams_pass_adds_up_a_product_that_has_left_its_ranges(M, N, Kd, plain_read):
+    """Bit for bit the kernel that finishes the product, then the pass."""
+    g = torch.Generator().manual_seed(N)
+    a, w, bias = dev(torch.randn(M, Kd, generator=g), torch.bfloat16), dev(torch.randn(N, Kd, generator=g) / math.sqrt(Kd), torch.bfloat16), dev(torch.randn(N, generator=g))
+    x0 = torch.randn(M, N, generator=g)
+    nw = None if plain_read else dev(1 + 0.1 * torch.randn(N, generator=g))
+    outs = []
+    for fold in (True, False):
+        x, h = dev(x0), torch.empty(M, N, dtype=torch.bfloat16, device=DEV)
+        pending = K().linear(a, w, bias, x, residual=x, may_leave_pending=True)
+        if pending is None:
+            pytest.skip("this shape's product does not split its sum")
+        if not fold:
+            K().finish(pending)
+            pending = None
+        K().group_norm_step(x, groups=1, eps=1e-5, weight=nw, h_out=h, pending=pending, plain_read=plain_read)
+        outs.append((x.cpu(), h.cpu()))
+    torch.testing.assert_close(outs[0][0], outs[1][0], rtol=1e-6, atol=1e-6)
+    torch.testing.assert_close(outs[0][1].float(), outs[1][1].float(), rtol=1e-2, atol=1e-2)
+    # only the selected rows, and the stream is not stored
+    x, h = dev(x0), torch.empty(2, N, dtype=torch.bfloat16, device=DEV)
+    pending = K().linear(a, w, bias, x, residual=x, may_leave_pending=True)
+    K().group_norm_step(x, groups=1, eps=1e-5, weight=nw, h_out=h, pending=pending, plain_read=plain_read, rows=ints([M - 1, M - 1]))
+    assert torch.equal(h.cpu()[0], outs[0][1][M - 1]) and torch.equal(h.cpu()[1], h.cpu()[0]) and torch.equal(x.cpu(), x0)
+
+
+# ---- attention with a sink over shuffled pages -------------------------------------------------------------------------------------
+def run_attention(dtype, H, G, dk, dv, runs, scale, q, k, v, sinks, ps=16, seed=0):
+    """Keys and values of every request in shuffled pages that hold NaN where nothing was written."""
+    kern = K()
+    kv_lens = [kv for _, kv in runs]
+    n_pages = sum((n + ps - 1) // ps for n in kv_lens) + 3
+    bt = random_block_tables(kv_lens, ps, n_pages, seed, DEV)
+    k_pages = torch.full((n_pages, G * dk * ps), float("nan"), dtype=dtype, device=DEV)
+    v_pages = torch.full((n_pages, G * dv * ps), float("nan"), dtype=dtype, device=DEV)
+    for i, n in enumerate(kv_lens):
+        dest = ints([int(bt[i, p // ps]) * ps + p % ps for p in range(n)])
+        kern.kv_write(dev(k[i].reshape(n, -1), dtype), dev(v[i].reshape(n, -1), dtype), k_pages, v_pages, dest, G, dk, ps, value_dim=dv)
+    meta = make_meta(runs, DEV)
+    qq = dev(torch.cat([x.reshape(x.shape[0], -1) for x in q]), dtype)
+    o = torch.empty(qq.shape[0], H, 1, dv, dtype=torch.float32, device=DEV)
+    kern.attention_values(qq, o, k_pages, v_pages, meta, n_heads=H, n_kv_heads=G, head_dim=dk, value_dim=dv, all_value_heads=False, page_size=ps, scale=scale,
+                          window=None, block_tables=bt, sinks=dev(sinks))
+    return o.view(qq.shape[0], H, dv).cpu().double()
+
+
+def plain_attention(H, G, dk, dv, runs, scale, q, k, v, sinks):
+    outs = []
+    for i, (q_len, kv_len) in enumerate(runs):
+        full_q = torch.zeros(kv_len, H, dk, dtype=torch.float64)
+        full_q[kv_len - q_len:] = q[i]
+        outs.append(P.sink_attention(full_q, k[i], v[i], scale, sinks)[kv_len - q_len:])
+    return torch.cat(outs)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,dk,dv", [(4, 2, 32, 16), (6, 3, 64, 64), (3, 3, 48, 32), (6, 1, 24, 16), (2, 1, 128, 64), (34, 2, 32, 32)])
+def test_attention_with_sinks_prompts_portions_and_single_tokens(dtype, H, G, dk, dv):
+    g = torch.Generator().manual_seed(H * 100 + dk)
+    runs = [(70, 70), (1, 130), (19, 83), (1, 1), (2, 2), (1, 17), (130, 261), (1, 48), (1, 241), (5, 245), (1, 500), (64, 320)]  # (queries, keys after the step)
+    q, k, v = ([bfn(torch.randn(r[i], n, d, generator=g)) for r in runs] for i, n, d in ((0, H, dk), (1, G, dk), (1, G, dv)))
+    sinks = torch.randn(H, generator=g).double() * 2 + 1
+    sinks[0] = 30.0  # takes nearly all the weight
+    args = (H, G, dk, dv, runs, 2.0 / math.sqrt(dk), q, k, v, sinks)
+    got, want = run_attention(dtype, *args, seed=dk), plain_attention(*args)
+    torch.testing.assert_close(got, want, **tol(dtype, f32=3e-5, bf16=3e-2))
+    assert float(want[:, 0].abs().max()) < 1e-3 and (plain_attention(*args[:-1], torch.full((H,), -40.0, dtype=torch.float64)) - want).abs().max() > 0.3
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("single", [True, False])
+@pytest.mark.parametrize("ps", [16, 64])
+def test_a_far_key_among_hundreds_at_page_borders(dtype, single, ps):
+    """A key whose score stands out against the sink and all other keys, at the first and last places of pages and of the sequence."""
+    H, G, dk, dv, n = 4, 2, 64, 32, 900
+    g = torch.Generator().manual_seed(5)
+    sinks = torch.full((H,), 10.0, dtype=torch.float64)
+    for j in (0, 1, ps - 1, ps, 13 * ps - 1, 512, n - 2, n - 1):
+        kk, qq, vv = bfn(torch.randn(n, G, dk, generator=g) * 0.05), bfn(torch.randn(n, H, dk, generator=g)), bfn(torch.randn(n, G, dv, generator=g) * 0.1)
+        kk[j, 0] = qq[n - 1, 1]
+        vv[j, 0] = 100.0
+        ql = 1 if single else 200
+        args = (H, G, dk, dv, [(ql, n)], 1.0, [qq[n - ql:]], [kk], [vv], sinks)
+        got = run_attention(dtype, *args, ps=ps, seed=j)
+        torch.testing.assert_close(got, plain_attention(*args), **tol(dtype, f32=3e-5, bf16=3e-2))
+        assert bool((got[-1, 1] > 90).all()) and bool((got[-1, 2:].abs() < 5).all()), f"key {j}"  # heads 2 and 3 read the other key/value head
+
+
+# ---- whole models -----------------------------------------------------------------------------------------------------------------
+# a model of middle sizes for the GPU alone: heads of 64 and 128, a state of 128, several chunks of 64 tokens a prompt
+MIDDLE = (P.make_config(vocab=1000, width=256, eps=1e-6, side=32, loop=(1, 3, 2), layers=[
+    P.parallel_layer(left=P.left_sizes(heads=8, kv_heads=2, dim=64, vdim=64, rot_dims=32, base=500000.0),
+                     right=P.right_sizes(heads=4, kv_heads=2, dim=128, vdim=64, conv=4), ff=384),
+    P.mamba_layer(heads=8, vdim=64, state=128, groups=2, norm_groups=4, conv=4),
+    P.parallel_layer(left=P.left_sizes(heads=4, kv_heads=4, dim=128, vdim=32, rot_dims=128), right=P.right_sizes(heads=4, kv_heads=1, dim=64, vdim=128, conv=2), ff=None),
+    P.mamba_layer(heads=6, vdim=32, state=64, groups=3, norm_groups=1, conv=3, ff=200),
+]), 31)
+
+
+def model_folder(name, tmp, store):
+    raw, seed = MIDDLE if name == "middle" else LEL[name]
+    W = P.random_weights(raw, seed)
+    return raw, W, P.write_folder(raw, W, os.path.join(str(tmp), name), store)
+
+
+def row_error(got, want):
+    """Difference of two rows of logits, mean taken off, relative to the spread of the wanted row."""
+    d = got - want
+    d = d - d.mean(-1, keepdim=True)
+    return (d.pow(2).mean(-1).sqrt() / want.std(-1)).max().item()
+
+
+LENGTHS = {"A": [70, 45, 100, 37, 64, 33], "B": [90, 130, 41, 200, 64, 17], "C": [40, 12, 150, 3], "D": [33, 50, 21, 64, 80], "middle": [520, 340, 45]}
+
+
+@pytest.mark.parametrize("name", list(LEL) + ["middle"])
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_trace_run_all_cuttings(name, dtype, tmp_path):
+    """Whole prompts, the last 32 tokens one by one, portions down to two tokens, and twice mixed with other requests in a pool of exactly
+    the peak need (pages and slots are used again), through ``bin/trace_run``."""
+    from test_gpu_replay import read_step, run_trace
+
+    raw, W, d = model_folder(name, tmp_path, torch.float32 if dtype == "float32" else torch.bfloat16)
+    reqs = TR.random_requests(raw["vocab"], LENGTHS[name], 21)
+    plain = {rid: P.plain_logits(W, raw, t) for rid, t in reqs.items()}
+    steps = TR.number(TR.trace_whole(reqs) + TR.trace_prefill_then_singles(reqs) + TR.trace_portions(reqs)
+                      + TR.trace_mixed(reqs, seed=3) + TR.trace_mixed(reqs, seed=4, prefix="n"))
+    out = run_trace(d, dtype, steps, TR.peak_tokens(steps), extra=("--max-seqs", "4"))
+    want = TR.expected_rows(steps, lambda rid: plain[rid[1:]])
+    if dtype == "float32":
+        limit_of = {rid: torch.full((len(t), 1), 2e-4) for rid, t in reqs.items()}
+    else:  # three times what rounding the products' inputs and results alone does at the position (at least what it does at one in ten)
+        limit_of = {}
+        for rid, t in reqs.items():
+            with P.rounded_products():
+                rounded = P.plain_logits(W, raw, t)
+            err = torch.tensor([row_error(rounded[i:i + 1], plain[rid][i:i + 1]) for i in range(len(t))])
+            limit_of[rid] = (3 * err.clamp(min=float(err.quantile(0.9)))).view(-1, 1)
+    limits = TR.expected_rows(steps, lambda rid: limit_of[rid[1:]])
+    worst, rows, over = 0.0, 0, []
+    for s in steps:
+        k = s["step"]
+        assert (k in want) == os.path.exists(os.path.join(out, f"{k}.f32"))
+        if k not in want:
+            continue
+        got = read_step(out, k, raw["vocab"]).double()
+        for r in range(got.shape[0]):
+            err = row_error(got[r:r + 1], want[k][r:r + 1])
+            rows += 1
+            if err >= float(limits[k][r]):
+                over.append(f"step {k} row {r}: {err}")
+            else:
+                worst = max(worst, err)
+    print(f"lelatar {name} {dtype}: worst relative row error {worst:.3e} over {rows} rows, {len(over)} over the limit")
+    # a first token whose query and key nearly cancel makes the delta rule's head norm divide a number of the size of sqrt(eps) by itself, and
+    # another rounding then gives another result: one row in a hundred may miss the limit there
+    assert rows >= 100 and len(over) <= rows // 100, over[:10]
+
+
+def _engine(d, dtype, **kw):
+    from levanter_amd.config import InferenceEngineConfig
+    from levanter_amd.engine import InferenceEngine
+
+    cfg = InferenceEngineConfig(**{**dict(max_seqs=4, page_size=16, max_pages_per_seq=32, compute_dtype=dtype), **kw})
+    return InferenceEngine.from_pretrained(d, cfg)
+
+
+def check_greedy(W, raw, prompt, generated, margin):
+    logits = P.plain_logits(W, raw, list(prompt) + list(generated))
+    clear = 0
+    for i, tok in enumerate(generated):
+        row = logits[len(prompt) - 1 + i]
+        top = row.topk(2).values
+        if float(top[0] - top[1]) > margin:
+            clear += 1
+            assert int(row.argmax()) == tok, f"generated token {i}"
+    return clear
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_greedy_generation_through_the_entry_point(dtype, tmp_path):
+    from levanter_amd.engine import Request
+
+    raw, W, d = model_folder("A", tmp_path, torch.float32 if dtype == "float32" else torch.bfloat16)
+    g = torch.Generator().manual_seed(0)
+    prompts = [torch.randint(0, raw["vocab"], (n,), generator=g).tolist() for n in (5, 17, 33, 1)]
+    engine = _engine(d, dtype)
+    res = engine.generate([Request(prompt_tokens=p, request_id=i, max_new_tokens=20) for i, p in enumerate(prompts)])
+    assert [len(t) for t in res.tokens] == [20] * 4 and res.finish_reasons == ["length"] * 4
+    margin = 1e-3 if dtype == "float32" else 0.25
+    clear = sum(check_greedy(W, raw, p, out, margin) for p, out in zip(prompts, res.tokens))
+    print(f"greedy {dtype}: {clear} of 80 positions decided by more than {margin}")
+    assert clear >= (76 if dtype == "float32" else 30)
+    engine.cache.check_invariants()
+    assert engine.cache.n_free_slots == 4
+
+
+@pytest.mark.parametrize("name", ["A", "D"])
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_long_decoding_in_replayed_steps(name, dtype, tmp_path):
+    """One prompt token, then 300 decoded ones: both recurrences run 300 steps from their slots, every pass of the loop from its own, and from
+    the third step on the steps are replayed from a graph ("D": a model without any attention, so without pages). Then the first tokens of
+    sequences of one, two and three tokens in one batch, in slots that were used before."""
+    from levanter_amd.engine import Request
+
+    raw, W, d = model_folder(name, tmp_path, torch.float32 if dtype == "float32" else torch.bfloat16)
+    engine = _engine(d, dtype, max_pages=40)
+    assert engine.model.graph_safe
+    res = engine.generate([Request(prompt_tokens=[7], request_id=0, max_new_tokens=300)])
+    out = res.tokens[0]
+    assert len(out) == 300
+    margin = 1e-3 if dtype == "float32" else 0.25
+    clear = check_greedy(W, raw, [7], out, margin)
+    print(f"long decoding {name} {dtype}: {clear} of 300 positions decided clearly")
+    assert clear >= (280 if dtype == "float32" else 100)
+    res = engine.generate([Request(prompt_tokens=p, request_id=i + 1, max_new_tokens=3) for i, p in enumerate(([5], [9, 4], [1, 2, 3]))])
+    for p, o in zip(([5], [9, 4], [1, 2, 3]), res.tokens):
+        check_greedy(W, raw, p, o, margin)
+    engine.cache.check_invariants()
+
+
+def test_the_command_line_generates_from_a_folder(tmp_path):
+    """``python -m levanter_amd.main.sample_lm`` on a Lelatar folder: greedy tokens are the plain implementation's."""
+    import json
+    import re
+    import subprocess
+    import sys
+
+    raw, W, d = model_folder("B", tmp_path, torch.float32)
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    prompts = [[3, 14, 15, 9, 2], [6]]
+    p = subprocess.run([sys.executable, "-m", "levanter_amd.main.sample_lm", "--hf_checkpoint", d, "--prompt_ids", json.dumps(prompts),
+                        "--temperature", "0", "--max_new_tokens", "12", "--n_rounds", "1", "--engine.compute_dtype", "float32",
+                        "--engine.max_seqs", "2", "--engine.max_pages_per_seq", "4"], capture_output=True, text=True, cwd=root, timeout=300)
+    assert p.returncode == 0, p.stderr[-2000:]
+    found = re.findall(r"round 0 sequence (\d+) \(12 tokens, length\): (\[.*\])", p.stdout)
+    assert len(found) == 2
+    for i, toks in found:
+        check_greedy(W, raw, prompts[int(i)], json.loads(toks), 1e-3)
