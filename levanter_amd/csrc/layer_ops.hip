@@ -718,11 +718,57 @@ norm_sum2_kernel(const float* __restrict__ a, const float* __restrict__ b, const
   }
 }
 
+// The same with the rows in registers: 16-byte loads, all of them in flight at once (NV vectors of 4 per thread and tensor).
+template <int NV>
+__global__ void __launch_bounds__(256)
+norm_sum2_reg_kernel(const float* __restrict__ a, const float* __restrict__ b, const float* __restrict__ wa, const float* __restrict__ wb, float sa,
+                     float sb, float eps, float* __restrict__ y, int D, int accumulate) {
+  __shared__ float red[8];
+  const size_t row = (size_t)blockIdx.x * D;
+  float4 av[NV], bv[NV], u[NV], v[NV], yv[NV];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int d = min((threadIdx.x + 256 * i) * 4, D - 4);
+    av[i] = *reinterpret_cast<const float4*>(a + row + d);
+    bv[i] = *reinterpret_cast<const float4*>(b + row + d);
+    u[i] = *reinterpret_cast<const float4*>(wa + d);
+    v[i] = *reinterpret_cast<const float4*>(wb + d);
+    if (accumulate) yv[i] = *reinterpret_cast<const float4*>(y + row + d);
+    else yv[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+  }
+  float ssa = 0.f, ssb = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i)
+    if ((threadIdx.x + 256 * i) * 4 < D) {
+      ssa = fmaf(av[i].x, av[i].x, fmaf(av[i].y, av[i].y, fmaf(av[i].z, av[i].z, fmaf(av[i].w, av[i].w, ssa))));
+      ssb = fmaf(bv[i].x, bv[i].x, fmaf(bv[i].y, bv[i].y, fmaf(bv[i].z, bv[i].z, fmaf(bv[i].w, bv[i].w, ssb))));
+    }
+  // both sums through one pair of barriers
+  ssa = wave_sum(ssa), ssb = wave_sum(ssb);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ssa, red[4 + (threadIdx.x >> 6)] = ssb;
+  __syncthreads();
+  ssa = (red[0] + red[1]) + (red[2] + red[3]), ssb = (red[4] + red[5]) + (red[6] + red[7]);
+  const float ra = sa / sqrtf(ssa / (float)D + eps), rb = sb / sqrtf(ssb / (float)D + eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int d = (threadIdx.x + 256 * i) * 4;
+    if (d < D)
+      *reinterpret_cast<float4*>(y + row + d) = make_float4(
+          yv[i].x + (av[i].x * ra * u[i].x + bv[i].x * rb * v[i].x), yv[i].y + (av[i].y * ra * u[i].y + bv[i].y * rb * v[i].y),
+          yv[i].z + (av[i].z * ra * u[i].z + bv[i].z * rb * v[i].z), yv[i].w + (av[i].w * ra * u[i].w + bv[i].w * rb * v[i].w));
+  }
+}
+
 extern "C" int lev_norm_sum2(const float* a, const float* b, const float* wa, const float* wb, float sa, float sb, float eps, float* y, int T, int D,
                              int accumulate, hipStream_t stream) {
   LEV_REQUIRE(T >= 0 && D > 0 && a && b && wa && wb && y, "norm_sum2: a tensor is missing or bad sizes T=%d D=%d", T, D);
   if (T == 0) return 0;
-  norm_sum2_kernel<<<T, 256, 0, stream>>>(a, b, wa, wb, sa, sb, eps, y, D, accumulate);
+  const bool vec = D % 4 == 0 && (((uintptr_t)a | (uintptr_t)b | (uintptr_t)wa | (uintptr_t)wb | (uintptr_t)y) & 15) == 0;
+  if (vec && D <= 1024) norm_sum2_reg_kernel<1><<<T, 256, 0, stream>>>(a, b, wa, wb, sa, sb, eps, y, D, accumulate);
+  else if (vec && D <= 2048) norm_sum2_reg_kernel<2><<<T, 256, 0, stream>>>(a, b, wa, wb, sa, sb, eps, y, D, accumulate);
+  else if (vec && D <= 4096) norm_sum2_reg_kernel<4><<<T, 256, 0, stream>>>(a, b, wa, wb, sa, sb, eps, y, D, accumulate);
+  else if (vec && D <= 8192) norm_sum2_reg_kernel<8><<<T, 256, 0, stream>>>(a, b, wa, wb, sa, sb, eps, y, D, accumulate);
+  else norm_sum2_kernel<<<T, 256, 0, stream>>>(a, b, wa, wb, sa, sb, eps, y, D, accumulate);
   return lev_check_launch("norm_sum2");
 }
 
@@ -755,13 +801,15 @@ extern "C" int lev_token_gate(const float* z, long z_stride, const int* tokens, 
 // head is paired with i + n_pairs, else 2i with 2i + 1; i < n_pairs, the rest of a head passes unrotated. Queries change in place. With
 // pages (steps of single tokens) keys and values go into them at dest[t] and stay as they are in k and v; without, keys change in place
 // and values are not touched. The arithmetic is the same either way. norm_dim_*: the projections' true sizes (heads may carry zeros).
+#define PNR_KEEP 8
+#define PNR_MAX_PAIRS 512
 template <typename T>
 __global__ void __launch_bounds__(256)
 projection_norm_rotate_kernel(T* __restrict__ q, long q_stride, int H, T* __restrict__ k, long k_stride, int G, int hd, const T* __restrict__ v,
                               long v_stride, int vd, float eps, int norm_dim_q, int norm_dim_k, const float* __restrict__ wq,
                               const float* __restrict__ wk, const float* __restrict__ freqs, int n_pairs, int half, const int* __restrict__ positions,
                               T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ dest, int PS) {
-  __shared__ float red[4];
+  __shared__ float red[4], s_sin[PNR_MAX_PAIRS], s_cos[PNR_MAX_PAIRS];
   const int t = blockIdx.x, tid = threadIdx.x;
   const int dst = k_pages ? dest[t] : 0, page = max(dst, 0) / max(PS, 1), off = k_pages ? max(dst, 0) % PS : 0;
   if (blockIdx.y == 2) {  // values: single tokens only
@@ -770,37 +818,78 @@ projection_norm_rotate_kernel(T* __restrict__ q, long q_stride, int H, T* __rest
     return;
   }
   const bool is_q = blockIdx.y == 0;
-  const int heads = is_q ? H : G, n = heads * hd;
+  const int heads = is_q ? H : G;
   T* row = is_q ? q + (size_t)t * q_stride : k + (size_t)t * k_stride;
   const float* w = is_q ? wq : wk;
-  float ss = 0.f;
-  for (int d = tid; d < n; d += 256) {
-    const float x = to_float<T>(row[d]);
-    ss = fmaf(x, x, ss);
+  // an item is a pair, or one of a head's dimensions that do not turn; the first PNR_KEEP items of a thread stay in registers from
+  // the sum to the result, their loads all in flight at once
+  const int items = hd - n_pairs, total = heads * items;
+  auto place = [&](int it, int& d0, int& d1) {
+    const int head = it / items, i = it - head * items;
+    d0 = head * hd + (i < n_pairs ? (half ? i : 2 * i) : i + n_pairs);
+    d1 = i < n_pairs ? (half ? d0 + n_pairs : d0 + 1) : d0;
+    return i;
+  };
+  T ra[PNR_KEEP], rb[PNR_KEEP];
+  float w0[PNR_KEEP], w1[PNR_KEEP];
+#pragma unroll
+  for (int m = 0; m < PNR_KEEP; ++m) {
+    int d0, d1;
+    place(min(tid + 256 * m, total - 1), d0, d1);
+    ra[m] = row[d0], rb[m] = row[d1];
+    w0[m] = w[d0], w1[m] = w[d1];
   }
-  ss = block_sum<256>(ss, red);
+  if (n_pairs) {  // the angles are the same for every head
+    const float pos = (float)positions[t];
+    for (int i = tid; i < n_pairs; i += 256) sincosf(pos * freqs[i], &s_sin[i], &s_cos[i]);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int m = 0; m < PNR_KEEP; ++m) {
+    if (tid + 256 * m >= total) continue;
+    int d0, d1;
+    place(tid + 256 * m, d0, d1);
+    const float a = to_float<T>(ra[m]), b = d1 != d0 ? to_float<T>(rb[m]) : 0.f;
+    ss = fmaf(a, a, fmaf(b, b, ss));
+  }
+  for (int it = tid + 256 * PNR_KEEP; it < total; it += 256) {
+    int d0, d1;
+    place(it, d0, d1);
+    const float a = to_float<T>(row[d0]), b = d1 != d0 ? to_float<T>(row[d1]) : 0.f;
+    ss = fmaf(a, a, fmaf(b, b, ss));
+  }
+  ss = block_sum<256>(ss, red);  // its barriers also stand between the table of angles and its readers
   const float r = 1.0f / sqrtf(ss / (float)(is_q ? norm_dim_q : norm_dim_k) + eps);
   if (!is_q && dst < 0) return;
-  const float pos = n_pairs ? (float)positions[t] : 0.f;
   T* kd = is_q || !k_pages ? nullptr : k_pages + (size_t)page * G * hd * PS;
-  auto put = [&](int head, int d, float val) {
-    if (kd) kd[(size_t)head * hd * PS + ((size_t)(d >> 3) * PS + off) * 8 + (d & 7)] = from_float<T>(val);
-    else row[head * hd + d] = from_float<T>(val);
-  };
-  const int items = hd - n_pairs;  // of a head: its pairs, then the dimensions that do not turn
-  for (int it = tid; it < heads * items; it += 256) {
-    const int head = it / items, i = it - head * items;
-    if (i < n_pairs) {
-      const int d0 = half ? i : 2 * i, d1 = half ? i + n_pairs : 2 * i + 1;
-      const float a = to_float<T>(row[head * hd + d0]) * r * w[head * hd + d0], b = to_float<T>(row[head * hd + d1]) * r * w[head * hd + d1];
-      float sn, cs;
-      sincosf(pos * freqs[i], &sn, &cs);
-      put(head, d0, a * cs - b * sn);
-      put(head, d1, b * cs + a * sn);
+  auto put = [&](int e, float val) {
+    if (kd) {
+      const int head = e / hd, d = e - head * hd;
+      kd[(size_t)head * hd * PS + ((size_t)(d >> 3) * PS + off) * 8 + (d & 7)] = from_float<T>(val);
     } else {
-      const int d = i + n_pairs;
-      put(head, d, to_float<T>(row[head * hd + d]) * r * w[head * hd + d]);
+      row[e] = from_float<T>(val);
     }
+  };
+  auto finish = [&](int it, float a, float b, float wa, float wb) {
+    int d0, d1;
+    const int i = place(it, d0, d1);
+    a = a * r * wa;
+    if (i < n_pairs) {
+      b = b * r * wb;
+      const float sn = s_sin[i], cs = s_cos[i];
+      put(d0, a * cs - b * sn);
+      put(d1, b * cs + a * sn);
+    } else {
+      put(d0, a);
+    }
+  };
+#pragma unroll
+  for (int m = 0; m < PNR_KEEP; ++m)
+    if (tid + 256 * m < total) finish(tid + 256 * m, to_float<T>(ra[m]), to_float<T>(rb[m]), w0[m], w1[m]);
+  for (int it = tid + 256 * PNR_KEEP; it < total; it += 256) {
+    int d0, d1;
+    place(it, d0, d1);
+    finish(it, to_float<T>(row[d0]), to_float<T>(row[d1]), w[d0], w[d1]);
   }
 }
 
@@ -811,7 +900,7 @@ extern "C" int lev_projection_norm_rotate(void* q, long q_stride, int H, void* k
   LEV_REQUIRE(T >= 0 && H > 0 && G > 0 && hd > 0 && hd % 8 == 0, "projection_norm_rotate: bad sizes T=%d heads=%d/%d size=%d", T, H, G, hd);
   LEV_REQUIRE(q && k && wq && wk && norm_dim_q > 0 && norm_dim_q <= H * hd && norm_dim_k > 0 && norm_dim_k <= G * hd, "projection_norm_rotate: a tensor is missing or bad divisors");
   LEV_REQUIRE(q_stride >= (long)H * hd && k_stride >= (long)G * hd, "projection_norm_rotate: row strides are smaller than the heads");
-  LEV_REQUIRE(n_pairs >= 0 && 2 * n_pairs <= hd && (n_pairs == 0 || (freqs && positions)), "projection_norm_rotate: %d rotated pairs need frequencies, positions and a head of at least twice their number", n_pairs);
+  LEV_REQUIRE(n_pairs >= 0 && n_pairs <= PNR_MAX_PAIRS && 2 * n_pairs <= hd && (n_pairs == 0 || (freqs && positions)), "projection_norm_rotate: %d rotated pairs need frequencies, positions and a head of at least twice their number", n_pairs);
   LEV_REQUIRE(!k_pages || (v && v_pages && dest && vd > 0 && PS > 0 && PS % 16 == 0 && v_stride >= (long)G * vd), "projection_norm_rotate: pages need values, destinations and a page size that is a multiple of 16");
   LEV_REQUIRE(dtype == LEV_F32 || dtype == LEV_BF16, "projection_norm_rotate: unknown dtype %d", dtype);
   if (T == 0) return 0;

@@ -53,16 +53,31 @@ __device__ __forceinline__ void sc_split(const float (&v)[8], sc_u32x4 (&out)[3]
       rest[2 * i + 1] -= __uint_as_float(w & 0xffff0000u);
     }
 }
+// the decays from tokens 4 grp + r of a tile to the token whose running sum is cs_i, zero for the tokens behind it in its own tile
+// (`diagonal`; the condition goes into the exponent: around the exponential it would become a branch per element)
+__device__ __forceinline__ sc_f32x4 sc_decays(double cs_i, const double* cs, bool diagonal, int grp, int col) {
+  typedef __attribute__((ext_vector_type(2))) double sc_f64x2;
+  const sc_f64x2 a = *reinterpret_cast<const sc_f64x2*>(cs), b = *reinterpret_cast<const sc_f64x2*>(cs + 2);
+  sc_f32x4 x = {(float)(cs_i - a[0]), (float)(cs_i - a[1]), (float)(cs_i - b[0]), (float)(cs_i - b[1])};
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    x[r] = diagonal && 4 * grp + r > col ? -INFINITY : fminf(x[r], 0.f);
+    x[r] = expf(x[r]);
+  }
+  return x;
+}
 __device__ __forceinline__ sc_u32x4 sc_read16(const bf16_t* p) { return *reinterpret_cast<const sc_u32x4*>(p); }
 __device__ __forceinline__ sc_u32x4 sc_read8x2(const bf16_t* p, const bf16_t* q) {
   const sc_u32x2 a = *reinterpret_cast<const sc_u32x2*>(p), b = *reinterpret_cast<const sc_u32x2*>(q);
   return sc_u32x4{a[0], a[1], b[0], b[1]};
 }
-// eight channels from i0 on of a row; zeros beyond dk
-__device__ __forceinline__ sc_u32x4 sc_load8(const bf16_t* row, int i0, int dk, int vec) {
+// eight channels from i0 on of a row of dk. VEC (rows are multiples of 8 channels at 16-byte boundaries): what lies beyond the row is some
+// other of its channels and the load stands under no condition (nothing waits for it before it is used); sc_mask8 puts zeros there.
+template <bool VEC>
+__device__ __forceinline__ sc_u32x4 sc_load8(const bf16_t* row, int i0, int dk) {
   sc_u32x4 v = {0, 0, 0, 0};
-  if (vec) {
-    if (i0 < dk) v = *reinterpret_cast<const sc_u32x4*>(row + i0);
+  if (VEC) {
+    v = *reinterpret_cast<const sc_u32x4*>(row + min(i0, dk - 8));
   } else {
 #pragma unroll
     for (int e = 0; e < 8; ++e)
@@ -70,27 +85,36 @@ __device__ __forceinline__ sc_u32x4 sc_load8(const bf16_t* row, int i0, int dk, 
   }
   return v;
 }
+__device__ __forceinline__ sc_u32x4 sc_mask8(sc_u32x4 v, int i0, int dk) {
+  const uint32_t keep = i0 < dk ? 0xffffffffu : 0u;
+  return sc_u32x4{v[0] & keep, v[1] & keep, v[2] & keep, v[3] & keep};
+}
 
-template <int DKM, int RULE>
+template <int DKM, int RULE, bool VEC>
 __global__ void __launch_bounds__(256)
 sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, float* __restrict__ state, const int* __restrict__ token_slots,
-                float* __restrict__ o, int vec, SrShape s) {
+                float* __restrict__ o, SrShape s) {
   constexpr int LDK = DKM + 8, KS = DKM / 32, NTW = DKM / 64, KI = DKM / 64, QI = DKM / 32;
   constexpr bool DELTA = RULE == SR_DELTA;
   __shared__ __attribute__((aligned(16))) bf16_t s_q[SC_Q][LDK], s_k[SC_Q][LDK], s_kt[DKM][SC_LDT], s_S[3][SC_VB][LDK];
   __shared__ __attribute__((aligned(16))) bf16_t s_x[DELTA ? 1 : SC_VB][SC_LDT];
-  __shared__ double s_cs[SC_Q];
+  __shared__ __attribute__((aligned(16))) double s_cs[SC_Q];
   __shared__ __attribute__((aligned(16))) float s_ecs[SC_Q], s_wend[SC_Q], s_w[SC_Q], s_rk[SC_Q], s_rq[SC_Q];
   __shared__ float s_end;
   __shared__ __attribute__((aligned(16))) sc_f32x4 s_A[DELTA ? 6 : 1][64], s_R[DELTA ? 4 : 1][64], s_T[DELTA ? 4 : 1][64];
   __shared__ __attribute__((aligned(16))) float s_At[DELTA ? 4 : 1][16][16];
   __shared__ int tmp[256 + 2];
-  const int h = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, grp = lane >> 4;
+  // Workgroups go to the 8 chiplets in turn: the runs a step may have and does not must not be every second or fourth of them, so the run is
+  // the slowest index; and the heads of a chiplet are neighbours, which read the same keys and queries through its cache.
+  const int n_items = gridDim.x, per_xcd = n_items / 8;
+  const int item = n_items % 8 == 0 ? (blockIdx.x % 8) * per_xcd + blockIdx.x / 8 : blockIdx.x;
+  const int n_blocks = (s.dv + SC_VB - 1) / SC_VB, h = item / n_blocks;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), col = lane & 15, grp = lane >> 4;
   const int g = h / (s.H / s.G), n_scal = 2 * s.H + 2 * s.G, dk = s.dk, dv = s.dv;
-  const int j = blockIdx.z * SC_VB + col;  // this lane's value column
+  const int j = (item - h * n_blocks) * SC_VB + col;  // this lane's value column
   const bool live = j < dv;
   int t0, t_end, slot;
-  if (!sr_find_run<256>(blockIdx.x, token_slots, s.Tn, tmp, t0, t_end, slot)) return;
+  if (!sr_find_run<256>(blockIdx.y, token_slots, s.Tn, tmp, t0, t_end, slot)) return;
   const bf16_t* uk = u + s.k_off + (size_t)g * dk;
   const bf16_t* uq = u + s.q_off + (size_t)g * dk;
   const bf16_t* uv = u + s.v_off + (size_t)h * dv;
@@ -108,38 +132,45 @@ sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, fl
 
   // what of the next chunk is on its way: keys (two neighbouring tokens, eight channels), queries, values, scalars
   sc_u32x4 nk[KI][2], nq[QI];
-  float nv[4], n_ld = 0.f, n_w = 0.f, n_rk = 0.f, n_rq = 0.f;
+  bf16_t nv[4];
+  float n_ld = 0.f, n_w = 0.f, n_rk = 0.f, n_rq = 0.f;
+  int n_tokens = 0;
+  // raw loads only: whatever is computed from them here would wait for their way through the memory
+  const int jc = live ? j : 0;
   auto fetch = [&](int tb) {
 #pragma unroll
     for (int n = 0; n < KI; ++n) {
       const int idx = tid + 256 * n, pair = idx & 31, i0 = (idx >> 5) * 8;
 #pragma unroll
-      for (int e = 0; e < 2; ++e) nk[n][e] = sc_load8(uk + (size_t)min(tb + 2 * pair + e, t_end - 1) * s.C, i0, dk, vec);
+      for (int e = 0; e < 2; ++e) nk[n][e] = sc_load8<VEC>(uk + (size_t)min(tb + 2 * pair + e, t_end - 1) * s.C, i0, dk);
     }
 #pragma unroll
     for (int n = 0; n < QI; ++n) {
       const int idx = tid + 256 * n, row = idx / (DKM / 8), i0 = (idx % (DKM / 8)) * 8;
-      nq[n] = sc_load8(uq + (size_t)min(tb + row, t_end - 1) * s.C, i0, dk, vec);
+      nq[n] = sc_load8<VEC>(uq + (size_t)min(tb + row, t_end - 1) * s.C, i0, dk);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       // DELTA: the rows and the column of this lane's part of R; SSD: 16 columns of four tokens per thread, for the transposed copy
       const int t = DELTA ? tb + 16 * wave + 4 * grp + r : tb + (tid >> 4) + 16 * r;
-      nv[r] = live ? to_float<bf16_t>(uv[(size_t)min(t, t_end - 1) * s.C + j]) : 0.f;
+      nv[r] = uv[(size_t)min(t, t_end - 1) * s.C + jc];
     }
     if (wave == 0) {
-      const int t = min(tb + lane, t_end - 1);
-      const float in = tb + lane < t_end ? 1.f : 0.f;  // tokens behind the run's end: no decay, no weight
-      const float* sc = scal + (size_t)t * n_scal;
-      n_ld = in * sc[h], n_w = in * sc[s.H + h], n_rk = in * sc[2 * s.H + g], n_rq = in * sc[2 * s.H + s.G + g];
+      const float* sc = scal + (size_t)min(tb + lane, t_end - 1) * n_scal;
+      n_ld = sc[h], n_w = sc[s.H + h];
+      if (DELTA) n_rk = sc[2 * s.H + g], n_rq = sc[2 * s.H + s.G + g];
     }
+    n_tokens = t_end - tb;
   };
   auto stage = [&]() {
 #pragma unroll
     for (int n = 0; n < KI; ++n) {
       const int idx = tid + 256 * n, pair = idx & 31, i0 = (idx >> 5) * 8;
 #pragma unroll
-      for (int e = 0; e < 2; ++e) *reinterpret_cast<sc_u32x4*>(&s_k[2 * pair + e][i0]) = nk[n][e];
+      for (int e = 0; e < 2; ++e) {
+        if (VEC) nk[n][e] = sc_mask8(nk[n][e], i0, dk);
+        *reinterpret_cast<sc_u32x4*>(&s_k[2 * pair + e][i0]) = nk[n][e];
+      }
 #pragma unroll
       for (int c = 0; c < 4; ++c) {  // channels i0 + 2 c and i0 + 2 c + 1 of both tokens, transposed
         const uint32_t a = nk[n][0][c], b = nk[n][1][c];
@@ -150,11 +181,11 @@ sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, fl
 #pragma unroll
     for (int n = 0; n < QI; ++n) {
       const int idx = tid + 256 * n, row = idx / (DKM / 8), i0 = (idx % (DKM / 8)) * 8;
-      *reinterpret_cast<sc_u32x4*>(&s_q[row][i0]) = nq[n];
+      *reinterpret_cast<sc_u32x4*>(&s_q[row][i0]) = VEC ? sc_mask8(nq[n], i0, dk) : nq[n];
     }
     if (!DELTA)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) s_x[col][(tid >> 4) + 16 * r] = float_to_bf16(nv[r]);
+      for (int r = 0; r < 4; ++r) s_x[col][(tid >> 4) + 16 * r] = live ? nv[r] : (bf16_t)0;
 #pragma unroll
     for (int n = 0; n < NTW; ++n) {
       float rest[4];
@@ -169,6 +200,8 @@ sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, fl
       }
     }
     if (wave == 0) {
+      const float in = lane < n_tokens ? 1.f : 0.f;  // tokens behind the run's end: no decay, no weight
+      n_ld *= in, n_w *= in, n_rk *= in, n_rq *= in;
       double cs = (double)n_ld;
 #pragma unroll
       for (int d = 1; d < 64; d <<= 1) {
@@ -189,8 +222,8 @@ sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, fl
     float v_now[4];
     stage();
 #pragma unroll
-    for (int r = 0; r < 4; ++r) v_now[r] = nv[r];
-    __syncthreads();
+    for (int r = 0; r < 4; ++r) v_now[r] = live ? to_float<bf16_t>(nv[r]) : 0.f;
+    lds_barrier();  // the loads and stores in flight are the thread's own and are not waited for
     if (tb + SC_Q < t_end) fetch(tb + SC_Q);
 
     // rows of the result: tokens 16 wave + .. ; S0^T q and (DELTA) S0^T k
@@ -233,13 +266,12 @@ sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, fl
           kk = sc_mfma(a, sc_read16(&s_k[16 * wave + col][32 * ks + 8 * grp]), kk);
           pq[jt] = sc_mfma(a, sc_read16(&s_q[16 * wave + col][32 * ks + 8 * grp]), pq[jt]);
         }
+        const sc_f32x4 dec = sc_decays(cs_i, &s_cs[16 * jt + 4 * grp], jt == wave, grp, col) * *reinterpret_cast<const sc_f32x4*>(&s_rk[16 * jt + 4 * grp]);
+        kk *= dec * wk_i;
+        pq[jt] *= dec * rq_i;
+        if (jt == wave) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int jj = 16 * jt + 4 * grp + r;
-          const float dec = expf(fminf((float)(cs_i - s_cs[jj]), 0.f)) * s_rk[jj];
-          const bool below = jt < wave || 4 * grp + r < col, upto = jt < wave || 4 * grp + r <= col;
-          kk[r] = below ? wk_i * dec * kk[r] : 0.f;
-          pq[jt][r] = upto ? rq_i * dec * pq[jt][r] : 0.f;
+          for (int r = 0; r < 4; ++r) kk[r] = 4 * grp + r == col ? 0.f : kk[r];  // A has nothing on the diagonal
         }
         if (jt < wave) {
           s_A[wave * (wave - 1) / 2 + jt][lane] = sc_f32x4{-kk[0], -kk[1], -kk[2], -kk[3]};
@@ -268,7 +300,7 @@ sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, fl
           s_T[wave][lane] = T;
         }
       }
-      __syncthreads();
+      lds_barrier();
       // every wave solves the whole system for the workgroup's columns: U stays in its registers
       sc_f32x4 U[4];
 #pragma unroll
@@ -308,12 +340,7 @@ sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, fl
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks)
           pq[jt] = sc_mfma(sc_read16(&s_k[16 * jt + col][32 * ks + 8 * grp]), sc_read16(&s_q[16 * wave + col][32 * ks + 8 * grp]), pq[jt]);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int jj = 16 * jt + 4 * grp + r;
-          const bool upto = jt < wave || 4 * grp + r <= col;
-          pq[jt][r] = upto ? pq[jt][r] * (expf(fminf((float)(cs_i - s_cs[jj]), 0.f)) * s_w[jj]) : 0.f;
-        }
+        pq[jt] *= sc_decays(cs_i, &s_cs[16 * jt + 4 * grp], jt == wave, grp, col) * *reinterpret_cast<const sc_f32x4*>(&s_w[16 * jt + 4 * grp]);
       }
       oq = oq * ecs_rows;
       const float dend = s_end;
@@ -351,7 +378,7 @@ sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, fl
       const int t = tb + 16 * wave + 4 * grp + r;
       if (live && t < t_end) o[((size_t)t * s.H + h) * dv + j] = oq[r];
     }
-    __syncthreads();  // the chunk's tiles have been read by every wave
+    lds_barrier();  // the chunk's tiles have been read by every wave
   }
   if (live) {
 #pragma unroll
@@ -367,11 +394,14 @@ sc_chunk_kernel(const bf16_t* __restrict__ u, const float* __restrict__ scal, fl
 int sr_chunks_launch(int rule, const bf16_t* u, const float* scal, float* state, const int* token_slots, float* o, int max_runs, const SrShape& s,
                      hipStream_t stream) {
   const int vec = s.C % 8 == 0 && s.dk % 8 == 0 && s.k_off % 8 == 0 && s.q_off % 8 == 0 && ((uintptr_t)u & 15) == 0;
-  const dim3 grid(max_runs, s.H, (s.dv + SC_VB - 1) / SC_VB);
+  const dim3 grid(s.H * ((s.dv + SC_VB - 1) / SC_VB), max_runs);
+  LEV_REQUIRE(max_runs <= 65535, "state recurrence: too many runs (%d)", max_runs);
 #define SC_GO(DKM)                                                                                                                   \
   do {                                                                                                                               \
-    if (rule == SR_DELTA) sc_chunk_kernel<DKM, SR_DELTA><<<grid, 256, 0, stream>>>(u, scal, state, token_slots, o, vec, s);            \
-    else sc_chunk_kernel<DKM, SR_SSD><<<grid, 256, 0, stream>>>(u, scal, state, token_slots, o, vec, s);                               \
+    if (rule == SR_DELTA && vec) sc_chunk_kernel<DKM, SR_DELTA, true><<<grid, 256, 0, stream>>>(u, scal, state, token_slots, o, s);     \
+    else if (rule == SR_DELTA) sc_chunk_kernel<DKM, SR_DELTA, false><<<grid, 256, 0, stream>>>(u, scal, state, token_slots, o, s);      \
+    else if (vec) sc_chunk_kernel<DKM, SR_SSD, true><<<grid, 256, 0, stream>>>(u, scal, state, token_slots, o, s);                      \
+    else sc_chunk_kernel<DKM, SR_SSD, false><<<grid, 256, 0, stream>>>(u, scal, state, token_slots, o, s);                              \
   } while (0)
   if (s.dk <= 64) SC_GO(64);
   else if (s.dk <= 128) SC_GO(128);

@@ -29,11 +29,18 @@ __device__ __forceinline__ bool sr_find_run(int run, const int* __restrict__ tok
   const int per = (Tn + NT - 1) / NT, lo = min(Tn, tid * per), hi = min(Tn, lo + per);
   int mine = 0;
   for (int t = lo; t < hi; ++t) mine += (token_slots[t] >= 0 && (t == 0 || token_slots[t - 1] != token_slots[t])) ? 1 : 0;
-  tmp[tid] = mine;
   if (tid == 0) tmp[NT] = -1, tmp[NT + 1] = Tn;
+  // the starts in the stretches before this thread's: across the lanes of its wave, then the waves before it
+  int upto = mine;
+#pragma unroll
+  for (int d = 1; d < 64; d <<= 1) {
+    const int up = __shfl_up(upto, d, 64);
+    if ((tid & 63) >= d) upto += up;
+  }
+  if ((tid & 63) == 63) tmp[tid >> 6] = upto;
   __syncthreads();
-  int before = 0;
-  for (int i = 0; i < tid; ++i) before += tmp[i];
+  int before = upto - mine;
+  for (int i = 0; i < (tid >> 6); ++i) before += tmp[i];
   if (run >= before && run < before + mine) {
     int seen = before;
     for (int t = lo; t < hi; ++t)
@@ -46,11 +53,11 @@ __device__ __forceinline__ bool sr_find_run(int run, const int* __restrict__ tok
   t0 = tmp[NT];
   if (t0 < 0) return false;  // the whole workgroup
   slot = token_slots[t0];
-  for (int t = max(lo, t0 + 1); t < hi; ++t)
-    if (token_slots[t] != slot) {
-      atomicMin(&tmp[NT + 1], t);
-      break;
-    }
+  int end = Tn;  // the first later token of another slot
+#pragma unroll 8
+  for (int t = tid; t < Tn; t += NT)
+    if (t > t0 && token_slots[t] != slot) end = min(end, t);
+  if (end < Tn) atomicMin(&tmp[NT + 1], end);
   __syncthreads();
   t_end = tmp[NT + 1];
   return true;

@@ -123,10 +123,10 @@ sr_walk_kernel(const T* __restrict__ u, const float* __restrict__ scal, float* _
   constexpr int IP = DKM / 8;
   __shared__ float s_k[SR_WT][DKM], s_q[SR_WT][DKM];
   __shared__ int tmp[256 + 2];
-  const int h = blockIdx.y, tid = threadIdx.x, part = tid & 7, j = blockIdx.z * SR_WC + (tid >> 3);
+  const int h = blockIdx.x, tid = threadIdx.x, part = tid & 7, j = blockIdx.y * SR_WC + (tid >> 3);
   const int g = h / (s.H / s.G), n_scal = 2 * s.H + 2 * s.G;
   int t0, t_end, slot;
-  if (!sr_find_run<256>(blockIdx.x, token_slots, s.Tn, tmp, t0, t_end, slot)) return;
+  if (!sr_find_run<256>(blockIdx.z, token_slots, s.Tn, tmp, t0, t_end, slot)) return;
   const bool live = j < s.dv;
   float* sp = state + (size_t)slot * s.slot_stride + (size_t)s.K * s.C + (size_t)h * s.dk * s.dv + (live ? j : 0);
   float S[IP];
@@ -275,23 +275,51 @@ sr_token_kernel(const T* __restrict__ x, const float* __restrict__ taps, const f
     }
   }
   // convolution of this head's values and its group's keys and queries; the shared channels' ring row is the first head's to write
-  for (int idx = tid; idx < DVM + 2 * DKM; idx += NT) {
-    const int which = idx < DVM ? 0 : idx < DVM + DKM ? 1 : 2, i = which == 0 ? idx : which == 1 ? idx - DVM : idx - DVM - DKM;
-    const bool in = i < (which == 0 ? dv : dk);
-    float val = 0.f;
-    if (in) {
-      const int c = which == 0 ? s.v_off + h * dv + i : which == 1 ? s.k_off + g * dk + i : s.q_off + g * dk + i;
-      const float cur = to_float<T>(x[(size_t)t * s.x_stride + c]);
-      float acc = conv_bias ? conv_bias[c] : 0.f;
-      acc = fmaf(taps[(size_t)c * K + K - 1], cur, acc);
-      for (int k = 1; k < K; ++k)
-        if (pos - k >= 0) acc = fmaf(taps[(size_t)c * K + K - 1 - k], ring[(size_t)((pos - k) % K) * C + c], acc);
-      val = to_float<T>(from_float<T>(sr_silu(acc)));
-      if (which == 0 || h % rep == 0) ring[(size_t)(pos % K) * C + c] = cur;
+  {
+    constexpr int NIT = (DVM + 2 * DKM + NT - 1) / NT;
+    // the channel of a thread's n-th item (clamped: loads stand under no condition) and whether there is one
+    auto item = [&](int n, int& which, int& i, bool& in) {
+      const int idx = min(tid + NT * n, DVM + 2 * DKM - 1);
+      which = idx < DVM ? 0 : idx < DVM + DKM ? 1 : 2;
+      i = which == 0 ? idx : which == 1 ? idx - DVM : idx - DVM - DKM;
+      in = i < (which == 0 ? dv : dk);
+      const int ic = in ? i : 0;
+      return which == 0 ? s.v_off + h * dv + ic : which == 1 ? s.k_off + g * dk + ic : s.q_off + g * dk + ic;
+    };
+    T cur[NIT];
+    float acc[NIT], tap[NIT][4], old[NIT][3];
+#pragma unroll
+    for (int n = 0; n < NIT; ++n) {
+      int which, i;
+      bool in;
+      const int c = item(n, which, i, in);
+      cur[n] = x[(size_t)t * s.x_stride + c];
+      acc[n] = conv_bias ? conv_bias[c] : 0.f;
+#pragma unroll
+      for (int k = 0; k < 4; ++k) tap[n][k] = taps[(size_t)c * K + max(K - 1 - k, 0)];
+#pragma unroll
+      for (int k = 1; k < 4; ++k) old[n][k - 1] = ring[(size_t)((pos + 4 * K - k) % K) * C + c];
     }
-    if (which == 0) s_v[i] = val;
-    else if (which == 1) s_k[i] = val;
-    else s_q[i] = val;
+#pragma unroll
+    for (int n = 0; n < NIT; ++n) {
+      int which, i;
+      bool in;
+      const int c = item(n, which, i, in);
+      const float cf = to_float<T>(cur[n]);
+      acc[n] = fmaf(tap[n][0], cf, acc[n]);
+#pragma unroll
+      for (int k = 1; k < 4; ++k)
+        if (k < K && pos - k >= 0) acc[n] = fmaf(tap[n][k], old[n][k - 1], acc[n]);
+      for (int k = 4; k < K; ++k)
+        if (pos - k >= 0) acc[n] = fmaf(taps[(size_t)c * K + K - 1 - k], ring[(size_t)((pos - k) % K) * C + c], acc[n]);
+      const float val = in ? to_float<T>(from_float<T>(sr_silu(acc[n]))) : 0.f;
+      if (tid + NT * n < DVM + 2 * DKM) {
+        if (in && (which == 0 || h % rep == 0)) ring[(size_t)(pos % K) * C + c] = cf;
+        if (which == 0) s_v[i] = val;
+        else if (which == 1) s_k[i] = val;
+        else s_q[i] = val;
+      }
+    }
   }
   const float sft = sr_softplus(to_float<T>(a[(size_t)t * s.a_stride + h]) + a_bias[h]);
   const float d = expf(-rate[h] * sft);
@@ -301,11 +329,12 @@ sr_token_kernel(const T* __restrict__ x, const float* __restrict__ taps, const f
   __syncthreads();
   float rk = 1.f, rq = 1.f, qk = 0.f;
   if (RULE == SR_DELTA) {
-    float kk = 0.f, qq = 0.f;
-    for (int i = tid; i < DKM; i += NT) kk = fmaf(s_k[i], s_k[i], kk), qq = fmaf(s_q[i], s_q[i], qq), qk = fmaf(s_k[i], s_q[i], qk);
-    kk = block_sum<NT>(kk, red);
-    qq = block_sum<NT>(qq, red);
-    qk = block_sum<NT>(qk, red);
+    float kk = 0.f, qq = 0.f;  // every wave for itself: no barrier
+#pragma unroll
+    for (int i = tid & 63; i < DKM; i += 64) kk = fmaf(s_k[i], s_k[i], kk), qq = fmaf(s_q[i], s_q[i], qq), qk = fmaf(s_k[i], s_q[i], qk);
+    kk = wave_sum(kk);
+    qq = wave_sum(qq);
+    qk = wave_sum(qk);
     rk = 1.0f / sqrtf(kk + s.key_eps);
     rq = s.q_scale / sqrtf(qq + s.key_eps);
     qk *= rk * rq;
@@ -361,6 +390,7 @@ sr_token_kernel(const T* __restrict__ x, const float* __restrict__ taps, const f
       }
     }
   }
+  if (DVM == 64 && tid >= 64) return;  // one wave has the columns, and no barrier follows
   float o = 0.f;
   const bool mine = tid < dv;
   if (mine) {
@@ -377,7 +407,7 @@ sr_token_kernel(const T* __restrict__ x, const float* __restrict__ taps, const f
     for (int i = 0; i < 16; ++i) ks += s_pk[i][tid];
     o = fmaf(qk, w * (s_v[tid] - d * rk * ks), d * rq * o);
   }
-  const float ss = block_sum<NT>(mine ? o * o : 0.f, red);
+  const float ss = block_sum<DVM == 64 ? 64 : NT>(mine ? o * o : 0.f, red);
   if (mine) out[(size_t)t * s.o_stride + vcol + tid] = from_float<T>(o / sqrtf(ss / (float)dv + s.norm_eps) * nw * sr_silu(gt));
 }
 
@@ -452,7 +482,8 @@ static int sr_runs_launch(const T* x, const float* taps, const float* conv_bias,
     sr_finish_launch<T, RULE>(o, u, skip, gate, norm_w, token_slots, out, norm_groups, s, stream);
     return lev_check_launch("state recurrence (norm)");
   }
-  const dim3 walk(max_runs, s.H, (s.dv + SR_WC - 1) / SR_WC);
+  LEV_REQUIRE(max_runs <= 65535, "state recurrence: too many runs (%d)", max_runs);
+  const dim3 walk(s.H, (s.dv + SR_WC - 1) / SR_WC, max_runs);
   if (s.dk <= 64) sr_walk_kernel<T, 64, RULE><<<walk, 256, 0, stream>>>(u, scal, state, token_slots, o, s);
   else if (s.dk <= 128) sr_walk_kernel<T, 128, RULE><<<walk, 256, 0, stream>>>(u, scal, state, token_slots, o, s);
   else sr_walk_kernel<T, 256, RULE><<<walk, 256, 0, stream>>>(u, scal, state, token_slots, o, s);
