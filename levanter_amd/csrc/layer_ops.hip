@@ -795,6 +795,60 @@ extern "C" int lev_token_gate(const float* z, long z_stride, const int* tokens, 
   return lev_check_launch("token_gate");
 }
 
+// The product and the gate in one kernel for a few rows: out[t][i] = gelu_tanh(h[t] . w[i]) * table[tokens[t]][i]. A wave has one output i and TT
+// rows: 16-byte loads, a lane's share of the row at once, 32-bit sums across the lanes.
+template <typename T, int TT>
+__global__ void __launch_bounds__(256)
+token_gate_linear_kernel(const T* __restrict__ h, long h_stride, const T* __restrict__ w, const int* __restrict__ tokens, const T* __restrict__ table,
+                         T* __restrict__ out, int Tn, int N, int K) {
+  constexpr int E = 16 / (int)sizeof(T);
+  typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
+  union Chunk { u32x4 raw; T v[E]; };
+  const int lane = threadIdx.x & 63, i = blockIdx.x * 4 + (threadIdx.x >> 6), t0 = blockIdx.y * TT;
+  if (i >= N) return;
+  float acc[TT];
+#pragma unroll
+  for (int tt = 0; tt < TT; ++tt) acc[tt] = 0.f;
+#pragma unroll 4
+  for (int c = lane * E; c < K; c += 64 * E) {
+    Chunk wc;
+    wc.raw = *reinterpret_cast<const u32x4*>(w + (size_t)i * K + c);
+#pragma unroll
+    for (int tt = 0; tt < TT; ++tt) {
+      Chunk hc;
+      hc.raw = *reinterpret_cast<const u32x4*>(h + (size_t)min(t0 + tt, Tn - 1) * h_stride + c);
+#pragma unroll
+      for (int e = 0; e < E; ++e) acc[tt] = fmaf(to_float<T>(hc.v[e]), to_float<T>(wc.v[e]), acc[tt]);
+    }
+  }
+#pragma unroll
+  for (int tt = 0; tt < TT; ++tt) {
+    const float z = wave_sum(acc[tt]);
+    const int t = t0 + tt;
+    if (lane == tt && t < Tn)
+      out[(size_t)t * N + i] = from_float<T>(lev_activate(z, LEV_ACT_GELU_TANH) * to_float<T>(table[(size_t)tokens[t] * N + i]));
+  }
+}
+
+extern "C" int lev_token_gate_linear(const void* h, long h_stride, const void* w, const int* tokens, const void* table, void* out, int T, int N, int K,
+                                     int dtype, hipStream_t stream) {
+  LEV_REQUIRE(T >= 0 && N > 0 && K > 0 && h && w && tokens && table && out && h_stride >= K, "token_gate_linear: a tensor is missing or bad sizes T=%d N=%d K=%d", T, N, K);
+  LEV_REQUIRE(dtype == LEV_F32 || dtype == LEV_BF16, "token_gate_linear: unknown dtype %d", dtype);
+  LEV_REQUIRE(K % 8 == 0 && h_stride % 8 == 0 && (((uintptr_t)h | (uintptr_t)w) & 15) == 0, "token_gate_linear: rows must be multiples of 8 numbers at 16-byte boundaries");
+  if (T == 0) return 0;
+  const int tt = T <= 8 ? 1 : 4;
+  const dim3 grid((N + 3) / 4, (T + tt - 1) / tt);
+  LEV_REQUIRE(grid.y <= 65535, "token_gate_linear: too many rows (%d)", T);
+#define TGL(TY, TT) token_gate_linear_kernel<TY, TT><<<grid, 256, 0, stream>>>((const TY*)h, h_stride, (const TY*)w, tokens, (const TY*)table, (TY*)out, T, N, K)
+  if (dtype == LEV_F32) {
+    if (tt == 1) TGL(float, 1); else TGL(float, 4);
+  } else {
+    if (tt == 1) TGL(bf16_t, 1); else TGL(bf16_t, 4);
+  }
+#undef TGL
+  return lev_check_launch("token_gate_linear");
+}
+
 // ------------------------------------------------------------------------------------------
 // Queries and keys normed over their whole projections (all heads of a token at once, with a weight as wide as the projection), then
 // rotated, in one kernel with 32-bit numbers between the two: one workgroup per (token, queries | keys | values). `half`: dimension i of a

@@ -69,6 +69,55 @@ sr_conv_kernel(const T* __restrict__ x, const float* __restrict__ taps, const fl
   }
 }
 
+// four neighbouring elements: 8 bytes of bfloat16 or 16 of float32
+template <typename T>
+struct __attribute__((aligned(4 * sizeof(T)))) SrQuad {
+  T v[4];
+};
+
+// The same for up to four taps with four channels a thread (8-byte or 16-byte loads; C and the row stride multiples of 4).
+template <typename T>
+__global__ void __launch_bounds__(256)
+sr_conv_quad_kernel(const T* __restrict__ x, const float* __restrict__ taps, const float* __restrict__ bias, const float* __restrict__ state,
+                    const int* __restrict__ token_slots, const int* __restrict__ positions, T* __restrict__ u, SrShape s) {
+  const int c = (blockIdx.y * 256 + threadIdx.x) * 4, t0 = blockIdx.x * SR_CT;
+  const int C = s.C, K = s.K;
+  if (c >= C) return;
+  float b[4], tap[4][4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    b[e] = bias ? bias[c + e] : 0.f;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) tap[k][e] = k < K ? taps[(size_t)(c + e) * K + max(K - 1 - k, 0)] : 0.f;
+  }
+  SrQuad<T> xv[SR_CT + 3];
+#pragma unroll
+  for (int i = 0; i < SR_CT + 3; ++i) xv[i] = *reinterpret_cast<const SrQuad<T>*>(x + (size_t)min(max(t0 + i - 3, 0), s.Tn - 1) * s.x_stride + c);
+#pragma unroll
+  for (int i = 0; i < SR_CT; ++i) {
+    const int t = t0 + i;
+    if (t >= s.Tn) break;
+    const int slot = token_slots[t], pos = positions[t];
+    float acc[4] = {b[0], b[1], b[2], b[3]};
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      if (k >= K || slot < 0) continue;
+      if (k == 0 || (t - k >= 0 && token_slots[t - k] == slot)) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[e] = fmaf(tap[k][e], to_float<T>(xv[i + 3 - k].v[e]), acc[e]);
+      } else if (pos - k >= 0) {
+        const float* row = state + (size_t)slot * s.slot_stride + (size_t)((pos - k) % K) * C + c;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[e] = fmaf(tap[k][e], row[e], acc[e]);
+      }
+    }
+    SrQuad<T> w;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) w.v[e] = from_float<T>(slot < 0 ? 0.f : sr_silu(acc[e]));
+    *reinterpret_cast<SrQuad<T>*>(u + (size_t)t * C + c) = w;
+  }
+}
+
 // ---- per token: log decay and write rate of every head, inverse norms of keys and queries, the ring of inputs ----------------
 // scal: [Tn][2 H + 2 G] = log decays | write rates | 1 / |k| | q_scale / |q|  (SSD: ones)
 template <typename T, int RULE>
@@ -229,6 +278,65 @@ sr_finish_kernel(const float* __restrict__ o, const T* __restrict__ u, const flo
   for (int i = 0; i < KEEP; ++i)
     if (tid + NT * i < len) store(tid + NT * i, kept[i]);
   for (int c = tid + NT * KEEP; c < len; c += NT) store(c, value(c));
+}
+
+// The same with four neighbouring numbers a lane, NV of them: LANES lanes share a part (a wave or less: several parts a workgroup; 256: the
+// whole workgroup). Everything is a multiple of 4 and aligned; LANES * NV * 4 >= len.
+template <typename T, int RULE, int LANES, int NV>
+__global__ void __launch_bounds__(256)
+sr_finish_quad_kernel(const float* __restrict__ o, const T* __restrict__ u, const float* __restrict__ skip, const T* __restrict__ gate,
+                      const float* __restrict__ norm_w, const int* __restrict__ token_slots, T* __restrict__ out, int len, int parts, SrShape s) {
+  __shared__ float red[4];
+  const int t = blockIdx.x, lane = threadIdx.x % LANES;
+  const int part = min((int)(blockIdx.y * (256 / LANES) + threadIdx.x / LANES), parts - 1);  // the last workgroup's surplus lanes repeat the last part
+  const int c0 = part * len;
+  const bool nobody = token_slots[t] < 0;
+  float y[NV][4];
+  SrQuad<T> gv[NV];
+  float4 wv[NV];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = min((lane + LANES * i) * 4, len - 4);
+    const float4 ov = *reinterpret_cast<const float4*>(o + (size_t)t * s.H * s.dv + c0 + c);
+    gv[i] = *reinterpret_cast<const SrQuad<T>*>(gate + (size_t)t * s.gate_stride + c0 + c);
+    wv[i] = *reinterpret_cast<const float4*>(norm_w + c0 + c);
+    y[i][0] = ov.x, y[i][1] = ov.y, y[i][2] = ov.z, y[i][3] = ov.w;
+    if (RULE == SR_SSD && u) {
+      const SrQuad<T> x = *reinterpret_cast<const SrQuad<T>*>(u + (size_t)t * s.C + s.v_off + c0 + c);
+      const float sk = skip[(c0 + c) / s.dv];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[i][e] = fmaf(sk, to_float<T>(x.v[e]), y[i][e]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NV; ++i)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      if (RULE == SR_SSD) y[i][e] *= sr_silu(to_float<T>(gv[i].v[e]));
+      if ((lane + LANES * i) * 4 < len) ss = fmaf(y[i][e], y[i][e], ss);
+    }
+  if (LANES == 256) {
+    ss = block_sum<256>(ss, red);
+  } else {
+#pragma unroll
+    for (int d = LANES / 2; d > 0; d >>= 1) ss += __shfl_xor(ss, d, 64);
+  }
+  const float r = 1.0f / sqrtf(ss / (float)len + s.norm_eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (lane + LANES * i) * 4;
+    if (c >= len) continue;
+    const float w4[4] = {wv[i].x, wv[i].y, wv[i].z, wv[i].w};
+    SrQuad<T> w;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      float z = y[i][e] * r * w4[e];
+      if (RULE == SR_DELTA) z *= sr_silu(to_float<T>(gv[i].v[e]));
+      w.v[e] = from_float<T>(nobody ? 0.f : z);
+    }
+    *reinterpret_cast<SrQuad<T>*>(out + (size_t)t * s.o_stride + c0 + c) = w;
+  }
 }
 
 // ---- steps of single tokens ----------------------------------------------------------------------------------------------------------
@@ -431,6 +539,22 @@ template <typename T, int RULE>
 static void sr_finish_launch(const float* o, const T* u, const float* skip, const T* gate, const float* norm_w, const int* token_slots, T* out,
                              int norm_groups, const SrShape& s, hipStream_t stream) {
   const int parts = RULE == SR_DELTA ? s.H : norm_groups, len = s.H * s.dv / parts;
+  const uintptr_t a4 = 4 * sizeof(T) - 1;
+  const bool quad = len % 4 == 0 && s.dv % 4 == 0 && s.C % 4 == 0 && s.v_off % 4 == 0 && s.gate_stride % 4 == 0 && s.o_stride % 4 == 0 &&
+                    (((uintptr_t)o | (uintptr_t)norm_w) & 15) == 0 && (((uintptr_t)u | (uintptr_t)gate | (uintptr_t)out) & a4) == 0;
+#define SR_FQ(LANES, NV)                                                                                                                         \
+  do {                                                                                                                                           \
+    sr_finish_quad_kernel<T, RULE, LANES, NV><<<dim3(s.Tn, (parts + 256 / LANES - 1) / (256 / LANES)), 256, 0, stream>>>(o, u, skip, gate, norm_w,  \
+                                                                                                                        token_slots, out, len, parts, s); \
+    return;                                                                                                                                      \
+  } while (0)
+  if (quad && len <= 64) SR_FQ(16, 1);
+  if (quad && len <= 128) SR_FQ(32, 1);
+  if (quad && len <= 256) SR_FQ(64, 1);
+  if (quad && len <= 1024) SR_FQ(256, 1);
+  if (quad && len <= 2048) SR_FQ(256, 2);
+  if (quad && len <= 4096) SR_FQ(256, 4);
+#undef SR_FQ
   if (len <= 128) sr_finish_kernel<T, RULE, 64><<<dim3(s.Tn, parts), 64, 0, stream>>>(o, u, skip, gate, norm_w, token_slots, out, len, s);
   else if (len <= 1024) sr_finish_kernel<T, RULE, 256><<<dim3(s.Tn, parts), 256, 0, stream>>>(o, u, skip, gate, norm_w, token_slots, out, len, s);
   else sr_finish_kernel<T, RULE, 1024><<<dim3(s.Tn, parts), 1024, 0, stream>>>(o, u, skip, gate, norm_w, token_slots, out, len, s);
@@ -473,7 +597,11 @@ static int sr_runs_launch(const T* x, const float* taps, const float* conv_bias,
   float* o = ws;
   float* scal = o + sr_pad4((long)s.Tn * s.H * s.dv);
   T* u = reinterpret_cast<T*>(scal + sr_pad4((long)s.Tn * (2 * s.H + 2 * s.G)));
-  sr_conv_kernel<T><<<dim3((s.Tn + SR_CT - 1) / SR_CT, (s.C + 255) / 256), 256, 0, stream>>>(x, taps, conv_bias, state, token_slots, positions, u, s);
+  const uintptr_t a4 = 4 * sizeof(T) - 1;
+  if (s.K <= 4 && s.C % 4 == 0 && s.x_stride % 4 == 0 && (((uintptr_t)x | (uintptr_t)u) & a4) == 0)
+    sr_conv_quad_kernel<T><<<dim3((s.Tn + SR_CT - 1) / SR_CT, (s.C / 4 + 255) / 256), 256, 0, stream>>>(x, taps, conv_bias, state, token_slots, positions, u, s);
+  else
+    sr_conv_kernel<T><<<dim3((s.Tn + SR_CT - 1) / SR_CT, (s.C + 255) / 256), 256, 0, stream>>>(x, taps, conv_bias, state, token_slots, positions, u, s);
   if (lev_check_launch("state recurrence (convolution)")) return -1;
   sr_prepare_kernel<T, RULE><<<s.Tn, 256, 0, stream>>>(x, u, a, b, a_bias, rate, state, token_slots, positions, scal, s);
   if (lev_check_launch("state recurrence (prepare)")) return -1;

@@ -306,6 +306,7 @@ register_unit("core", ["errors.hip", "elementwise.hip", "layer_ops.hip", "gemm_s
     "lev_head_talk": [_P, _P, _P, _L, _P, _L] + [_I] * 5 + [_F, _I, _I, _P],
     "lev_glu_activate": [_P, _L, _P, _L, _I, _I, _I, _F, _F, _I, _P],
     "lev_norm_sum2": [_P, _P, _P, _P, _F, _F, _F, _P, _I, _I, _I, _P],
+    "lev_token_gate_linear": [_P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "lev_token_gate": [_P, _L, _P, _P, _P, _I, _I, _I, _P],
     "lev_projection_norm_rotate": [_P, _L, _I, _P, _L, _I, _I, _P, _L, _I, _F, _I, _I, _P, _P, _P, _I, _I, _P, _P, _P, _P, _I, _I, _I, _P],
     "lev_state_recurrence": [_I, _P, _L, _P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _P, _P, _L, _P, _P, _P, _L, _P] + [_I] * 12 + [_F, _F, _F, _I, _I, _P],

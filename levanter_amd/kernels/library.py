@@ -1049,6 +1049,22 @@ class HipKernels:
             _req(w.dtype == torch.float32 and w.is_contiguous() and w.numel() == D, "norm_sum2: the weights must be float32 [D]")
         self._check(self.lib.lev_norm_sum2(_ptr(a), _ptr(b), _ptr(weight_a), _ptr(weight_b), float(scale_a), float(scale_b), float(eps), _ptr(y), T, D, int(bool(accumulate)), self._s()))
 
+    TOKEN_GATE_MAX_ROWS = 64  # more rows than this take the matrix product and ``token_gate``
+
+    def token_gate_linear(self, h, w, tokens, table, out) -> bool:
+        """``out[t] = gelu_tanh(w h[t]) * table[tokens[t]]`` in one kernel, for a few rows: ``h`` ``[T, K]``, ``w`` ``[D, K]``, ``table`` ``[vocab, D]`` and ``out``
+        ``[T, D]`` of one compute dtype, 32-bit sums. False (nothing launched): more rows or other alignments than it takes."""
+        _dev(h, w, tokens, table, out)
+        T, N = out.shape
+        Kd, dt = h.shape[1], h.dtype
+        _req(dt in _DT and dt == w.dtype == table.dtype == out.dtype and h.shape[0] == T and tuple(w.shape) == (N, Kd) and w.is_contiguous(), "token_gate_linear: h [T, K], w [D, K], out [T, D] of one compute dtype")
+        _req(tokens.dtype == torch.int32 and tokens.numel() == T and table.is_contiguous() and out.is_contiguous() and table.dim() == 2 and table.shape[1] == N, "token_gate_linear: one int32 token per row, contiguous table [vocab, D] and out")
+        hs = _rows(h, "token_gate_linear: h")
+        if T > self.TOKEN_GATE_MAX_ROWS or Kd % 8 or hs % 8 or (h.data_ptr() | w.data_ptr()) % 16:
+            return False
+        self._check(self.lib.lev_token_gate_linear(_ptr(h), hs, _ptr(w), _ptr(tokens), _ptr(table), _ptr(out), T, N, Kd, _DT[dt], self._s()))
+        return True
+
     def token_gate(self, z, tokens, table, out) -> None:
         """``out[t] = gelu_tanh(z[t]) * table[tokens[t]]``: ``z`` float32 ``[T, D]`` (rows may be strided), ``table`` ``[vocab, D]`` and ``out``
         ``[T, D]`` of one compute dtype. Token ids are trusted (the step checks them)."""

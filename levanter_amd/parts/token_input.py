@@ -53,9 +53,10 @@ class GatedTokenInput(Part):
 
     def add(self, x: torch.Tensor, ctx: StepContext) -> None:
         K = ctx.kernels
-        z = self.gate(read_stream(x, ctx, 1, self.eps), ctx, out_dtype=torch.float32)
+        h = read_stream(x, ctx, 1, self.eps)
         g = ctx.empty(x.shape[0], self.padded)
-        K.token_gate(z, ctx.tokens, self.table, g)
+        if not K.token_gate_linear(h, self.gate.weight, ctx.tokens, self.table, g):
+            K.token_gate(self.gate(h, ctx, out_dtype=torch.float32), ctx.tokens, self.table, g)
         y = self.proj(g, ctx, out_dtype=torch.float32)
         pending = K.group_norm_step(x, groups=1, eps=self.eps, y=y, post_weight=self.norm_weight, defer=True)
         if ctx.may_defer:

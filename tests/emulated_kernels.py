@@ -330,6 +330,12 @@ class EmulatedKernels:
                 o = o / torch.sqrt((o * o).mean(-1, keepdim=True) + norm_eps)
                 out[t] = (o.reshape(-1) * norm_weight * F.silu(gate[t].float())).to(out.dtype)
 
+    def token_gate_linear(self, h, w, tokens, table, out) -> bool:
+        if h.shape[0] > 8:  # both ways are taken
+            return False
+        self.token_gate(h.float() @ w.float().t(), tokens, table, out)
+        return True
+
     def token_gate(self, z, tokens, table, out) -> None:
         out.copy_((F.gelu(z.float(), approximate="tanh") * table[tokens.long()].float()).to(out.dtype))
 

@@ -321,6 +321,19 @@ def test_the_token_tables_gate(dtype, T, D):
     torch.testing.assert_close(out.cpu().double(), P.gelu_tanh(z[:, :D].double()) * table[tokens], **tol(dtype, f32=1e-5, bf16=1e-2))
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,N,Kd", [(1, 8, 64), (5, 24, 256), (8, 128, 2048), (9, 16, 40), (64, 64, 1032), (65, 16, 64), (3, 16, 36)])
+def test_the_gate_product_and_the_token_tables_gate_in_one_kernel(dtype, T, N, Kd):
+    g = torch.Generator().manual_seed(T + Kd)
+    h, w, table = bfn(torch.randn(T, Kd, generator=g)), bfn(torch.randn(N, Kd, generator=g) / math.sqrt(Kd)), bfn(torch.randn(40, N, generator=g))
+    tokens = torch.randint(0, 40, (T,), generator=g)
+    out = torch.empty(T, N, dtype=dtype, device=DEV)
+    took = K().token_gate_linear(dev(h, dtype), dev(w, dtype), ints(tokens.tolist()), dev(table, dtype), out)
+    assert took == (T <= 64 and Kd % 8 == 0)
+    if took:
+        torch.testing.assert_close(out.cpu().double(), P.gelu_tanh(h @ w.T) * table[tokens], **tol(dtype, f32=1e-5, bf16=1e-2))
+
+
 @pytest.mark.parametrize("T,D", [(5, 64), (3, 1000), (1, 7)])
 def test_the_sum_of_two_normed_branches_is_added_to_the_stream(T, D):
     g = torch.Generator().manual_seed(D)
