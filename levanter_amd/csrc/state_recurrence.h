@@ -63,7 +63,8 @@ __device__ __forceinline__ bool sr_find_run(int run, const int* __restrict__ tok
   return true;
 }
 
-// Steps with runs, bfloat16: the recurrence in chunks of 64 tokens on the matrix cores (state_chunks.hip); the same inputs and outputs as the
-// walk token by token.
-int sr_chunks_launch(int rule, const bf16_t* u, const float* scal, float* state, const int* token_slots, float* o, int max_runs, const SrShape& s,
-                     hipStream_t stream);
+// Steps with runs, bfloat16: the recurrence in chunks of up to 64 tokens on the matrix cores (state_chunks.hip); the same inputs and outputs as
+// the walk token by token. workspace: sr_chunks_workspace floats at a 16-byte boundary.
+int sr_chunks_launch(int rule, const bf16_t* u, const float* scal, float* state, const int* token_slots, float* o, float* workspace, int max_runs,
+                     const SrShape& s, hipStream_t stream);
+long sr_chunks_workspace(int rule, int Tn, int H);

@@ -588,6 +588,7 @@ static int sr_tokens_launch(const T* x, const float* taps, const float* conv_bia
   return 0;
 }
 
+static long sr_pad8(long n) { return (n + 7) / 8 * 8; }
 static long sr_pad4(long n) { return (n + 3) / 4 * 4; }  // parts of the scratch memory start at 16-byte boundaries
 
 template <typename T, int RULE>
@@ -606,7 +607,7 @@ static int sr_runs_launch(const T* x, const float* taps, const float* conv_bias,
   sr_prepare_kernel<T, RULE><<<s.Tn, 256, 0, stream>>>(x, u, a, b, a_bias, rate, state, token_slots, positions, scal, s);
   if (lev_check_launch("state recurrence (prepare)")) return -1;
   if (sizeof(T) == 2 && use_mfma) {
-    if (sr_chunks_launch(RULE, (const bf16_t*)(const void*)u, scal, state, token_slots, o, max_runs, s, stream)) return -1;
+    if (sr_chunks_launch(RULE, (const bf16_t*)(const void*)u, scal, state, token_slots, o, reinterpret_cast<float*>(u + sr_pad8((long)s.Tn * s.C)), max_runs, s, stream)) return -1;
     sr_finish_launch<T, RULE>(o, u, skip, gate, norm_w, token_slots, out, norm_groups, s, stream);
     return lev_check_launch("state recurrence (norm)");
   }
@@ -620,10 +621,12 @@ static int sr_runs_launch(const T* x, const float* taps, const float* conv_bias,
   return lev_check_launch("state recurrence (norm)");
 }
 
-// scratch memory in bytes. Steps with runs: o [Tn][H][dv], the scalars, the convolution's output; steps of single tokens: o of the rule SSD
-extern "C" long lev_state_recurrence_workspace(int Tn, int H, int G, int dv, int C, int runs, int dtype) {
+// scratch memory in bytes. Steps with runs: o [Tn][H][dv], the scalars, the convolution's output, bfloat16: the chunks' matrices; steps of single tokens: o of the rule SSD
+extern "C" long lev_state_recurrence_workspace(int rule, int Tn, int H, int G, int dv, int C, int runs, int dtype) {
   const long o = sr_pad4((long)Tn * H * dv) * 4;
-  return runs ? o + sr_pad4((long)Tn * (2L * H + 2L * G)) * 4 + (long)Tn * C * (dtype == LEV_F32 ? 4 : 2) : o;
+  return runs ? o + sr_pad4((long)Tn * (2L * H + 2L * G)) * 4 + sr_pad8((long)Tn * C) * (dtype == LEV_F32 ? 4 : 2) +
+                    (dtype == LEV_F32 ? 0 : sr_chunks_workspace(rule, Tn, H) * 4)
+              : o;
 }
 
 extern "C" int lev_state_recurrence(int rule, const void* x, long x_stride, const float* taps, const float* conv_bias, const void* a, long a_stride,

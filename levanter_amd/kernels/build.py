@@ -310,7 +310,7 @@ register_unit("core", ["errors.hip", "elementwise.hip", "layer_ops.hip", "gemm_s
     "lev_token_gate": [_P, _L, _P, _P, _P, _I, _I, _I, _P],
     "lev_projection_norm_rotate": [_P, _L, _I, _P, _L, _I, _I, _P, _L, _I, _F, _I, _I, _P, _P, _P, _I, _I, _P, _P, _P, _P, _I, _I, _I, _P],
     "lev_state_recurrence": [_I, _P, _L, _P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _P, _P, _L, _P, _P, _P, _L, _P] + [_I] * 12 + [_F, _F, _F, _I, _I, _P],
-    "lev_state_recurrence_workspace": [_I] * 7,
+    "lev_state_recurrence_workspace": [_I] * 8,
     "lev_gla_tokens": [_P, _P, _L, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _I, _I, _I, _I, _F, _F, _F, _I, _I, _P],
     "lev_gla_scan": [_P, _P, _L, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _P, _I, _I, _I, _I, _I, _F, _F, _F, _I, _I, _P],
     "lev_gla_scan_workspace": [_I, _I, _I, _I],

@@ -1019,7 +1019,7 @@ class HipKernels:
         for t in (token_slots, positions):
             _req(t.dtype == torch.int32 and t.numel() == T, "state recurrence: one int32 slot and position per token")
         runs = 0 if max_runs is None else max(1, min(int(max_runs), T))
-        ws = torch.empty(self.lib.lev_state_recurrence_workspace(T, H, G, dv, C, int(runs > 0), _DT[dt]), dtype=torch.uint8, device=x.device)
+        ws = torch.empty(self.lib.lev_state_recurrence_workspace(self.STATE_RULES[rule], T, H, G, dv, C, int(runs > 0), _DT[dt]), dtype=torch.uint8, device=x.device)
         self._check(self.lib.lev_state_recurrence(
             self.STATE_RULES[rule], _ptr(x), _rows(x, "state recurrence: x"), _ptr(taps), _ptr(conv_bias), _ptr(a), _rows(a, "state recurrence: a"), _ptr(b),
             _rows(b, "state recurrence: b") if b is not None else H, _ptr(a_bias), _ptr(rate), _ptr(skip), _ptr(gate), _rows(gate, "state recurrence: gate"),
