@@ -886,12 +886,12 @@ projection_norm_rotate_kernel(T* __restrict__ q, long q_stride, int H, T* __rest
   };
   T ra[PNR_KEEP], rb[PNR_KEEP];
   float w0[PNR_KEEP], w1[PNR_KEEP];
+  int e0[PNR_KEEP], e1[PNR_KEEP], pair[PNR_KEEP];
 #pragma unroll
   for (int m = 0; m < PNR_KEEP; ++m) {
-    int d0, d1;
-    place(min(tid + 256 * m, total - 1), d0, d1);
-    ra[m] = row[d0], rb[m] = row[d1];
-    w0[m] = w[d0], w1[m] = w[d1];
+    pair[m] = place(min(tid + 256 * m, total - 1), e0[m], e1[m]);
+    ra[m] = row[e0[m]], rb[m] = row[e1[m]];
+    w0[m] = w[e0[m]], w1[m] = w[e1[m]];
   }
   if (n_pairs) {  // the angles are the same for every head
     const float pos = (float)positions[t];
@@ -901,9 +901,7 @@ projection_norm_rotate_kernel(T* __restrict__ q, long q_stride, int H, T* __rest
 #pragma unroll
   for (int m = 0; m < PNR_KEEP; ++m) {
     if (tid + 256 * m >= total) continue;
-    int d0, d1;
-    place(tid + 256 * m, d0, d1);
-    const float a = to_float<T>(ra[m]), b = d1 != d0 ? to_float<T>(rb[m]) : 0.f;
+    const float a = to_float<T>(ra[m]), b = e1[m] != e0[m] ? to_float<T>(rb[m]) : 0.f;
     ss = fmaf(a, a, fmaf(b, b, ss));
   }
   for (int it = tid + 256 * PNR_KEEP; it < total; it += 256) {
@@ -924,9 +922,7 @@ projection_norm_rotate_kernel(T* __restrict__ q, long q_stride, int H, T* __rest
       row[e] = from_float<T>(val);
     }
   };
-  auto finish = [&](int it, float a, float b, float wa, float wb) {
-    int d0, d1;
-    const int i = place(it, d0, d1);
+  auto finish = [&](int i, int d0, int d1, float a, float b, float wa, float wb) {
     a = a * r * wa;
     if (i < n_pairs) {
       b = b * r * wb;
@@ -939,11 +935,124 @@ projection_norm_rotate_kernel(T* __restrict__ q, long q_stride, int H, T* __rest
   };
 #pragma unroll
   for (int m = 0; m < PNR_KEEP; ++m)
-    if (tid + 256 * m < total) finish(tid + 256 * m, to_float<T>(ra[m]), to_float<T>(rb[m]), w0[m], w1[m]);
+    if (tid + 256 * m < total) finish(pair[m], e0[m], e1[m], to_float<T>(ra[m]), to_float<T>(rb[m]), w0[m], w1[m]);
   for (int it = tid + 256 * PNR_KEEP; it < total; it += 256) {
     int d0, d1;
+    const int i = place(it, d0, d1);
+    finish(i, d0, d1, to_float<T>(row[d0]), to_float<T>(row[d1]), w[d0], w[d1]);
+  }
+}
+
+// The same with four neighbouring dimensions at a time (8-byte or 16-byte accesses), for the rotate-half layout (or none): n_pairs and the
+// strides multiples of 4. The sums and results are formed element by element as above.
+template <typename T>
+struct __attribute__((aligned(4 * sizeof(T)))) PnrQuad {
+  T v[4];
+};
+#define PNR_QUADS 4  // items that a thread keeps in registers
+template <typename T>
+__global__ void __launch_bounds__(256)
+projection_norm_rotate_quad_kernel(T* __restrict__ q, long q_stride, int H, T* __restrict__ k, long k_stride, int G, int hd, const T* __restrict__ v,
+                                   long v_stride, int vd, float eps, int norm_dim_q, int norm_dim_k, const float* __restrict__ wq,
+                                   const float* __restrict__ wk, const float* __restrict__ freqs, int n_pairs, const int* __restrict__ positions,
+                                   T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ dest, int PS) {
+  __shared__ float red[4];
+  __shared__ __attribute__((aligned(16))) float s_sin[PNR_MAX_PAIRS], s_cos[PNR_MAX_PAIRS];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int dst = k_pages ? dest[t] : 0, page = max(dst, 0) / max(PS, 1), off = k_pages ? max(dst, 0) % PS : 0;
+  if (blockIdx.y == 2) {  // values: single tokens only
+    if (dst < 0) return;
+    for (int e = tid; e < G * vd; e += 256) v_pages[((size_t)page * G * vd + e) * PS + off] = v[(size_t)t * v_stride + e];
+    return;
+  }
+  const bool is_q = blockIdx.y == 0;
+  const int heads = is_q ? H : G;
+  T* row = is_q ? q + (size_t)t * q_stride : k + (size_t)t * k_stride;
+  const float* w = is_q ? wq : wk;
+  const int items = (hd - n_pairs) / 4, total = heads * items;  // of a head: four pairs each, then four dimensions that do not turn each
+  auto place = [&](int it, int& d0, int& d1) {
+    const int head = it / items, i = (it - head * items) * 4;
+    d0 = head * hd + (i < n_pairs ? i : i + n_pairs);
+    d1 = i < n_pairs ? d0 + n_pairs : d0;
+    return i;
+  };
+  PnrQuad<T> ra[PNR_QUADS], rb[PNR_QUADS];
+  float4 w0[PNR_QUADS], w1[PNR_QUADS];
+#pragma unroll
+  for (int m = 0; m < PNR_QUADS; ++m) {
+    if (256 * m >= total) break;  // the whole workgroup
+    int d0, d1;
+    place(min(tid + 256 * m, total - 1), d0, d1);
+    ra[m] = *reinterpret_cast<const PnrQuad<T>*>(row + d0), rb[m] = *reinterpret_cast<const PnrQuad<T>*>(row + d1);
+    w0[m] = *reinterpret_cast<const float4*>(w + d0), w1[m] = *reinterpret_cast<const float4*>(w + d1);
+  }
+  if (n_pairs) {  // the angles are the same for every head
+    const float pos = (float)positions[t];
+    for (int i = tid; i < n_pairs; i += 256) sincosf(pos * freqs[i], &s_sin[i], &s_cos[i]);
+  }
+  float ss = 0.f;
+  auto add = [&](const PnrQuad<T>& a, const PnrQuad<T>& b, bool both) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float x = to_float<T>(a.v[e]), y = both ? to_float<T>(b.v[e]) : 0.f;
+      ss = fmaf(x, x, fmaf(y, y, ss));
+    }
+  };
+#pragma unroll
+  for (int m = 0; m < PNR_QUADS; ++m) {
+    if (tid + 256 * m >= total) break;
+    int d0, d1;
+    place(tid + 256 * m, d0, d1);
+    add(ra[m], rb[m], d1 != d0);
+  }
+  for (int it = tid + 256 * PNR_QUADS; it < total; it += 256) {
+    int d0, d1;
     place(it, d0, d1);
-    finish(it, to_float<T>(row[d0]), to_float<T>(row[d1]), w[d0], w[d1]);
+    add(*reinterpret_cast<const PnrQuad<T>*>(row + d0), *reinterpret_cast<const PnrQuad<T>*>(row + d1), d1 != d0);
+  }
+  ss = block_sum<256>(ss, red);  // its barriers also stand between the table of angles and its readers
+  const float r = 1.0f / sqrtf(ss / (float)(is_q ? norm_dim_q : norm_dim_k) + eps);
+  if (!is_q && dst < 0) return;
+  T* kd = is_q || !k_pages ? nullptr : k_pages + (size_t)page * G * hd * PS;
+  auto put = [&](int e, const float (&val)[4]) {
+    PnrQuad<T> x;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) x.v[i] = from_float<T>(val[i]);
+    T* to = row + e;
+    if (kd) {
+      const int head = e / hd, d = e - head * hd;  // four of a chunk of 8
+      to = kd + (size_t)head * hd * PS + ((size_t)(d >> 3) * PS + off) * 8 + (d & 7);
+    }
+    *reinterpret_cast<PnrQuad<T>*>(to) = x;
+  };
+  auto finish = [&](int it, const PnrQuad<T>& a, const PnrQuad<T>& b, const float4& wa, const float4& wb) {
+    int d0, d1;
+    const int i = place(it, d0, d1);
+    const float wa4[4] = {wa.x, wa.y, wa.z, wa.w}, wb4[4] = {wb.x, wb.y, wb.z, wb.w};
+    float lo[4], hi[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) lo[e] = to_float<T>(a.v[e]) * r * wa4[e], hi[e] = to_float<T>(b.v[e]) * r * wb4[e];
+    if (i < n_pairs) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float x = lo[e], y = hi[e], sn = s_sin[i + e], cs = s_cos[i + e];
+        lo[e] = x * cs - y * sn;
+        hi[e] = y * cs + x * sn;
+      }
+      put(d1, hi);
+    }
+    put(d0, lo);
+  };
+#pragma unroll
+  for (int m = 0; m < PNR_QUADS; ++m) {
+    if (tid + 256 * m >= total) break;
+    finish(tid + 256 * m, ra[m], rb[m], w0[m], w1[m]);
+  }
+  for (int it = tid + 256 * PNR_QUADS; it < total; it += 256) {
+    int d0, d1;
+    place(it, d0, d1);
+    finish(it, *reinterpret_cast<const PnrQuad<T>*>(row + d0), *reinterpret_cast<const PnrQuad<T>*>(row + d1), *reinterpret_cast<const float4*>(w + d0),
+           *reinterpret_cast<const float4*>(w + d1));
   }
 }
 
@@ -959,6 +1068,20 @@ extern "C" int lev_projection_norm_rotate(void* q, long q_stride, int H, void* k
   LEV_REQUIRE(dtype == LEV_F32 || dtype == LEV_BF16, "projection_norm_rotate: unknown dtype %d", dtype);
   if (T == 0) return 0;
   const dim3 grid(T, k_pages ? 3 : 2);
+  const uintptr_t a4 = dtype == LEV_F32 ? 15 : 7;
+  const bool quad = (half || n_pairs == 0) && n_pairs % 4 == 0 && q_stride % 4 == 0 && k_stride % 4 == 0 && (((uintptr_t)wq | (uintptr_t)wk) & 15) == 0 &&
+                    (((uintptr_t)q | (uintptr_t)k | (uintptr_t)k_pages) & a4) == 0;
+  if (quad) {
+    if (dtype == LEV_F32)
+      projection_norm_rotate_quad_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, H, (float*)k, k_stride, G, hd, (const float*)v, v_stride, vd, eps,
+                                                                         norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, positions, (float*)k_pages,
+                                                                         (float*)v_pages, dest, PS);
+    else
+      projection_norm_rotate_quad_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)q, q_stride, H, (bf16_t*)k, k_stride, G, hd, (const bf16_t*)v, v_stride,
+                                                                          vd, eps, norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, positions,
+                                                                          (bf16_t*)k_pages, (bf16_t*)v_pages, dest, PS);
+    return lev_check_launch("projection_norm_rotate (quads)");
+  }
   if (dtype == LEV_F32)
     projection_norm_rotate_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, H, (float*)k, k_stride, G, hd, (const float*)v, v_stride, vd, eps,
                                                                   norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, half, positions, (float*)k_pages,

@@ -21,6 +21,10 @@
 // matrix cores: token by token); norm and gate.
 #include "state_recurrence.h"
 
+// the activation behind the convolution: what is rounded to bfloat16 takes the hardware's exponential and reciprocal (about 1 ulp each)
+template <typename T>
+__device__ __forceinline__ float sr_conv_silu(float x) { return sizeof(T) == 2 ? lev_sigmoid_mul(x, -1.4426950408889634f * x) : sr_silu(x); }
+
 // ---- the convolution of a step with runs ----------------------------------------------------------------------------------
 // A thread takes SR_CT tokens of one channel; with K <= 4 their inputs and the three before them are held in registers.
 #define SR_CT 8
@@ -52,7 +56,7 @@ sr_conv_kernel(const T* __restrict__ x, const float* __restrict__ taps, const fl
           v = pos - k >= 0 ? state[(size_t)slot * s.slot_stride + (size_t)((pos - k) % K) * C + c] : 0.f;
         acc = fmaf(tap[k], v, acc);
       }
-      u[(size_t)t * C + c] = from_float<T>(slot < 0 ? 0.f : sr_silu(acc));
+      u[(size_t)t * C + c] = from_float<T>(slot < 0 ? 0.f : sr_conv_silu<T>(acc));
     }
   } else {
     for (int i = 0; i < SR_CT && t0 + i < s.Tn; ++i) {
@@ -64,7 +68,7 @@ sr_conv_kernel(const T* __restrict__ x, const float* __restrict__ taps, const fl
         else if (pos - k >= 0) v = state[(size_t)slot * s.slot_stride + (size_t)((pos - k) % K) * C + c];
         acc = fmaf(taps[(size_t)c * K + K - 1 - k], v, acc);
       }
-      u[(size_t)t * C + c] = from_float<T>(slot < 0 ? 0.f : sr_silu(acc));
+      u[(size_t)t * C + c] = from_float<T>(slot < 0 ? 0.f : sr_conv_silu<T>(acc));
     }
   }
 }
@@ -113,7 +117,7 @@ sr_conv_quad_kernel(const T* __restrict__ x, const float* __restrict__ taps, con
     }
     SrQuad<T> w;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) w.v[e] = from_float<T>(slot < 0 ? 0.f : sr_silu(acc[e]));
+    for (int e = 0; e < 4; ++e) w.v[e] = from_float<T>(slot < 0 ? 0.f : sr_conv_silu<T>(acc[e]));
     *reinterpret_cast<SrQuad<T>*>(u + (size_t)t * C + c) = w;
   }
 }
@@ -420,7 +424,7 @@ sr_token_kernel(const T* __restrict__ x, const float* __restrict__ taps, const f
         if (k < K && pos - k >= 0) acc[n] = fmaf(tap[n][k], old[n][k - 1], acc[n]);
       for (int k = 4; k < K; ++k)
         if (pos - k >= 0) acc[n] = fmaf(taps[(size_t)c * K + K - 1 - k], ring[(size_t)((pos - k) % K) * C + c], acc[n]);
-      const float val = in ? to_float<T>(from_float<T>(sr_silu(acc[n]))) : 0.f;
+      const float val = in ? to_float<T>(from_float<T>(sr_conv_silu<T>(acc[n]))) : 0.f;
       if (tid + NT * n < DVM + 2 * DKM) {
         if (in && (which == 0 || h % rep == 0)) ring[(size_t)(pos % K) * C + c] = cf;
         if (which == 0) s_v[i] = val;
