@@ -5,6 +5,7 @@ from .nakurax import NakuraxConfig
 from .tativik import TativikConfig
 from .kegetar import KegetarConfig
 from .lelatar import LelatarConfig
+from .kelasun import KelasunConfig
 from .engine_config import InferenceEngineConfig
 
-__all__ = ["ConfigError", "LmConfig", "Gpt2Config", "ZederaxConfig", "NakuraxConfig", "TativikConfig", "KegetarConfig", "LelatarConfig", "InferenceEngineConfig"]
+__all__ = ["ConfigError", "LmConfig", "Gpt2Config", "ZederaxConfig", "NakuraxConfig", "TativikConfig", "KegetarConfig", "LelatarConfig", "KelasunConfig", "InferenceEngineConfig"]

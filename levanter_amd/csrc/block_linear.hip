@@ -1,6 +1,7 @@
 // A block-diagonal linear map: the input row is B parts of n_in columns, part b goes through its own matrix
 // w[b] ([n_out][n_in], each output's inputs contiguous) and gives part b of the output row:
 //     out[t][b * n_out + o] = sum_i w[b][o][i] * a[t][b * n_in + i] + bias[b * n_out + o]
+// times sigmoid(gate[t][b * n_out + o]) where there is a gate (of the weights' type; an output gate per element).
 // (per-head projections of an attention with a latent, the gates of a recurrence that are square matrices per block).
 // Plain 32-bit FMA for the few rows of a decoding step; the launcher sends prompt-sized row counts to the matrix
 // products, block by block. One wave per output column and tile of TT rows: the lanes share the inputs of the column
@@ -13,7 +14,7 @@
 template <typename TA, typename TW, typename TO>
 __global__ void __launch_bounds__(256)
 block_linear_kernel(const TA* __restrict__ a, long a_stride, const TW* __restrict__ w, const float* __restrict__ bias, TO* __restrict__ out,
-                    long o_stride, int T, int B, int n_in, int n_out) {
+                    long o_stride, const TW* __restrict__ gate, long g_stride, int T, int B, int n_in, int n_out) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const long col = (long)blockIdx.x * 4 + wave;  // over B * n_out
   if (col >= (long)B * n_out) return;
@@ -35,27 +36,31 @@ block_linear_kernel(const TA* __restrict__ a, long a_stride, const TW* __restric
 #pragma unroll
   for (int tt = 0; tt < BL_TT; ++tt) {
     const float s = wave_sum(acc[tt]);
-    if (lane == 0 && t0 + tt < T) out[(size_t)(t0 + tt) * o_stride + col] = from_float<TO>(s + bv);
+    if (lane == 0 && t0 + tt < T) {
+      const float gv = gate ? 1.0f / (1.0f + expf(-to_float<TW>(gate[(size_t)(t0 + tt) * g_stride + col]))) : 1.0f;
+      out[(size_t)(t0 + tt) * o_stride + col] = from_float<TO>((s + bv) * gv);
+    }
   }
 }
 
 template <typename TA, typename TW, typename TO>
-static void block_linear_launch(const void* a, long a_stride, const void* w, const float* bias, void* out, long o_stride, int T, int B,
-                                int n_in, int n_out, hipStream_t stream) {
+static void block_linear_launch(const void* a, long a_stride, const void* w, const float* bias, void* out, long o_stride,
+                                const void* gate, long g_stride, int T, int B, int n_in, int n_out, hipStream_t stream) {
   dim3 grid((unsigned)(((long)B * n_out + 3) / 4), (T + BL_TT - 1) / BL_TT);
-  block_linear_kernel<TA, TW, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, (const TW*)w, bias, (TO*)out, o_stride, T, B, n_in, n_out);
+  block_linear_kernel<TA, TW, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, (const TW*)w, bias, (TO*)out, o_stride, (const TW*)gate, g_stride, T, B,
+                                                         n_in, n_out);
 }
 
-extern "C" int lev_block_linear(const void* a, long a_stride, const void* w, const float* bias, void* out, long o_stride, int T, int B,
-                                int n_in, int n_out, int a_dtype, int w_dtype, int out_dtype, hipStream_t stream) {
+extern "C" int lev_block_linear(const void* a, long a_stride, const void* w, const float* bias, void* out, long o_stride, const void* gate,
+                                long g_stride, int T, int B, int n_in, int n_out, int a_dtype, int w_dtype, int out_dtype, hipStream_t stream) {
   LEV_REQUIRE(T >= 0 && B > 0 && n_in > 0 && n_out > 0, "block_linear: bad sizes T=%d blocks=%d in=%d out=%d", T, B, n_in, n_out);
   LEV_REQUIRE(a && w && out, "block_linear: a tensor is missing");
-  LEV_REQUIRE(a_stride >= (long)B * n_in && o_stride >= (long)B * n_out, "block_linear: row strides are smaller than the rows");
+  LEV_REQUIRE(a_stride >= (long)B * n_in && o_stride >= (long)B * n_out && (!gate || g_stride >= (long)B * n_out), "block_linear: row strides are smaller than the rows");
   LEV_REQUIRE((T + BL_TT - 1) / BL_TT <= 65535, "block_linear: too many rows (%d) for this kernel", T);
   if (T == 0) return 0;
 #define BL_CASE(A, W, O, TA, TW, TO)                                                                                   \
   if (a_dtype == A && w_dtype == W && out_dtype == O) {                                                                \
-    block_linear_launch<TA, TW, TO>(a, a_stride, w, bias, out, o_stride, T, B, n_in, n_out, stream);                 \
+    block_linear_launch<TA, TW, TO>(a, a_stride, w, bias, out, o_stride, gate, g_stride, T, B, n_in, n_out, stream); \
     return lev_check_launch("block_linear");                                                                          \
   }
   BL_CASE(LEV_F32, LEV_F32, LEV_F32, float, float, float)
@@ -93,7 +98,7 @@ __device__ __forceinline__ blm_u32x4 blm_load8(const float* p) {
 template <typename TA, typename TO, int BLM_NT>
 __global__ void __launch_bounds__(256)
 block_linear_mfma_kernel(const TA* __restrict__ a, long a_stride, const bf16_t* __restrict__ w, const float* __restrict__ bias,
-                         TO* __restrict__ out, long o_stride, int T, int n_in, int n_out, int col_sets) {
+                         TO* __restrict__ out, long o_stride, const bf16_t* __restrict__ gate, long g_stride, int T, int n_in, int n_out, int col_sets) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 15, g = lane >> 4;
   const int t0 = (blockIdx.x * 4 + wave) * 16;
   if (t0 >= T) return;  // the whole wave
@@ -125,17 +130,21 @@ block_linear_mfma_kernel(const TA* __restrict__ a, long a_stride, const bf16_t* 
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int o = o0 + 16 * nt + 4 * g + r;
-      if (o < n_out) out[(size_t)t * o_stride + (size_t)b * n_out + o] = from_float<TO>(acc[nt][r] + (bias ? bias[(size_t)b * n_out + o] : 0.f));
+      if (o < n_out) {
+        const size_t c = (size_t)b * n_out + o;
+        const float gv = gate ? 1.0f / (1.0f + expf(-bf16_to_float(gate[(size_t)t * g_stride + c]))) : 1.0f;
+        out[(size_t)t * o_stride + c] = from_float<TO>((acc[nt][r] + (bias ? bias[c] : 0.f)) * gv);
+      }
     }
 }
 
-extern "C" int lev_block_linear_mfma(const void* a, long a_stride, const void* w, const float* bias, void* out, long o_stride, int T, int B,
-                                     int n_in, int n_out, int a_dtype, int out_dtype, hipStream_t stream) {
+extern "C" int lev_block_linear_mfma(const void* a, long a_stride, const void* w, const float* bias, void* out, long o_stride, const void* gate,
+                                     long g_stride, int T, int B, int n_in, int n_out, int a_dtype, int out_dtype, hipStream_t stream) {
   LEV_REQUIRE(T >= 0 && B > 0 && n_in > 0 && n_out > 0, "block_linear: bad sizes T=%d blocks=%d in=%d out=%d", T, B, n_in, n_out);
   LEV_REQUIRE(a && w && out, "block_linear: a tensor is missing");
   LEV_REQUIRE(n_in % 8 == 0 && a_stride % 8 == 0 && ((uintptr_t)a & 15) == 0 && ((uintptr_t)w & 15) == 0,
               "block_linear (matrix cores): inputs of %d a block and a row stride of %ld must be multiples of 8, operands 16-byte aligned", n_in, a_stride);
-  LEV_REQUIRE(a_stride >= (long)B * n_in && o_stride >= (long)B * n_out, "block_linear: row strides are smaller than the rows");
+  LEV_REQUIRE(a_stride >= (long)B * n_in && o_stride >= (long)B * n_out && (!gate || g_stride >= (long)B * n_out), "block_linear: row strides are smaller than the rows");
   if (T == 0) return 0;
   const int nt = T <= 32 ? 1 : 4;
   const int col_sets = (n_out + 16 * nt - 1) / (16 * nt);
@@ -144,10 +153,10 @@ extern "C" int lev_block_linear_mfma(const void* a, long a_stride, const void* w
 #define BLM_CASE(A, O, TA, TO)                                                                                                     \
   if (a_dtype == A && out_dtype == O) {                                                                                            \
     if (nt == 1)                                                                                                                   \
-      block_linear_mfma_kernel<TA, TO, 1><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, (const bf16_t*)w, bias, (TO*)out, o_stride, T, n_in, \
+      block_linear_mfma_kernel<TA, TO, 1><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, (const bf16_t*)w, bias, (TO*)out, o_stride, (const bf16_t*)gate, g_stride, T, n_in, \
                                                                    n_out, col_sets);                                               \
     else                                                                                                                           \
-      block_linear_mfma_kernel<TA, TO, 4><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, (const bf16_t*)w, bias, (TO*)out, o_stride, T, n_in, \
+      block_linear_mfma_kernel<TA, TO, 4><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, (const bf16_t*)w, bias, (TO*)out, o_stride, (const bf16_t*)gate, g_stride, T, n_in, \
                                                                    n_out, col_sets);                                               \
     return lev_check_launch("block_linear (matrix cores)");                                                                       \
   }

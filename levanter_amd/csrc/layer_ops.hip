@@ -302,14 +302,14 @@ extern "C" int lev_norm_write_latent(void* c, long c_stride, int R, int norm_dim
 // The same for a latent with a rotated key part behind it, and the rotation of the queries, in one launch (steps of single
 // tokens). A token's row `kv` holds [c (R) | k_rot (DR)]: c becomes its RMS norm with the weight `w` (mean of squares over
 // norm_dim), in place; k_rot has dimension i < n_pairs paired with dimension i + n_pairs and each pair turned by
-// positions[t] * freqs[i], in place; the key pages (one key head of R + DR) take [c | k_rot], the value pages (one head of
+// positions[t] * freqs[i] (cosine and sine times `magnitude`), in place; the key pages (one key head of R + DR) take [c | k_rot], the value pages (one head of
 // R) take c. Every head of `q` (HQ heads of q_head elements) has the vector that starts q_off elements into it turned the
 // same way. The arithmetic is that of head_prepare, rotary_half and kv_write, one after the other.
 template <typename T>
 __global__ void __launch_bounds__(256)
 latent_rope_write_kernel(T* __restrict__ kv, long kv_stride, int R, int DR, int norm_dim, float eps, const float* __restrict__ w,
                          T* __restrict__ q, long q_stride, int HQ, int q_head, int q_off, int n_pairs, const float* __restrict__ freqs,
-                         const int* __restrict__ positions, T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ dest,
+                         const int* __restrict__ positions, float magnitude, T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ dest,
                          int PS) {
   __shared__ float red[4];
   const int t = blockIdx.x;
@@ -340,6 +340,7 @@ latent_rope_write_kernel(T* __restrict__ kv, long kv_stride, int R, int DR, int 
     if (i < n_pairs) {
       float sn, cs;
       sincosf(p * freqs[i], &sn, &cs);
+      sn *= magnitude, cs *= magnitude;
       const float a = to_float<T>(row[R + i]), b = to_float<T>(row[R + i + n_pairs]);
       const T lo = from_float<T>(a * cs - b * sn), hi = from_float<T>(b * cs + a * sn);
       row[R + i] = lo;
@@ -361,6 +362,7 @@ latent_rope_write_kernel(T* __restrict__ kv, long kv_stride, int R, int DR, int 
       T* v = q + (size_t)t * q_stride + (size_t)head * q_head + q_off;
       float sn, cs;
       sincosf(p * freqs[i], &sn, &cs);
+      sn *= magnitude, cs *= magnitude;
       const float a = to_float<T>(v[i]), b = to_float<T>(v[i + n_pairs]);
       v[i] = from_float<T>(a * cs - b * sn);
       v[i + n_pairs] = from_float<T>(b * cs + a * sn);
@@ -369,8 +371,8 @@ latent_rope_write_kernel(T* __restrict__ kv, long kv_stride, int R, int DR, int 
 }
 
 extern "C" int lev_latent_rope_write(void* kv, long kv_stride, int R, int DR, int norm_dim, float eps, const float* w, void* q, long q_stride,
-                                     int HQ, int q_head, int q_off, int n_pairs, const float* freqs, const int* positions, void* k_pages,
-                                     void* v_pages, const int* dest, int PS, int T, int dtype, hipStream_t stream) {
+                                     int HQ, int q_head, int q_off, int n_pairs, const float* freqs, const int* positions, float magnitude,
+                                     void* k_pages, void* v_pages, const int* dest, int PS, int T, int dtype, hipStream_t stream) {
   LEV_REQUIRE(T >= 0 && R > 0 && R % 8 == 0 && DR >= 0 && DR % 8 == 0 && norm_dim > 0 && norm_dim <= R && kv_stride >= R + DR,
               "latent_rope_write: bad sizes T=%d R=%d of %d, rotated part %d", T, R, norm_dim, DR);
   LEV_REQUIRE(n_pairs >= 0 && 2 * n_pairs <= DR && (n_pairs == 0 || (freqs && positions)), "latent_rope_write: %d pairs do not fit a rotated part of %d", n_pairs, DR);
@@ -381,10 +383,10 @@ extern "C" int lev_latent_rope_write(void* kv, long kv_stride, int R, int DR, in
   if (T == 0) return 0;
   if (dtype == LEV_F32)
     latent_rope_write_kernel<float><<<T, 256, 0, stream>>>((float*)kv, kv_stride, R, DR, norm_dim, eps, w, (float*)q, q_stride, HQ, q_head, q_off, n_pairs,
-                                                          freqs, positions, (float*)k_pages, (float*)v_pages, dest, PS);
+                                                          freqs, positions, magnitude, (float*)k_pages, (float*)v_pages, dest, PS);
   else
     latent_rope_write_kernel<bf16_t><<<T, 256, 0, stream>>>((bf16_t*)kv, kv_stride, R, DR, norm_dim, eps, w, (bf16_t*)q, q_stride, HQ, q_head, q_off,
-                                                           n_pairs, freqs, positions, (bf16_t*)k_pages, (bf16_t*)v_pages, dest, PS);
+                                                           n_pairs, freqs, positions, magnitude, (bf16_t*)k_pages, (bf16_t*)v_pages, dest, PS);
   return lev_check_launch("latent_rope_write");
 }
 
@@ -855,14 +857,18 @@ extern "C" int lev_token_gate_linear(const void* h, long h_stride, const void* w
 // head is paired with i + n_pairs, else 2i with 2i + 1; i < n_pairs, the rest of a head passes unrotated. Queries change in place. With
 // pages (steps of single tokens) keys and values go into them at dest[t] and stay as they are in k and v; without, keys change in place
 // and values are not touched. The arithmetic is the same either way. norm_dim_*: the projections' true sizes (heads may carry zeros).
+// temp_every > 0: the queries at position p are also multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1).
 #define PNR_KEEP 8
 #define PNR_MAX_PAIRS 512
+__device__ __forceinline__ float query_temperature(int pos, float coef, float every) {
+  return every > 0.f ? 1.0f + coef * logf(floorf((float)(pos + 1) / every) + 1.0f) : 1.0f;
+}
 template <typename T>
 __global__ void __launch_bounds__(256)
 projection_norm_rotate_kernel(T* __restrict__ q, long q_stride, int H, T* __restrict__ k, long k_stride, int G, int hd, const T* __restrict__ v,
                               long v_stride, int vd, float eps, int norm_dim_q, int norm_dim_k, const float* __restrict__ wq,
-                              const float* __restrict__ wk, const float* __restrict__ freqs, int n_pairs, int half, const int* __restrict__ positions,
-                              T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ dest, int PS) {
+                              const float* __restrict__ wk, const float* __restrict__ freqs, int n_pairs, int half, const int* __restrict__ positions, float temp_coef,
+                              float temp_every, T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ dest, int PS) {
   __shared__ float red[4], s_sin[PNR_MAX_PAIRS], s_cos[PNR_MAX_PAIRS];
   const int t = blockIdx.x, tid = threadIdx.x;
   const int dst = k_pages ? dest[t] : 0, page = max(dst, 0) / max(PS, 1), off = k_pages ? max(dst, 0) % PS : 0;
@@ -911,7 +917,8 @@ projection_norm_rotate_kernel(T* __restrict__ q, long q_stride, int H, T* __rest
     ss = fmaf(a, a, fmaf(b, b, ss));
   }
   ss = block_sum<256>(ss, red);  // its barriers also stand between the table of angles and its readers
-  const float r = 1.0f / sqrtf(ss / (float)(is_q ? norm_dim_q : norm_dim_k) + eps);
+  float r = 1.0f / sqrtf(ss / (float)(is_q ? norm_dim_q : norm_dim_k) + eps);
+  if (is_q && temp_every > 0.f) r *= query_temperature(positions[t], temp_coef, temp_every);
   if (!is_q && dst < 0) return;
   T* kd = is_q || !k_pages ? nullptr : k_pages + (size_t)page * G * hd * PS;
   auto put = [&](int e, float val) {
@@ -955,7 +962,7 @@ __global__ void __launch_bounds__(256)
 projection_norm_rotate_quad_kernel(T* __restrict__ q, long q_stride, int H, T* __restrict__ k, long k_stride, int G, int hd, const T* __restrict__ v,
                                    long v_stride, int vd, float eps, int norm_dim_q, int norm_dim_k, const float* __restrict__ wq,
                                    const float* __restrict__ wk, const float* __restrict__ freqs, int n_pairs, const int* __restrict__ positions,
-                                   T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ dest, int PS) {
+                                   float temp_coef, float temp_every, T* __restrict__ k_pages, T* __restrict__ v_pages, const int* __restrict__ dest, int PS) {
   __shared__ float red[4];
   __shared__ __attribute__((aligned(16))) float s_sin[PNR_MAX_PAIRS], s_cos[PNR_MAX_PAIRS];
   const int t = blockIdx.x, tid = threadIdx.x;
@@ -1011,7 +1018,8 @@ projection_norm_rotate_quad_kernel(T* __restrict__ q, long q_stride, int H, T* _
     add(*reinterpret_cast<const PnrQuad<T>*>(row + d0), *reinterpret_cast<const PnrQuad<T>*>(row + d1), d1 != d0);
   }
   ss = block_sum<256>(ss, red);  // its barriers also stand between the table of angles and its readers
-  const float r = 1.0f / sqrtf(ss / (float)(is_q ? norm_dim_q : norm_dim_k) + eps);
+  float r = 1.0f / sqrtf(ss / (float)(is_q ? norm_dim_q : norm_dim_k) + eps);
+  if (is_q && temp_every > 0.f) r *= query_temperature(positions[t], temp_coef, temp_every);
   if (!is_q && dst < 0) return;
   T* kd = is_q || !k_pages ? nullptr : k_pages + (size_t)page * G * hd * PS;
   auto put = [&](int e, const float (&val)[4]) {
@@ -1058,12 +1066,13 @@ projection_norm_rotate_quad_kernel(T* __restrict__ q, long q_stride, int H, T* _
 
 extern "C" int lev_projection_norm_rotate(void* q, long q_stride, int H, void* k, long k_stride, int G, int hd, const void* v, long v_stride, int vd,
                                           float eps, int norm_dim_q, int norm_dim_k, const float* wq, const float* wk, const float* freqs, int n_pairs,
-                                          int half, const int* positions, void* k_pages, void* v_pages, const int* dest, int PS, int T, int dtype,
-                                          hipStream_t stream) {
+                                          int half, const int* positions, float temp_coef, float temp_every, void* k_pages, void* v_pages,
+                                          const int* dest, int PS, int T, int dtype, hipStream_t stream) {
   LEV_REQUIRE(T >= 0 && H > 0 && G > 0 && hd > 0 && hd % 8 == 0, "projection_norm_rotate: bad sizes T=%d heads=%d/%d size=%d", T, H, G, hd);
   LEV_REQUIRE(q && k && wq && wk && norm_dim_q > 0 && norm_dim_q <= H * hd && norm_dim_k > 0 && norm_dim_k <= G * hd, "projection_norm_rotate: a tensor is missing or bad divisors");
   LEV_REQUIRE(q_stride >= (long)H * hd && k_stride >= (long)G * hd, "projection_norm_rotate: row strides are smaller than the heads");
   LEV_REQUIRE(n_pairs >= 0 && n_pairs <= PNR_MAX_PAIRS && 2 * n_pairs <= hd && (n_pairs == 0 || (freqs && positions)), "projection_norm_rotate: %d rotated pairs need frequencies, positions and a head of at least twice their number", n_pairs);
+  LEV_REQUIRE(temp_every <= 0.f || positions, "projection_norm_rotate: a temperature of the queries needs their positions");
   LEV_REQUIRE(!k_pages || (v && v_pages && dest && vd > 0 && PS > 0 && PS % 16 == 0 && v_stride >= (long)G * vd), "projection_norm_rotate: pages need values, destinations and a page size that is a multiple of 16");
   LEV_REQUIRE(dtype == LEV_F32 || dtype == LEV_BF16, "projection_norm_rotate: unknown dtype %d", dtype);
   if (T == 0) return 0;
@@ -1074,21 +1083,21 @@ extern "C" int lev_projection_norm_rotate(void* q, long q_stride, int H, void* k
   if (quad) {
     if (dtype == LEV_F32)
       projection_norm_rotate_quad_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, H, (float*)k, k_stride, G, hd, (const float*)v, v_stride, vd, eps,
-                                                                         norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, positions, (float*)k_pages,
+                                                                         norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, positions, temp_coef, temp_every, (float*)k_pages,
                                                                          (float*)v_pages, dest, PS);
     else
       projection_norm_rotate_quad_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)q, q_stride, H, (bf16_t*)k, k_stride, G, hd, (const bf16_t*)v, v_stride,
-                                                                          vd, eps, norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, positions,
+                                                                          vd, eps, norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, positions, temp_coef, temp_every,
                                                                           (bf16_t*)k_pages, (bf16_t*)v_pages, dest, PS);
     return lev_check_launch("projection_norm_rotate (quads)");
   }
   if (dtype == LEV_F32)
     projection_norm_rotate_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, H, (float*)k, k_stride, G, hd, (const float*)v, v_stride, vd, eps,
-                                                                  norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, half, positions, (float*)k_pages,
+                                                                  norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, half, positions, temp_coef, temp_every, (float*)k_pages,
                                                                   (float*)v_pages, dest, PS);
   else
     projection_norm_rotate_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)q, q_stride, H, (bf16_t*)k, k_stride, G, hd, (const bf16_t*)v, v_stride, vd, eps,
-                                                                   norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, half, positions, (bf16_t*)k_pages,
+                                                                   norm_dim_q, norm_dim_k, wq, wk, freqs, n_pairs, half, positions, temp_coef, temp_every, (bf16_t*)k_pages,
                                                                    (bf16_t*)v_pages, dest, PS);
   return lev_check_launch("projection_norm_rotate");
 }

@@ -1,8 +1,8 @@
 // A feed-forward made of many small experts of which every token uses a few (a mixture of experts), steered from the device:
 // no count ever goes to the host, so the launches depend on the number of tokens alone.
 //
-//   route     per token: scores s = sigmoid(z) of the router's logits z (float32 [T][E]), or with `softmax` the softmax of z over all
-//             E outputs; the choice goes by c = s + correction;
+//   route     per token: scores s of the router's logits z (float32 [T][E]): sigmoid(z) (scoring 0), the softmax of z over all E outputs
+//             (1) or z itself (2: the weights are then the softmax over the winners' s alone); the choice goes by c = s + correction;
 //             the experts form G equal groups of neighbours, a group's score is the sum of its `group_top` largest c, only the
 //             experts of the `keep` best groups can be chosen (the others count as -inf); the `top` largest c win (ties: the
 //             lower index); the weights are the winners' s (times 1 / their sum if `renormalize`), in the order of falling c.
@@ -11,7 +11,8 @@
 //             tile_rows is 16, or 64 for steps with many rows an expert (a wave then runs four row tiles on every weight
 //             fragment it loads).
 //   linear    for every tile: out[pos][o] = sum_k w[expert][o][k] a[row(pos)][k], row(pos) = the pair's token (gather) or pos
-//             itself; with glu the expert's matrix is [gate ; up] (2F rows) and out[pos][f] = act(gate_f) * up_f.
+//             itself, through the activation (none for the second product); with glu the expert's matrix is [gate ; up] (2F rows) and
+//             out[pos][f] = act(gate_f) * up_f.
 //             bfloat16 on the matrix cores (16x16x32): few tiles of 16 rows with K split over a workgroup's waves, many with a
 //             wave per tile, tiles of 64 rows with both operands staged through LDS; float32 in plain arithmetic. Workgroups
 //             beyond n_tiles return at once.
@@ -29,13 +30,13 @@
 // ---- route ------------------------------------------------------------------------------------
 __global__ void __launch_bounds__(64)
 moe_route_kernel(const float* __restrict__ z, long z_stride, const float* __restrict__ correction, int E, int G, int keep, int group_top, int top,
-                 int renormalize, int softmax, int* __restrict__ chosen, float* __restrict__ weights) {
+                 int renormalize, int scoring, int* __restrict__ chosen, float* __restrict__ weights) {
   __shared__ float s_s[MOE_MAX_E], c_s[MOE_MAX_E], g_s[MOE_MAX_E];
   __shared__ int sel[MOE_MAX_TOP];
   const int t = blockIdx.x, lane = threadIdx.x;
   const int per = E / G;
   float z_max = 0.f, inv_sum = 1.0f;
-  if (softmax) {
+  if (scoring == 1) {
     float mx = -INFINITY;
     for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[(size_t)t * z_stride + e]);
     z_max = wave_max(mx);
@@ -45,7 +46,7 @@ moe_route_kernel(const float* __restrict__ z, long z_stride, const float* __rest
   }
   for (int e = lane; e < E; e += 64) {
     const float ze = z[(size_t)t * z_stride + e];
-    const float s = softmax ? expf(ze - z_max) * inv_sum : 1.0f / (1.0f + expf(-ze));
+    const float s = scoring == 2 ? ze : scoring == 1 ? expf(ze - z_max) * inv_sum : 1.0f / (1.0f + expf(-ze));
     s_s[e] = s;
     c_s[e] = s + (correction ? correction[e] : 0.f);
   }
@@ -99,6 +100,17 @@ moe_route_kernel(const float* __restrict__ z, long z_stride, const float* __rest
     wsum += s_s[best_e];
     __syncthreads();
   }
+  if (scoring == 2) {  // every lane sums the same few numbers
+    float mx = -INFINITY, sum = 0.f;
+    for (int n = 0; n < top; ++n) mx = fmaxf(mx, s_s[sel[n]]);
+    for (int n = 0; n < top; ++n) sum += expf(s_s[sel[n]] - mx);
+    if (lane < top) {
+      const int e = sel[lane];
+      chosen[(size_t)t * top + lane] = e;
+      weights[(size_t)t * top + lane] = expf(s_s[e] - mx) / sum;
+    }
+    return;
+  }
   if (lane < top) {
     const int e = sel[lane];
     chosen[(size_t)t * top + lane] = e;
@@ -107,13 +119,14 @@ moe_route_kernel(const float* __restrict__ z, long z_stride, const float* __rest
 }
 
 extern "C" int lev_moe_route(const float* z, long z_stride, const float* correction, int T, int E, int G, int keep, int group_top, int top,
-                             int renormalize, int softmax, int* chosen, float* weights, hipStream_t stream) {
+                             int renormalize, int scoring, int* chosen, float* weights, hipStream_t stream) {
+  LEV_REQUIRE(scoring >= 0 && scoring <= 2, "experts: unknown scoring %d", scoring);
   LEV_REQUIRE(T >= 0 && E > 0 && E <= MOE_MAX_E, "experts: %d experts (at most %d)", E, MOE_MAX_E);
   LEV_REQUIRE(G > 0 && E % G == 0 && keep > 0 && keep <= G && group_top > 0, "experts: %d groups of %d experts, %d kept", G, E, keep);
   LEV_REQUIRE(top > 0 && top <= MOE_MAX_TOP && top <= keep * (E / G), "experts: %d experts a token out of %d that can be chosen (at most %d)", top, keep * (E / G), MOE_MAX_TOP);
   LEV_REQUIRE(z && chosen && weights && z_stride >= E, "experts: a tensor is missing");
   if (T == 0) return 0;
-  moe_route_kernel<<<T, 64, 0, stream>>>(z, z_stride, correction, E, G, keep, group_top, top, renormalize, softmax, chosen, weights);
+  moe_route_kernel<<<T, 64, 0, stream>>>(z, z_stride, correction, E, G, keep, group_top, top, renormalize, scoring, chosen, weights);
   return lev_check_launch("moe_route");
 }
 
@@ -197,6 +210,8 @@ moe_linear_plain_kernel(const T* __restrict__ a, long a_stride, const T* __restr
       const T* wu = wg + (size_t)F * K;
       for (int kk = 0; kk < K; ++kk) acc_up = fmaf(to_float<T>(wu[kk]), to_float<T>(ar[kk]), acc_up);
       acc = moe_act(acc, acc_up, act, limit, up_shift);
+    } else {
+      acc = lev_activate(acc, act);
     }
     out[(size_t)pos * o_stride + o] = from_float<TO>(acc);
   }
@@ -273,7 +288,7 @@ moe_linear_mfma_kernel(const bf16_t* __restrict__ a, long a_stride, const bf16_t
       for (int r = 0; r < 4; ++r) {
         const int o = o0 + 16 * nt + 4 * g + r;
         if (o < F)
-          out[(size_t)(first + 16 * rt + col) * o_stride + o] = from_float<TO>(GLU ? moe_act(acc[rt][nt][r], acc_up[rt][nt][r], act, limit, up_shift) : acc[rt][nt][r]);
+          out[(size_t)(first + 16 * rt + col) * o_stride + o] = from_float<TO>(GLU ? moe_act(acc[rt][nt][r], acc_up[rt][nt][r], act, limit, up_shift) : lev_activate(acc[rt][nt][r], act));
       }
   }
 }
@@ -328,7 +343,7 @@ moe_linear_splitk_kernel(const bf16_t* __restrict__ a, long a_stride, const bf16
       if (GLU) sum_up += part[q][1][r][lane];
     }
     const int o = o0 + 4 * g + r;
-    if (o < F) out[(size_t)(first + col) * o_stride + o] = from_float<TO>(GLU ? moe_act(sum, sum_up, act, limit, up_shift) : sum);
+    if (o < F) out[(size_t)(first + col) * o_stride + o] = from_float<TO>(GLU ? moe_act(sum, sum_up, act, limit, up_shift) : lev_activate(sum, act));
   }
 }
 
@@ -416,7 +431,7 @@ moe_linear_tile_kernel(const bf16_t* __restrict__ a, long a_stride, const bf16_t
       for (int r = 0; r < 4; ++r) {
         const int o = o0 + wave * 32 + 16 * nt + 4 * g + r;
         if (o < F)
-          out[(size_t)(first + 16 * rt + col) * o_stride + o] = from_float<TO>(GLU ? moe_act(acc[rt][nt][r], acc_up[rt][nt][r], act, limit, up_shift) : acc[rt][nt][r]);
+          out[(size_t)(first + 16 * rt + col) * o_stride + o] = from_float<TO>(GLU ? moe_act(acc[rt][nt][r], acc_up[rt][nt][r], act, limit, up_shift) : lev_activate(acc[rt][nt][r], act));
       }
   }
 }

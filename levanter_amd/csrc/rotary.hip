@@ -42,11 +42,11 @@ extern "C" int lev_rotary_pairs(void* q, long q_stride, int HQ, void* k, long k_
 
 // The same rotation in the "rotate half" layout: within a head, dimension i < n_pairs is paired with dimension i + n_pairs.
 // The rotated vector starts `offset` elements into each head of `head_stride` elements (a head may carry dimensions that
-// never turn ahead of it and behind it); one tensor at a time, in place.
+// never turn ahead of it and behind it); one tensor at a time, in place. `magnitude` as above.
 template <typename T>
 __global__ void __launch_bounds__(256)
 rotary_half_kernel(T* __restrict__ x, long x_stride, int H, int head_stride, int offset, int n_pairs, const float* __restrict__ freqs,
-                   const int* __restrict__ positions) {
+                   const int* __restrict__ positions, float magnitude) {
   const int t = blockIdx.x;
   const float p = (float)positions[t];
   const int items = H * n_pairs;
@@ -55,6 +55,7 @@ rotary_half_kernel(T* __restrict__ x, long x_stride, int H, int head_stride, int
     T* v = x + (size_t)t * x_stride + (size_t)head * head_stride + offset;
     float s, c;
     sincosf(p * freqs[i], &s, &c);
+    s *= magnitude, c *= magnitude;
     const float a = to_float<T>(v[i]), b = to_float<T>(v[i + n_pairs]);
     v[i] = from_float<T>(a * c - b * s);
     v[i + n_pairs] = from_float<T>(b * c + a * s);
@@ -62,7 +63,7 @@ rotary_half_kernel(T* __restrict__ x, long x_stride, int H, int head_stride, int
 }
 
 extern "C" int lev_rotary_half(void* x, long x_stride, int H, int head_stride, int offset, int n_pairs, const float* freqs, const int* positions,
-                               int T, int dtype, hipStream_t stream) {
+                               float magnitude, int T, int dtype, hipStream_t stream) {
   LEV_REQUIRE(T >= 0 && H > 0 && head_stride > 0 && offset >= 0 && n_pairs >= 0, "rotary: bad sizes T=%d heads=%d head=%d offset=%d", T, H, head_stride, offset);
   LEV_REQUIRE(offset + 2 * n_pairs <= head_stride, "rotary: %d pairs from element %d on do not fit a head of %d", n_pairs, offset, head_stride);
   LEV_REQUIRE(x && freqs && positions, "rotary: a tensor is missing");
@@ -70,8 +71,8 @@ extern "C" int lev_rotary_half(void* x, long x_stride, int H, int head_stride, i
   LEV_REQUIRE(dtype == LEV_F32 || dtype == LEV_BF16, "rotary: unknown dtype %d", dtype);
   if (T == 0 || n_pairs == 0) return 0;
   if (dtype == LEV_F32)
-    rotary_half_kernel<float><<<T, 256, 0, stream>>>((float*)x, x_stride, H, head_stride, offset, n_pairs, freqs, positions);
+    rotary_half_kernel<float><<<T, 256, 0, stream>>>((float*)x, x_stride, H, head_stride, offset, n_pairs, freqs, positions, magnitude);
   else
-    rotary_half_kernel<bf16_t><<<T, 256, 0, stream>>>((bf16_t*)x, x_stride, H, head_stride, offset, n_pairs, freqs, positions);
+    rotary_half_kernel<bf16_t><<<T, 256, 0, stream>>>((bf16_t*)x, x_stride, H, head_stride, offset, n_pairs, freqs, positions, magnitude);
   return lev_check_launch("rotary_half");
 }

@@ -272,13 +272,14 @@ _P, _I, _L, _F = ctypes.c_void_p, ctypes.c_int, ctypes.c_long, ctypes.c_float
 
 register_unit("core", ["errors.hip", "elementwise.hip", "layer_ops.hip", "gemm_simple.hip", "attention_simple.hip", "attention_values.hip",
                        "attention_common.hip", "stream_ops.hip", "rotary.hip", "block_linear.hip", "recurrent_ops.hip", "group_norm.hip", "delta_rule.hip",
-                       "moe_ops.hip", "linear_attention.hip", "state_recurrence.hip", "state_chunks.hip"], signatures={
+                       "moe_ops.hip", "linear_attention.hip", "state_recurrence.hip", "state_chunks.hip", "sum_norm.hip"], signatures={
     "lev_embed": [_P] * 5 + [_I, _I, _I, _F, _P],
     "lev_pair_embed_add": [_P] * 6 + [_I, _I, _I, _L, _L, _I, _P],
     "lev_streams_step": [_P, _I, _I, _I, _P, _P, _P, _P, _P, _P, _F, _P, _P, _P, _I, _I, _P, _I, _P, _P],
+    "lev_sum_norm": [_P, _F, _P, _P, _I, _I, _P, _P, _P, _P, _I, _P, _P, _F, _I, _P, _P, _F, _I, _P, _I, _P, _I, _I, _P],
     "lev_rotary_pairs": [_P, _L, _I, _P, _L, _I, _I, _I, _P, _P, _F, _I, _I, _P],
-    "lev_latent_rope_write": [_P, _L, _I, _I, _I, _F, _P, _P, _L, _I, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _I, _P],
-    "lev_rotary_half": [_P, _L, _I, _I, _I, _I, _P, _P, _I, _I, _P],
+    "lev_latent_rope_write": [_P, _L, _I, _I, _I, _F, _P, _P, _L, _I, _I, _I, _I, _P, _P, _F, _P, _P, _P, _I, _I, _I, _P],
+    "lev_rotary_half": [_P, _L, _I, _I, _I, _I, _P, _P, _F, _I, _I, _P],
     "lev_group_norm_step": [_P, _P, _P, _L, _I, _P, _F, _P, _P, _I, _P, _I, _I, _I, _F, _P, _I, _I, _P, _P],
     "lev_delta_rule": [_P] * 5 + [_L, _P, _L, _P, _P, _P, _P, _L, _I, _I, _I, _F, _F, _F, _I, _P],
     "lev_delta_rule_scan": [_P] * 5 + [_L, _P, _L, _P, _P, _P, _P, _L, _P, _I, _I, _I, _I, _F, _F, _F, _I, _P],
@@ -288,8 +289,8 @@ register_unit("core", ["errors.hip", "elementwise.hip", "layer_ops.hip", "gemm_s
     "lev_moe_sort": [_P, _I, _I, _I, _I, _P, _P, _P, _P, _P],
     "lev_moe_linear": [_P, _L, _P, _P, _L, _P, _P, _P] + [_I] * 8 + [_F, _F, _I, _I, _I, _P],
     "lev_moe_combine": [_P, _P, _P, _P, _I, _I, _I, _I, _P, _I, _P, _L, _I, _P],
-    "lev_block_linear": [_P, _L, _P, _P, _P, _L] + [_I] * 7 + [_P],
-    "lev_block_linear_mfma": [_P, _L, _P, _P, _P, _L] + [_I] * 6 + [_P],
+    "lev_block_linear": [_P, _L, _P, _P, _P, _L, _P, _L] + [_I] * 7 + [_P],
+    "lev_block_linear_mfma": [_P, _L, _P, _P, _P, _L, _P, _L] + [_I] * 6 + [_P],
     "lev_causal_conv": [_P, _L, _P, _P, _P, _P, _P, _L, _I, _I, _I, _I, _P],
     "lev_gated_recurrence": [_P, _L, _P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _L, _I, _I, _I, _I, _F, _I, _P],
     "lev_gated_recurrence_scan": [_P, _L, _P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _L, _P, _I, _I, _I, _I, _F, _I, _P],
@@ -308,7 +309,7 @@ register_unit("core", ["errors.hip", "elementwise.hip", "layer_ops.hip", "gemm_s
     "lev_norm_sum2": [_P, _P, _P, _P, _F, _F, _F, _P, _I, _I, _I, _P],
     "lev_token_gate_linear": [_P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "lev_token_gate": [_P, _L, _P, _P, _P, _I, _I, _I, _P],
-    "lev_projection_norm_rotate": [_P, _L, _I, _P, _L, _I, _I, _P, _L, _I, _F, _I, _I, _P, _P, _P, _I, _I, _P, _P, _P, _P, _I, _I, _I, _P],
+    "lev_projection_norm_rotate": [_P, _L, _I, _P, _L, _I, _I, _P, _L, _I, _F, _I, _I, _P, _P, _P, _I, _I, _P, _F, _F, _P, _P, _P, _I, _I, _I, _P],
     "lev_state_recurrence": [_I, _P, _L, _P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _P, _P, _L, _P, _P, _P, _L, _P] + [_I] * 12 + [_F, _F, _F, _I, _I, _P],
     "lev_state_recurrence_workspace": [_I] * 8,
     "lev_gla_tokens": [_P, _P, _L, _P, _P, _L, _P, _L, _P, _P, _P, _P, _L, _I, _I, _I, _I, _F, _F, _F, _I, _I, _P],

@@ -85,6 +85,29 @@ class PendingGatedNorm:
         self.out, self.y, self.gate, self.post_weight, self.mult, self.groups, self.eps = out, y, gate, post_weight, mult, groups, eps
 
 
+class PendingExperts:
+    """Routed experts' outputs (float32 ``[pairs, D]``) that have not been summed: token t's result is
+    ``sum_c weights[t, c] * expert_out[pos_of[t * top + c]]``. ``alone``: nothing else belongs to the feed-forward's result."""
+
+    __slots__ = ("expert_out", "pos_of", "weights", "alone")
+
+    def __init__(self, expert_out, pos_of, weights, alone):
+        self.expert_out, self.pos_of, self.weights, self.alone = expert_out, pos_of, weights, alone
+
+
+class PendingSumNorm:
+    """A sublayer's result that has not entered the residual stream ``out`` (float32 ``[T, D]``) yet (``HipKernels.sum_norm_step`` with
+    ``defer``): ``out`` still has to become ``N(alpha * out + result)``, the result being the sum of ``y`` (float32 ``[T, D]``), a product's
+    unsummed ranges (``product``: its ``out`` holds nothing yet) and routed experts' unsummed outputs, whichever are there. ``norm``:
+    (weight, bias, eps, rms). The next pass that reads ``out`` does it (``sum_norm_step(..., pending=)``, ``norm``); ``HipKernels.finish``
+    runs it by itself."""
+
+    __slots__ = ("out", "alpha", "y", "product", "experts", "norm")
+
+    def __init__(self, out, alpha, y, product, experts, norm):
+        self.out, self.alpha, self.y, self.product, self.experts, self.norm = out, alpha, y, product, experts, norm
+
+
 def _ptr(t: Optional[torch.Tensor]):
     """A tensor's address as ctypes takes it for a ``c_void_p`` parameter: a plain integer, or None."""
     return None if t is None else t.data_ptr()
@@ -266,6 +289,10 @@ class HipKernels:
             _req(n == x.shape[0], "norm: out must have as many rows as x")
         else:
             _req(rows.dtype == torch.int32 and rows.numel() == n, "norm: rows must be int32, one per output row")
+        if isinstance(pending, PendingSumNorm):  # the stream's own norm behind its sum, then this one, in one pass
+            _req(pending.out is x, "norm: the unfinished sum belongs to another tensor")
+            self.sum_norm_step(x, pending=pending, norm=(weight, bias, eps, rms), h_out=out, rows=rows)
+            return
         if isinstance(pending, PendingGatedNorm):  # another kind of norm behind a gated sublayer: finish that first
             self.finish(pending)
             pending = None
@@ -321,6 +348,9 @@ class HipKernels:
         """Finish a product that ``linear(..., may_leave_pending=True)`` left unfinished, or a deferred sum of streams."""
         if isinstance(pending, PendingStreams):
             self.streams_step(pending.streams, y=pending.y, mix=pending.mix, w_out=pending.w_out, x_out=pending.out, y_pending=pending.y_pending)
+            return
+        if isinstance(pending, PendingSumNorm):
+            self.sum_norm_step(pending.out, pending=pending)
             return
         if isinstance(pending, PendingGatedNorm):
             self.group_norm_step(pending.out, groups=pending.groups, eps=pending.eps, pending=pending)
@@ -536,11 +566,12 @@ class HipKernels:
 
     def projection_norm_rotate(self, q, k, n_heads: int, n_kv_heads: int, head_dim: int, eps: float, q_weight, k_weight, q_norm_dim: Optional[int] = None,
                                k_norm_dim: Optional[int] = None, freqs=None, positions=None, half: bool = False, v=None, value_dim: int = 0, k_pages=None,
-                               v_pages=None, dest=None, page_size: int = 0) -> None:
+                               v_pages=None, dest=None, page_size: int = 0, temperature=None) -> None:
         """Queries and keys (``[T, heads*head_dim]``) divided by the root mean square of their whole rows (mean over ``*_norm_dim``; the rows may
         carry zeros) and multiplied by float32 weights as wide as the rows, then rotated by ``positions[t] * freqs[i]`` (``freqs`` None: not at all):
         dimension ``i`` of a head with ``i + len(freqs)`` (``half``) or ``2i`` with ``2i + 1``. Queries in place; keys in place, or, with pages, into
-        them at ``dest`` together with the values (``kv_write``). One kernel, the same arithmetic either way."""
+        them at ``dest`` together with the values (``kv_write``). ``temperature`` (coef, every; or None): the queries at position p also times
+        ``1 + coef ln(floor((p + 1) / every) + 1)``. One kernel, the same arithmetic either way."""
         _dev(q, k, q_weight, k_weight, freqs, positions, v, k_pages, v_pages, dest)
         T, dt = q.shape[0], q.dtype
         _req(dt in _DT and k.dtype == dt and q.shape == (T, n_heads * head_dim) and k.shape == (T, n_kv_heads * head_dim), "projection_norm_rotate: q and k must be [T, heads*head_dim] of one compute dtype")
@@ -551,6 +582,9 @@ class HipKernels:
             _req(freqs.dtype == torch.float32 and freqs.is_contiguous() and 2 * freqs.numel() <= head_dim, "projection_norm_rotate: float32 frequencies, at most head_dim / 2")
             _req(positions is not None and positions.dtype == torch.int32 and positions.numel() == T, "projection_norm_rotate: one int32 position per token")
             n_pairs = freqs.numel()
+        coef, every = (0.0, 0.0) if temperature is None else (float(temperature[0]), float(temperature[1]))
+        if temperature is not None:
+            _req(every > 0.0 and positions is not None and positions.dtype == torch.int32 and positions.numel() == T, "projection_norm_rotate: a temperature needs a positive stretch and one int32 position per token")
         vs = 0
         if k_pages is not None:
             _req(dt == k_pages.dtype == v_pages.dtype == v.dtype and v.shape == (T, n_kv_heads * value_dim), "projection_norm_rotate: values must be [T, kv_heads*value_dim] of the pages' dtype")
@@ -562,7 +596,7 @@ class HipKernels:
         self._check(self.lib.lev_projection_norm_rotate(
             _ptr(q), _rows(q, "projection_norm_rotate: q"), int(n_heads), _ptr(k), _rows(k, "projection_norm_rotate: k"), int(n_kv_heads), int(head_dim),
             _ptr(v) if k_pages is not None else None, vs, int(value_dim), float(eps), int(q_norm_dim or n_heads * head_dim), int(k_norm_dim or n_kv_heads * head_dim),
-            _ptr(q_weight), _ptr(k_weight), _ptr(freqs) if n_pairs else None, n_pairs, int(bool(half)), _ptr(positions) if n_pairs else None, _ptr(k_pages),
+            _ptr(q_weight), _ptr(k_weight), _ptr(freqs) if n_pairs else None, n_pairs, int(bool(half)), _ptr(positions) if n_pairs or every else None, coef, every, _ptr(k_pages),
             _ptr(v_pages), _ptr(dest) if k_pages is not None else None, int(page_size), T, _DT[dt], self._s()))
 
     def norm_write_latent(self, c, weight, eps: float, norm_dim: int, k_pages, v_pages, dest, page_size: int) -> None:
@@ -580,12 +614,12 @@ class HipKernels:
                                                    _ptr(v_pages), _ptr(dest), page_size, T, _DT[c.dtype], self._s()))
 
     def latent_rope_write(self, kv, latent_dim: int, weight, eps: float, norm_dim: int, q, n_heads: int, q_head: int, q_offset: int, freqs, positions,
-                          k_pages, v_pages, dest, page_size: int) -> None:
+                          k_pages, v_pages, dest, page_size: int, magnitude: float = 1.0) -> None:
         """For steps of single tokens, in one kernel: ``kv`` ``[T, latent_dim + rotated part]`` has its latent normed (``head_prepare``
         with ``weight``, the mean of squares over ``norm_dim``) and its rotated part turned (``rotary_half`` from column
         ``latent_dim``), in place; the whole row goes into the key pages and the latent into the value pages at ``dest``
         (``kv_write``); the vectors at ``q_offset`` of the ``n_heads`` heads of ``q_head`` elements of ``q`` are turned too (``q`` None:
-        no queries). ``freqs`` float32 (may be empty: nothing turns)."""
+        no queries). ``freqs`` float32 (may be empty: nothing turns); cosine and sine are multiplied by ``magnitude``."""
         _dev(kv, weight, q, freqs, positions, k_pages, v_pages, dest)
         T, KD = kv.shape
         R, DR = int(latent_dim), KD - int(latent_dim)
@@ -600,8 +634,8 @@ class HipKernels:
         _req(q is None or (q.dim() == 2 and q.shape[0] == T and q.shape[1] >= n_heads * q_head), "latent_rope_write: q must be [T, heads*q_head]")
         self._check(self.lib.lev_latent_rope_write(_ptr(kv), _rows(kv, "latent_rope_write: kv"), R, DR, int(norm_dim), float(eps), _ptr(weight), _ptr(q),
                                                    _rows(q, "latent_rope_write: q") if q is not None else 0, int(n_heads), int(q_head), int(q_offset), n_pairs,
-                                                   _ptr(freqs) if n_pairs else None, _ptr(positions), _ptr(k_pages), _ptr(v_pages), _ptr(dest), page_size, T,
-                                                   _DT[dt], self._s()))
+                                                   _ptr(freqs) if n_pairs else None, _ptr(positions), float(magnitude), _ptr(k_pages), _ptr(v_pages), _ptr(dest),
+                                                   page_size, T, _DT[dt], self._s()))
 
     def recurrent_tokens(self, x, y, taps, conv_bias, gate_weight, gate_bias, decay, state, token_slots, out, out_scale: float = 1.0) -> None:
         """``causal_conv``, the block-diagonal product of the gates and ``gated_recurrence`` for a step in which every token is
@@ -785,11 +819,12 @@ class HipKernels:
     # ---- block-diagonal products ---------------------------------------------------------------
     BLOCK_LINEAR_MAX_ROWS = 128  # plain arithmetic: more rows than this go block by block to the matrix products (a launch per block)
 
-    def block_linear(self, a, w, bias, out) -> None:
+    def block_linear(self, a, w, bias, out, gate=None) -> None:
         """``out[:, b*n_out:(b+1)*n_out] = a[:, b*n_in:(b+1)*n_in] @ w[b].T + bias[b*n_out:(b+1)*n_out]`` for every block b of
         ``w`` ``[B, n_out, n_in]`` (compute dtype). ``a`` is of the weights' dtype or float32; ``out`` of it or float32. bfloat16
         weights whose blocks take a multiple of 8 inputs run on the matrix cores (float32 inputs are rounded to bfloat16 there);
-        everything else in plain 32-bit arithmetic."""
+        everything else in plain 32-bit arithmetic. ``gate`` (``[T, blocks*out]`` of the weights' dtype, rows may be strided): the result
+        times its sigmoid, element by element."""
         _dev(a, w, bias, out)
         _req(w.dim() == 3 and w.is_contiguous() and w.dtype in _DT, "block_linear: the weights must be contiguous [blocks, out, in]")
         B, n_out, n_in = w.shape
@@ -799,19 +834,24 @@ class HipKernels:
         _req(a.dtype == w.dtype or a.dtype == torch.float32, "block_linear: a must have the weights' dtype or be float32")
         _req(out.dtype == w.dtype or out.dtype == torch.float32, "block_linear: out must have the weights' dtype or be float32")
         _req(bias is None or (bias.dtype == torch.float32 and bias.numel() == B * n_out and bias.is_contiguous()), "block_linear: bias must be float32 [blocks*out]")
+        gs = 0
+        if gate is not None:
+            _dev(gate)
+            _req(gate.dtype == w.dtype and gate.shape == out.shape, "block_linear: the gate must be [T, blocks*out] of the weights' dtype")
+            gs = _rows(gate, "block_linear: gate")
         lda = _rows(a, "block_linear: a")
         if (w.dtype == torch.bfloat16 and self.use_mfma and n_in % 8 == 0 and lda % 8 == 0 and a.data_ptr() % 16 == 0):
             # matrix cores: one launch for all blocks and any number of rows
-            self._check(self.lib.lev_block_linear_mfma(_ptr(a), lda, _ptr(w), _ptr(bias), _ptr(out), _rows(out, "block_linear: out"), T, B, n_in, n_out,
+            self._check(self.lib.lev_block_linear_mfma(_ptr(a), lda, _ptr(w), _ptr(bias), _ptr(out), _rows(out, "block_linear: out"), _ptr(gate), gs, T, B, n_in, n_out,
                                                        _DT[a.dtype], _DT[out.dtype], self._s()))
             return
-        if T > self.BLOCK_LINEAR_MAX_ROWS and a.dtype == w.dtype:
+        if T > self.BLOCK_LINEAR_MAX_ROWS and a.dtype == w.dtype and gate is None:
             for b in range(B):
                 self.linear(a[:, b * n_in:(b + 1) * n_in], w[b], None if bias is None else bias[b * n_out:(b + 1) * n_out],
                             out[:, b * n_out:(b + 1) * n_out])
             return
         self._check(self.lib.lev_block_linear(_ptr(a), _rows(a, "block_linear: a"), _ptr(w), _ptr(bias), _ptr(out), _rows(out, "block_linear: out"),
-                                              T, B, n_in, n_out, _DT[a.dtype], _DT[w.dtype], _DT[out.dtype], self._s()))
+                                              _ptr(gate), gs, T, B, n_in, n_out, _DT[a.dtype], _DT[w.dtype], _DT[out.dtype], self._s()))
 
     # ---- the recurrent branch ------------------------------------------------------------------
     def causal_conv(self, x, taps, bias, state, token_slots, u) -> None:
@@ -902,11 +942,63 @@ class HipKernels:
                                                  _DT[odt], _ptr(rows), n, D, int(groups), float(eps), _ptr(part), int(n_ranges), T, _ptr(part_bias), self._s()))
         return None
 
+    # ---- a stream that is normed behind every sum ----------------------------------------------
+    def sum_norm_step(self, x, *, alpha: float = 1.0, y=None, product: Optional[PendingProduct] = None, experts: Optional[PendingExperts] = None,
+                      write_norm=None, norm=None, h_out=None, rows=None, defer: bool = False, pending: Optional[PendingSumNorm] = None) -> Optional[PendingSumNorm]:
+        """One pass over the rows of the residual stream ``x`` (float32 ``[T, D]``). In this order, whatever is given: the write of a
+        sublayer's result, ``x <- N(alpha * x + result)`` with ``write_norm`` = (weight, bias or None, eps, rms), the result being the sum of
+        ``y``, a ``product`` that has left its K ranges and ``experts`` that nobody has summed; the read ``h_out`` = x as it is, or its norm by
+        ``norm`` (a tuple of the same form), in the compute dtype or float32. ``rows``: only these rows, into ``h_out [len(rows), D]``; ``x`` is
+        not stored then. ``defer``: nothing is launched; the write comes back as a ``PendingSumNorm`` for the next call (``pending=``)."""
+        if defer:
+            return PendingSumNorm(x, float(alpha), y, product, experts, write_norm)
+        if pending is not None:
+            _req(pending.out is x and write_norm is None, "sum norm: the unfinished sublayer belongs to another tensor")
+            alpha, y, product, experts, write_norm = pending.alpha, pending.y, pending.product, pending.experts, pending.norm
+        _req(x.dim() == 2 and x.dtype == torch.float32 and x.is_contiguous(), "sum norm: x must be contiguous float32 [T, D]")
+        T, D = x.shape
+
+        def norm_args(n, what):
+            if n is None:
+                return None, None, 0.0, 0
+            w, b, eps, rms = n
+            for t in (w, b):
+                _req(t is None or (t.dtype == torch.float32 and t.numel() == D and t.is_contiguous()), f"sum norm: {what} must have float32 [D] weights")
+            _dev(w, b)
+            return _ptr(w), _ptr(b), float(eps), int(bool(rms))
+
+        w1, b1, eps1, rms1 = norm_args(write_norm, "the norm behind the sum")
+        w2, b2, eps2, rms2 = norm_args(norm, "the norm of the read")
+        _dev(x, y, h_out, rows)
+        _req(y is None or (y.dtype == torch.float32 and tuple(y.shape) == (T, D) and y.is_contiguous()), "sum norm: a result must be contiguous float32 [T, D]")
+        part = part_bias = None
+        n_ranges = top = 0
+        if product is not None:
+            _req(tuple(product.out.shape) == (T, D) and product.ldo == D, "sum norm: the unfinished product has another shape")
+            part, n_ranges, part_bias = product.workspace, product.n_ranges, product.bias
+        eo = po = wt = None
+        if experts is not None:
+            eo, po, wt = experts.expert_out, experts.pos_of, experts.weights
+            _dev(eo, po, wt)
+            top = wt.shape[1]
+            _req(eo.dtype == wt.dtype == torch.float32 and eo.is_contiguous() and wt.is_contiguous() and wt.shape[0] == T and eo.shape[1] == D
+                 and eo.shape[0] >= T * top and po.dtype == torch.int32 and po.numel() >= T * top, "sum norm: bad experts' outputs")
+        n, odt = T, torch.float32
+        if rows is not None:
+            _req(rows.dtype == torch.int32 and rows.is_contiguous() and h_out is not None, "sum norm: rows must be int32 and need an output")
+            n = rows.numel()
+        if h_out is not None:
+            _req(h_out.dtype in _DT and h_out.is_contiguous() and tuple(h_out.shape) == (n, D), "sum norm: bad output")
+            odt = h_out.dtype
+        self._check(self.lib.lev_sum_norm(_ptr(x), float(alpha), _ptr(y), _ptr(part), int(n_ranges), T, _ptr(part_bias), _ptr(eo), _ptr(po), _ptr(wt), int(top),
+                                          w1, b1, eps1, rms1, w2, b2, eps2, rms2, _ptr(h_out), _DT[odt], _ptr(rows), n, D, self._s()))
+        return None
+
     # ---- rotation, "rotate half" layout --------------------------------------------------------
-    def rotary_half(self, x, n_heads: int, head_stride: int, offset: int, freqs, positions) -> None:
+    def rotary_half(self, x, n_heads: int, head_stride: int, offset: int, freqs, positions, magnitude: float = 1.0) -> None:
         """In place on ``x`` ``[T, >= n_heads*head_stride]``: within each head of ``head_stride`` columns, the vector that starts at
         column ``offset`` has its dimension i < len(freqs) paired with dimension i + len(freqs), and the pair turns by
-        ``positions[t] * freqs[i]``; every other column stays. 32-bit angles."""
+        ``positions[t] * freqs[i]``, cosine and sine both times ``magnitude``; every other column stays. 32-bit angles."""
         _dev(x, freqs, positions)
         T = x.shape[0]
         _req(x.dim() == 2 and x.dtype in _DT and x.shape[1] >= n_heads * head_stride, "rotary: x must be [T, heads*head_stride]")
@@ -916,7 +1008,7 @@ class HipKernels:
         if freqs.numel() == 0:
             return
         self._check(self.lib.lev_rotary_half(_ptr(x), _rows(x, "rotary: x"), int(n_heads), int(head_stride), int(offset), freqs.numel(), _ptr(freqs),
-                                             _ptr(positions), T, _DT[x.dtype], self._s()))
+                                             _ptr(positions), float(magnitude), T, _DT[x.dtype], self._s()))
 
     # ---- a matrix state per head with decay and removal (generalized delta rule) ----------------
     def delta_rule(self, r, k, v, a_pre, g, w_pre, norm_weight, state, token_slots, out, n_heads: int, head_dim: int, norm_eps: float,
@@ -1075,10 +1167,13 @@ class HipKernels:
         _req(table.dtype == out.dtype and table.dtype in _DT and table.is_contiguous() and out.is_contiguous() and table.dim() == 2 and table.shape[1] == D, "token_gate: table [vocab, D] and out [T, D] must be contiguous and of one compute dtype")
         self._check(self.lib.lev_token_gate(_ptr(z), _rows(z, "token_gate: z"), _ptr(tokens), _ptr(table), _ptr(out), T, D, _DT[out.dtype], self._s()))
 
+    MOE_SCORING = {"sigmoid": 0, "softmax": 1, "softmax_chosen": 2}
+
     # ---- mixture of experts --------------------------------------------------------------------
     def moe_route(self, z, correction, chosen, weights, *, n_groups: int = 1, keep: int = 1, group_top: int = 2, renormalize: bool = False,
-                  softmax: bool = False) -> None:
-        """Per token: ``s = sigmoid(z)`` (``z`` float32 ``[T, E]``), or with ``softmax`` the softmax of ``z`` over all E; the choice goes by ``s + correction``; only experts of the
+                  scoring: str = "sigmoid") -> None:
+        """Per token: ``s = sigmoid(z)`` (``z`` float32 ``[T, E]``), with ``scoring`` "softmax" the softmax of ``z`` over all E, with "softmax_chosen"
+        ``z`` itself, the weights then being the softmax over the winners' ``s``; the choice goes by ``s + correction``; only experts of the
         ``keep`` groups (of ``n_groups`` equal groups of neighbours) whose ``group_top`` largest choice scores sum highest can be
         chosen; ``chosen`` int32 ``[T, top]`` the winners in the order of falling choice score (ties: lower index first),
         ``weights`` float32 ``[T, top]`` their ``s`` (divided by their sum with ``renormalize``)."""
@@ -1089,7 +1184,7 @@ class HipKernels:
         _req(tuple(chosen.shape) == tuple(weights.shape) == (T, top) and chosen.is_contiguous() and weights.is_contiguous(), "experts: choices and weights must be [T, top]")
         _req(correction is None or (correction.dtype == torch.float32 and correction.numel() == E and correction.is_contiguous()), "experts: the correction must be float32 [E]")
         self._check(self.lib.lev_moe_route(_ptr(z), _rows(z, "experts: z"), _ptr(correction), T, E, int(n_groups), int(keep), int(group_top), top,
-                                           int(renormalize), int(bool(softmax)), _ptr(chosen), _ptr(weights), self._s()))
+                                           int(renormalize), self.MOE_SCORING[scoring], _ptr(chosen), _ptr(weights), self._s()))
 
     @staticmethod
     def moe_tile_rows(pairs: int, n_experts: int) -> int:
@@ -1113,7 +1208,7 @@ class HipKernels:
 
     def moe_linear(self, a, w, out, tiles, meta, sorted_pairs, *, top: int, gather: bool, glu: bool = False, activation: str = "none",
                    tile_rows: int = 16, limit: float = 0.0, up_shift: float = 0.0) -> None:
-        """For every tile of ``moe_sort``: ``out[pos] = w[expert] a[row(pos)]``, ``row(pos)`` the pair's token (``gather``) or
+        """For every tile of ``moe_sort``: ``out[pos] = act(w[expert] a[row(pos)])``, ``row(pos)`` the pair's token (``gather``) or
         ``pos`` itself. ``w`` ``[E, N, K]``; with ``glu`` N = 2F, gate rows then up rows, and ``out[pos][f] = act(gate_f) * (up_f + up_shift)``;
         with ``limit`` > 0 the gate sum is capped at it and the up sum clamped to +-limit first."""
         _dev(a, w, out, tiles, meta, sorted_pairs)

@@ -1,6 +1,6 @@
 """Parts that layers are put together from. Importing the package registers the built-in kinds."""
 from . import (attention, block, delta_rule, embedding, feed_forward, gated_block, head, hyper_connections, latent_attention, linear_attention, moe, norm,  # noqa: F401
-               parallel_mixers, position, recurrent, state_recurrence, stream_mix, talking_attention, token_input)
+               parallel_mixers, position, recurrent, state_recurrence, stream_mix, sum_norm, talking_attention, token_input)
 from .base import (AttentionMeta, Block, BuildEnv, CacheUnitView, Embedding, FeedForward, GroupView, Head, Mixer, Norm, Part,
                    PositionEncoding, StepContext, StreamEntry, StreamMix)
 from .decoder import DecoderLm

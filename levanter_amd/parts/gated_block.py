@@ -107,6 +107,10 @@ class GatedPostNorm(Part):
         self.gate = None
         return fused
 
+    def read(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
+        """The stream itself as a sublayer's input (blocks without a norm ahead of their sublayers)."""
+        return read_stream(x, ctx, self.groups, self.eps)
+
     def write(self, y: torch.Tensor, gate: Optional[torch.Tensor], x: torch.Tensor, ctx: StepContext) -> None:
         pending = ctx.kernels.group_norm_step(x, groups=self.groups, eps=self.eps, y=y, gate=gate, post_weight=self.weight, mult=self.mult, defer=True)
         if ctx.may_defer:
@@ -192,10 +196,11 @@ class GatedSandwichBlock(Block):
 
 @BLOCKS.register("post_norm")
 class PostNormBlock(Block):
-    """Sublayers that read the residual stream itself and whose results are normed on their way into it:
-    ``x <- x + connect1(mixer(x))``, then (if the layer has one) ``x <- x + connect2(feed_forward(x))``; a ``connect`` is a
-    ``gated_post_norm`` (its gate may be switched off). There is no norm ahead of a sublayer: its input is the stream, rounded to
-    the compute dtype by the pass that also does the write of the sublayer before (one row kernel a sublayer)."""
+    """Sublayers that read the residual stream itself and whose results meet a norm on their way into it: ``connect1`` takes the
+    mixer's result, then (if the layer has one) ``connect2`` the feed-forward's. A ``connect`` says how: ``gated_post_norm``,
+    ``x <- x + N(f(x))`` (its gate may be switched off), or ``norm_after_sum``, ``x <- N(alpha x + f(x))``. There is no norm ahead of a
+    sublayer: its input is the stream, rounded to the compute dtype by the pass that also does the write of the sublayer before (one
+    row kernel a sublayer)."""
 
     roles = ("mixer", "connect1")
     defers_residual = True  # the stream is read through that pass only
@@ -212,19 +217,30 @@ class PostNormBlock(Block):
             raise ValueError("block 'post_norm': a feed-forward needs connect2")
 
     def _sublayer(self, connect, run, x: torch.Tensor, ctx: StepContext) -> None:
+        """``run(h, y)`` computes the sublayer's result into ``y``; what it returns (experts' outputs that nobody has summed, or None)
+        belongs to the result too."""
         may_defer = ctx.may_defer
-        h = read_stream(x, ctx, connect.groups, connect.eps)  # the write that the sublayer before has left pending is done in the same pass
+        h = connect.read(x, ctx)  # the write that the sublayer before has left pending is done in the same pass
         y = torch.empty_like(x)
         ctx.may_defer = False  # a sublayer's result is complete before it is normed
-        run(h, y)
+        experts = run(h, y)
         product = ctx.take_product_pending(y)
+        if getattr(connect, "takes_unsummed", False):
+            ctx.may_defer = may_defer
+            connect.write(None if experts is not None and experts.alone else y, None, x, ctx, product=product, experts=experts)
+            return
         if product is not None:
             ctx.kernels.finish(product)
         gate = connect.gate_of(h, ctx)
         ctx.may_defer = may_defer
         connect.write(y, gate, x, ctx)
 
+    def _feed_forward(self, h: torch.Tensor, y: torch.Tensor, ctx: StepContext):
+        if getattr(self.connect2, "takes_unsummed", False) and hasattr(self.feed_forward, "compute_unsummed"):
+            return self.feed_forward.compute_unsummed(h, y, ctx)
+        return self.feed_forward.compute(h, y, ctx)
+
     def forward(self, x: torch.Tensor, ctx: StepContext, unit: CacheUnitView, writes_cache: bool) -> None:
         self._sublayer(self.connect1, lambda h, y: self.mixer.compute(h, y, ctx, unit, writes_cache), x, ctx)
         if self.feed_forward is not None:
-            self._sublayer(self.connect2, lambda h, y: self.feed_forward.compute(h, y, ctx), x, ctx)
+            self._sublayer(self.connect2, lambda h, y: self._feed_forward(h, y, ctx), x, ctx)

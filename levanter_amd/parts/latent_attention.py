@@ -16,12 +16,15 @@ Switched on by the description:
 * queries through a latent of their own: q = W_uq RMSNorm(W_dq h) (``query_latent_dim``);
 * a rotated part: every query head carries ``rope_dim`` more dimensions behind its dk, and W_dkv h ``rope_dim`` more rows behind
   the latent (not normed): one key part that all heads share. Both turn with the position (``rotary``: ``dims`` <= rope_dim
-  dimensions in the rotate-half layout, dimension i paired with i + dims/2, angle p * base^(-2i/dims)), and the score is
-  scale * (q_h . k_h + q_rot_h . k_rot). The cached key is [c | k_rot] (after the rotation), the cached value c: the queries'
+  dimensions in the rotate-half layout, dimension i paired with i + dims/2, or (``layout`` "pairs") 2i with 2i + 1, angle
+  p * base^(-2i/dims) or what ``scaling`` makes of it (``rotary_frequencies``), cosine and sine times ``magnitude``), and the score is
+  scale * (q_h . k_h + q_rot_h . k_rot). Neighbouring pairs are brought into the rotate-half order when the weights are loaded (the same
+  permutation of the rows that make the queries' and the key's rotated parts changes no score). The cached key is [c | k_rot] (after the rotation), the cached value c: the queries'
   rotated part passes the map into the latent's space unchanged (an identity block);
 * a window of the last ``window`` keys;
 * a sink per head: exp(sink_h) in the softmax's denominator, with no key and no value (``sinks``);
-* an output gate: head h times sigmoid(gate_h . h) (``gate``);
+* an output gate: head h times sigmoid(gate_h . h) (``gate``), or (``gate_kind`` "element") every element of the heads times the
+  sigmoid of a projection of its own, in the product that brings the result out of the latent's space;
 * a layer without W_dkv that reads the latent and rotated key part another layer has cached (``shared_kv``): its plan entry
   names that layer's cache unit and does not write. ``cache_window`` is what the unit keeps: the largest window of the
   layers that read it.
@@ -35,6 +38,7 @@ import torch
 from levanter_amd.cache.requirements import PagedKv
 from .base import BuildEnv, CacheUnitView, Mixer, StepContext
 from .linear import Linear
+from .position import rotary_frequencies
 from .registry import MIXERS
 from .spec import PartSpec
 
@@ -46,10 +50,12 @@ def _pad(n: int, step: int) -> int:
 @MIXERS.register("latent_attention")
 class LatentAttention(Mixer):
     """params: ``dim``, ``n_heads``, ``head_dim``, ``value_dim``, ``latent_dim``, ``scale``, ``norm_eps``; optional ``query_latent_dim``,
-    ``rope_dim`` with ``rotary`` (``{"dims", "base"}``), ``window``, ``cache_window``, ``sinks``, ``gate``, ``shared_kv``. Tensors
+    ``rope_dim`` with ``rotary`` (``{"dims", "base"}``, optional ``layout`` ("half"), ``scaling``, ``magnitude``), ``window``, ``cache_window``,
+    ``sinks``, ``gate``, ``gate_kind`` ("head"), ``shared_kv``. Tensors
     (``[out, in]``): ``q.weight`` ``[H*(dk+dr), dim]`` or, with a query latent, ``q_down.weight`` ``[Q, dim]``, ``q_norm.weight``
     ``[Q]``, ``q.weight`` ``[H*(dk+dr), Q]``; ``down.weight`` ``[R+dr, dim]``, ``latent_norm.weight`` ``[R]`` (not with ``shared_kv``);
-    ``up_k.weight`` ``[H*dk, R]``, ``up_v.weight`` ``[H*dv, R]``, ``out.weight`` ``[dim, H*dv]``; ``sinks`` ``[H]``; ``gate.weight`` ``[H, dim]``."""
+    ``up_k.weight`` ``[H*dk, R]``, ``up_v.weight`` ``[H*dv, R]``, ``out.weight`` ``[dim, H*dv]``; ``sinks`` ``[H]``; ``gate.weight`` ``[H, dim]`` (or
+    ``[H*dv, dim]``)."""
 
     graph_safe = True
 
@@ -85,8 +91,22 @@ class LatentAttention(Mixer):
             raise ValueError(f"latent_attention: {2 * n_pairs} rotated dimensions do not fit a rotated part of {dr}")
         self.freqs = None
         if n_pairs:
-            base = float(rot["base"])
-            self.freqs = torch.tensor([base ** (-2.0 * i / (2 * n_pairs)) for i in range(n_pairs)], dtype=torch.float64).to(torch.float32).to(env.device)
+            freqs = rotary_frequencies(2 * n_pairs, float(rot["base"]), rot.get("scaling"))
+            self.freqs = torch.tensor(freqs, dtype=torch.float64).to(torch.float32).to(env.device)
+        self.magnitude = {"magnitude": float(rot["magnitude"])} if rot.get("magnitude", 1.0) != 1.0 else {}
+        layout = rot.get("layout", "half")
+        if layout not in ("half", "pairs"):
+            raise ValueError(f"latent_attention: the rotation's layout is 'half' or 'pairs', got {layout!r}")
+        # the rows of a rotated part in the order the kernels turn them: i and i + n_pairs together
+        turned = list(range(dr)) if layout == "half" else [*range(0, 2 * n_pairs, 2), *range(1, 2 * n_pairs, 2), *range(2 * n_pairs, dr)]
+
+        def queries(w):
+            """A query projection's rows, every head's rotated part in that order."""
+            if layout == "half":
+                return w
+            heads = w.view(H, self.q_head, -1)
+            return torch.cat([heads[:, :dk], heads[:, dk:][:, turned]], 1).reshape(w.shape)
+
         # one product for everything that reads h: [queries or their latent | latent | rotated key part | gate], each part
         # starting at a multiple of 8 columns
         rows, at = [], 0
@@ -103,22 +123,24 @@ class LatentAttention(Mixer):
             self.q_cols = Qp
             part(f32("q_down.weight", (Q, self.dim)), Qp)
             self.q_norm_weight = torch.cat([f32("q_norm.weight", (Q,)), torch.zeros(Qp - Q)]).to(env.device).contiguous()
-            self.up_q = Linear(torch.cat([f32("q.weight", (H * self.q_head, Q)), torch.zeros(H * self.q_head, Qp - Q)], 1), None, "out_in", env)
+            self.up_q = Linear(torch.cat([queries(f32("q.weight", (H * self.q_head, Q))), torch.zeros(H * self.q_head, Qp - Q)], 1), None, "out_in", env)
         else:
             self.q_cols = H * self.q_head
-            part(f32("q.weight", (H * self.q_head, self.dim)), _pad(self.q_cols, 8))
+            part(queries(f32("q.weight", (H * self.q_head, self.dim))), _pad(self.q_cols, 8))
         self.c_off = at
         self.norm_weight = None
         if not self.shared_kv:
             w_down = f32("down.weight", (R + dr, self.dim))
             part(w_down[:R], Rp)
             if drp:
-                part(w_down[R:], drp)
+                part(w_down[R:][turned], drp)
             self.norm_weight = torch.cat([f32("latent_norm.weight", (R,)), torch.zeros(Rp - R)]).to(env.device).contiguous()
         self.g_off = at
         self.has_gate = bool(p.get("gate", False))
+        self.gate_elements = p.get("gate_kind", "head") == "element"
+        self.g_cols = H * dv if self.gate_elements else H
         if self.has_gate:
-            part(f32("gate.weight", (H, self.dim)), _pad(H, 8))
+            part(f32("gate.weight", (self.g_cols, self.dim)), _pad(self.g_cols, 8))
         self.proj = Linear(torch.cat(rows, 0), None, "out_in", env)
         self.sinks = f32("sinks", (H,)).to(env.device).contiguous() if p.get("sinks") else None
         # queries into the latent's space, head by head: [H, Rp + drp, dk + dr] = [[W_uk[h]^T, 0], [0, 1]]; results out of it:
@@ -161,18 +183,18 @@ class LatentAttention(Mixer):
             q = p[:, :self.q_cols]
         singles = ctx.attention.n_prefill_tiles == 0  # a step of single tokens: rotation, norm and cache write in one kernel
         if self.freqs is not None and not (singles and writes_cache and self.rope):
-            K.rotary_half(q, H, self.q_head, self.head_dim, self.freqs, positions)
+            K.rotary_half(q, H, self.q_head, self.head_dim, self.freqs, positions, **self.magnitude)
         if writes_cache:
             kv = p[:, self.c_off:self.c_off + KD]  # [latent | rotated key part]
             c = kv[:, :Rp]
             if singles and self.rope:
                 K.latent_rope_write(kv, Rp, self.norm_weight, self.eps, self.true_latent, q, H, self.q_head, self.head_dim, self.freqs, positions,
-                                    unit.k_pages, unit.v_pages, g.dest, g.page_size)
+                                    unit.k_pages, unit.v_pages, g.dest, g.page_size, **self.magnitude)
             elif singles:
                 K.norm_write_latent(c, self.norm_weight, self.eps, self.true_latent, unit.k_pages, unit.v_pages, g.dest, g.page_size)
             else:
                 if self.freqs is not None:
-                    K.rotary_half(kv, 1, KD, Rp, self.freqs, positions)
+                    K.rotary_half(kv, 1, KD, Rp, self.freqs, positions, **self.magnitude)
                 # the latent's RMS norm (32-bit statistics, the weight applied), in place; then into the pages, as key and as value
                 K.head_prepare(c, 1, Rp, self.eps, norm_dim=self.true_latent, norm_weight=self.norm_weight)
                 K.kv_write(kv, c, unit.k_pages, unit.v_pages, g.dest, 1, KD, g.page_size, value_dim=Rp)  # 16 tokens at a time, transposed through LDS
@@ -182,7 +204,9 @@ class LatentAttention(Mixer):
         extra = {} if self.sinks is None else {"sinks": self.sinks}
         K.attention_values(qa, o, unit.k_pages, unit.v_pages, ctx.attention, n_heads=H, n_kv_heads=1, head_dim=KD, value_dim=Rp,
                            all_value_heads=False, page_size=g.page_size, scale=self.scale, window=self.window, block_tables=g.block_tables, **extra)
-        if self.has_gate:  # head h times sigmoid(gate_h): a number per head commutes with the map out of the latent's space
+        if self.has_gate and self.gate_elements:  # the gate's product stands with the other projections; it is applied where the heads are made
+            K.block_linear(o.view(T, H * Rp), self.w_expand, None, a, gate=p[:, self.g_off:self.g_off + self.g_cols])
+        elif self.has_gate:  # head h times sigmoid(gate_h): a number per head commutes with the map out of the latent's space
             og = ctx.empty(T, H * Rp)
             K.head_talk(o, None, p[:, self.g_off:self.g_off + H], og, H, 1, Rp)
             K.block_linear(og, self.w_expand, None, a)

@@ -12,18 +12,19 @@ stretch into row tiles, and the two products run over the tiles with a grid size
 tiles that exist return at once), so the launches depend on the number of tokens alone and a step can be replayed from a
 HIP graph. Experts whose inner width is no multiple of 8 carry zeros behind it.
 
-Switches beside that: ``score`` "softmax" (the scores are the softmax of z over all router outputs); ``n_identity`` router outputs
+Switches beside that: ``score`` "softmax" (the scores are the softmax of z over all router outputs) or "softmax_chosen" (the choice goes
+by z, the weights are the softmax over the chosen z alone); ``gated`` False (an expert is W_down act(W_up h)); ``n_identity`` router outputs
 behind the experts' that stand for experts without weights whose result is their input (they take part in scores, groups and
 choice like any other); ``limit`` and ``up_shift`` in the experts' activation, act(min(gate, limit)) * (clamp(up, +-limit) +
 up_shift); ``shared``, the description of a feed-forward that runs for every token and is added.
 """
 from __future__ import annotations
 
-from typing import Dict
+from typing import Dict, Optional
 
 import torch
 
-from levanter_amd.kernels.library import ACTIVATIONS
+from levanter_amd.kernels.library import ACTIVATIONS, PendingExperts
 from .base import BuildEnv, FeedForward, StepContext
 from .linear import Linear
 from .embedding import tensors_of_nested
@@ -34,10 +35,10 @@ from .spec import PartSpec
 @FEED_FORWARDS.register("routed_experts")
 class RoutedExperts(FeedForward):
     """params: ``dim``, ``inner_dim``, ``n_experts``, ``top``, ``n_groups`` (1), ``keep`` (1), ``group_top`` (2), ``activation``
-    ("silu"), ``renormalize`` (False), ``correction`` (True: the tensor exists), ``score`` ("sigmoid" or "softmax"), ``n_identity`` (0),
-    ``limit`` (None), ``up_shift`` (0), ``shared`` (None, or the description of a feed-forward). Tensors: ``router.weight`` ``[E + n_identity, dim]``,
-    ``correction`` ``[E + n_identity]``, and per expert e ``experts.<e>.gate.weight``, ``experts.<e>.up.weight`` ``[inner, dim]``,
-    ``experts.<e>.down.weight`` ``[dim, inner]``."""
+    ("silu"), ``renormalize`` (False), ``correction`` (True: the tensor exists), ``score`` ("sigmoid", "softmax" or "softmax_chosen"),
+    ``gated`` (True), ``n_identity`` (0), ``limit`` (None), ``up_shift`` (0), ``shared`` (None, or the description of a feed-forward).
+    Tensors: ``router.weight`` ``[E + n_identity, dim]``, ``correction`` ``[E + n_identity]``, and per expert e ``experts.<e>.gate.weight``
+    (if gated), ``experts.<e>.up.weight`` ``[inner, dim]``, ``experts.<e>.down.weight`` ``[dim, inner]``."""
 
     graph_safe = True
 
@@ -54,10 +55,13 @@ class RoutedExperts(FeedForward):
         self.n_identity = int(p.get("n_identity", 0))
         N = self.n_outputs = E + self.n_identity  # what the router chooses among
         self.score = p.get("score", "sigmoid")
-        if self.score not in ("sigmoid", "softmax"):
-            raise ValueError(f"routed_experts: the scores are 'sigmoid' or 'softmax', got {self.score!r}")
+        if self.score not in ("sigmoid", "softmax", "softmax_chosen"):
+            raise ValueError(f"routed_experts: the scores are 'sigmoid', 'softmax' or 'softmax_chosen', got {self.score!r}")
+        self.gated = bool(p.get("gated", True))
         self.limit = float(p["limit"]) if p.get("limit") else 0.0
         self.up_shift = float(p.get("up_shift", 0.0))
+        if not self.gated and (self.limit or self.up_shift):
+            raise ValueError("routed_experts: a limit and a shift belong to gated experts")
         if N % self.n_groups or not 0 < self.keep <= self.n_groups or not 0 < self.top <= self.keep * (N // self.n_groups):
             raise ValueError(f"routed_experts: {N} experts in {self.n_groups} groups, {self.keep} kept, {self.top} used")
         Fp = self.inner_padded = (F + 7) // 8 * 8
@@ -75,12 +79,13 @@ class RoutedExperts(FeedForward):
         if shared is not None:
             self.shared = part_class(shared.kind, shared.family or "feed_forward")(shared, tensors_of_nested("shared", tensors), env)
             self.graph_safe = bool(self.shared.graph_safe)
-        # [E, gate rows then up rows, dim] and [E, dim, inner]
-        w_in = torch.zeros(E, 2 * Fp, D)
+        # [E, gate rows then up rows (not gated: up rows), dim] and [E, dim, inner]
+        w_in = torch.zeros(E, 2 * Fp if self.gated else Fp, D)
         w_down = torch.zeros(E, D, Fp)
         for e in range(E):
-            w_in[e, :F] = f32(f"experts.{e}.gate.weight", (F, D))
-            w_in[e, Fp:Fp + F] = f32(f"experts.{e}.up.weight", (F, D))
+            if self.gated:
+                w_in[e, :F] = f32(f"experts.{e}.gate.weight", (F, D))
+            w_in[e, -Fp:][:F] = f32(f"experts.{e}.up.weight", (F, D))
             w_down[e, :, :F] = f32(f"experts.{e}.down.weight", (D, F))
         self.w_in = w_in.to(env.device, env.dtype).contiguous()
         self.w_down = w_down.to(env.device, env.dtype).contiguous()
@@ -96,17 +101,28 @@ class RoutedExperts(FeedForward):
         computed as part of a larger product over ``h``."""
         self._run(h, y, ctx, False, z)
 
-    def _run(self, h: torch.Tensor, y: torch.Tensor, ctx: StepContext, accumulate: bool, z=None) -> None:
+    def compute_unsummed(self, h: torch.Tensor, y: torch.Tensor, ctx: StepContext) -> Optional[PendingExperts]:
+        """``compute`` that leaves the weighted sum over the chosen experts to the kernel that reads the result: ``y`` takes the shared
+        expert's part (nothing without one; its product may leave its K ranges), the experts' outputs come back."""
+        if self.n_identity:
+            self.compute(h, y, ctx)
+            return None
+        expert_out, pos_of, weights, _ = self._experts(h, ctx)
+        if self.shared is not None:
+            self.shared.compute(h, y, ctx)
+        return PendingExperts(expert_out, pos_of, weights, alone=self.shared is None)
+
+    def _experts(self, h: torch.Tensor, ctx: StepContext, z=None):
+        """Routing and the chosen experts' products: their outputs (float32 ``[T * top, dim]``, in the order of the experts), every pair's place
+        among them, the weights and the choices ``[T, top]``."""
         K = ctx.kernels
         T, E, top = h.shape[0], self.n_outputs, self.top
         dev = h.device
         if z is None:
             z = self.router(h, ctx, out_dtype=torch.float32)
-        if accumulate:
-            ctx.settle()  # the sum below reads the residual stream itself
         chosen = torch.empty((T, top), dtype=torch.int32, device=dev)
         weights = torch.empty((T, top), dtype=torch.float32, device=dev)
-        more = {"softmax": True} if self.score == "softmax" else {}
+        more = {"scoring": self.score} if self.score != "sigmoid" else {}
         K.moe_route(z, self.correction, chosen, weights, n_groups=self.n_groups, keep=self.keep, group_top=self.group_top, renormalize=self.renormalize, **more)
         P = T * top
         rows = K.moe_tile_rows(P, E)  # prompts: four row tiles on every weight fragment a wave loads
@@ -116,9 +132,18 @@ class RoutedExperts(FeedForward):
         K.moe_sort(chosen, E, sorted_pairs, pos_of, tiles, meta, tile_rows=rows, **own)
         inner = ctx.empty(P, self.inner_padded)
         clamp = {"limit": self.limit, "up_shift": self.up_shift} if self.limit or self.up_shift else {}
-        K.moe_linear(h, self.w_in, inner, tiles, meta, sorted_pairs, top=top, gather=True, glu=True, activation=self.activation, tile_rows=rows, **clamp)
+        K.moe_linear(h, self.w_in, inner, tiles, meta, sorted_pairs, top=top, gather=True, glu=self.gated, activation=self.activation, tile_rows=rows, **clamp)
         expert_out = ctx.empty(P, self.dim, torch.float32)
         K.moe_linear(inner, self.w_down, expert_out, tiles, meta, sorted_pairs, top=top, gather=False, tile_rows=rows)
+        return expert_out, pos_of, weights, chosen
+
+    def _run(self, h: torch.Tensor, y: torch.Tensor, ctx: StepContext, accumulate: bool, z=None) -> None:
+        K = ctx.kernels
+        if z is None:
+            z = self.router(h, ctx, out_dtype=torch.float32)
+        if accumulate:
+            ctx.settle()  # the sum below reads the residual stream itself
+        expert_out, pos_of, weights, chosen = self._experts(h, ctx, z)
         if self.n_identity:
             K.moe_combine(expert_out, pos_of, weights, y, accumulate=accumulate, chosen=chosen, n_real=self.n_experts, identity_in=h)
         else:

@@ -14,6 +14,9 @@ from .spec import PartSpec
 
 @NORMS.register("layernorm")
 class LayerNorm(Norm):
+    """params: ``dim``, ``eps``, ``bias`` (True), ``out_scale`` (1: a factor on the norm's output, for a model that scales its logits: the
+    factor stands ahead of the head's product, where it rounds nothing twice). Tensors: ``weight``, ``bias``."""
+
     graph_safe = True
     folds_pending = True
 
@@ -23,8 +26,9 @@ class LayerNorm(Norm):
         super().__init__(spec, tensors, env)
         self.dim = int(spec.params["dim"])
         self.eps = float(spec.params["eps"])
-        self.weight = tensors["weight"].to(env.device, torch.float32).contiguous()
-        self.bias = tensors["bias"].to(env.device, torch.float32).contiguous() if spec.params.get("bias", True) else None
+        out_scale = float(spec.params.get("out_scale", 1.0))
+        self.weight = (tensors["weight"].to(env.device, torch.float32) * out_scale).contiguous()
+        self.bias = (tensors["bias"].to(env.device, torch.float32) * out_scale).contiguous() if spec.params.get("bias", True) else None
 
     def __call__(self, x: torch.Tensor, ctx: StepContext, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
         n = x.shape[0] if rows is None else rows.numel()

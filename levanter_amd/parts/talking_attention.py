@@ -4,6 +4,7 @@
 * key and value heads of different sizes;
 * queries and keys divided by their root mean square per head (no weight), or (``qk_norm``) an RMS norm with a weight, per head
   with one weight for all query heads and one for all key heads, or over the whole projection at once; it comes before the rotation;
+* queries multiplied by a temperature that grows with their position p, ``1 + coef ln(floor((p + 1) / every) + 1)`` (``q_temperature``);
 * no value projection (``values_from_keys``): the keys as projected, before any norm, are the values;
 * a soft cap on the scaled score, then a term per head that grows with the distance, ``- slope[h] * (i - j)``;
 * a rotation of queries and keys by their positions before the keys are cached (``rotary``: a position encoding);
@@ -48,7 +49,7 @@ class TalkingHeadsAttention(Mixer):
     belong together share values), ``chunk`` (None: none), ``rotary`` (the description of a position encoding with a
     ``rotate``, or None), ``out_scale`` (1 by default), ``qk_norm`` (None, "head" or "projection") with ``qk_norm_eps`` and the tensors
     ``q_norm.weight`` / ``k_norm.weight`` (``[head_dim]``, or the whole projection's size), ``keep_first`` (0), ``gate_kind`` ("head" or
-    "element": ``gate.weight`` ``[heads * value_dim, dim]``), ``values_from_keys`` (False; True: no ``v.weight``). All tensors but the four matrices are optional. Tensors: ``q.weight``, ``k.weight``, ``v.weight``, ``out.weight`` (``[out, in]``), their
+    "element": ``gate.weight`` ``[heads * value_dim, dim]``), ``values_from_keys`` (False; True: no ``v.weight``), ``q_temperature`` (None, or ``{"coef", "every"}``; with ``qk_norm`` "projection"). All tensors but the four matrices are optional. Tensors: ``q.weight``, ``k.weight``, ``v.weight``, ``out.weight`` (``[out, in]``), their
     optional ``.bias``, optional ``gate.weight`` ``[heads, dim]``, ``talk`` ``[heads, heads]``, ``value_mix.weight`` (one number), ``sinks`` ``[heads]``."""
 
     graph_safe = True
@@ -72,6 +73,10 @@ class TalkingHeadsAttention(Mixer):
         if self.qk_norm is not None and self.unit_norm_eps is not None:
             raise ValueError("attention: queries and keys are normed once: unit_norm_eps or qk_norm")
         self.qk_norm_eps = float(p.get("qk_norm_eps", 0.0))
+        temp = p.get("q_temperature")
+        self.q_temperature = None if temp is None else (float(temp["coef"]), float(temp["every"]))
+        if self.q_temperature is not None and self.qk_norm != "projection":
+            raise ValueError("attention: the queries' temperature is part of the norm over the whole projection")
         self.gate_elements = p.get("gate_kind", "head") == "element"
         self.values_from_keys = bool(p.get("values_from_keys", False))
         if self.values_from_keys and self.value_dim != self.head_dim:
@@ -201,6 +206,8 @@ class TalkingHeadsAttention(Mixer):
             # one statistic over all heads of a token; the rotation behind it and, for single tokens, the write into the pages are the same kernel
             turns = rot_known and getattr(self.rotary, "magnitude", 1.0) == 1.0
             rot = {"freqs": self.rotary.freqs, "positions": ctx.attention.positions, "half": self.rotary.layout == "half"} if turns else {}
+            if self.q_temperature is not None:  # a factor on the whole query: it commutes with the rotation
+                rot.update(temperature=self.q_temperature, positions=ctx.attention.positions)
             written = single and self.value_mix is None and (turns or self.rotary is None)
             pages = {"v": v, "value_dim": self.value_dim, "k_pages": unit.k_pages, "v_pages": unit.v_pages, "dest": g.dest, "page_size": g.page_size} if written else {}
             K.projection_norm_rotate(q, k, self.n_heads, self.n_kv_heads, self.head_dim, self.qk_norm_eps, self.q_norm_weight, self.k_norm_weight,

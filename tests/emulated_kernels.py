@@ -14,6 +14,8 @@ import numpy as np
 import torch
 import torch.nn.functional as F
 
+from levanter_amd.kernels.library import PendingSumNorm
+
 
 def _act(name):
     return {
@@ -108,7 +110,44 @@ class EmulatedKernels:
             y = F.layer_norm(src, (src.shape[-1],), weight, bias, eps)
         out.copy_(y.to(out.dtype))
 
+    # ---- a stream that is normed behind every sum
+    @staticmethod
+    def _row_norm(v, norm):
+        w, b, eps, rms = norm
+        if not rms:
+            v = v - v.mean(-1, keepdim=True)
+        y = v / torch.sqrt((v * v).mean(-1, keepdim=True) + eps) * w
+        return y if b is None else y + b
+
+    def sum_norm_step(self, x, *, alpha=1.0, y=None, product=None, experts=None, write_norm=None, norm=None, h_out=None, rows=None, defer=False,
+                      pending=None):
+        assert product is None, "this stand-in never leaves a product unfinished"
+        if defer:
+            return PendingSumNorm(x, alpha, y, None, experts, write_norm)
+        if pending is not None:
+            assert pending.out is x and write_norm is None
+            alpha, y, experts, write_norm = pending.alpha, pending.y, pending.experts, pending.norm
+        cur = x
+        if write_norm is not None:
+            v = alpha * x
+            if y is not None:
+                v = v + y
+            if experts is not None:
+                s = torch.zeros_like(x)
+                self.moe_combine(experts.expert_out, experts.pos_of, experts.weights, s)
+                v = v + s
+            cur = self._row_norm(v, write_norm)
+            if rows is None:
+                x.copy_(cur)
+        if h_out is not None:
+            src = cur if rows is None else cur[rows.long()]
+            h_out.copy_((src if norm is None else self._row_norm(src, norm)).to(h_out.dtype))
+        return None
+
     def finish(self, pending) -> None:
+        if isinstance(pending, PendingSumNorm):
+            self.sum_norm_step(pending.out, pending=pending)
+            return
         if hasattr(pending, "post_weight"):
             self.group_norm_step(pending.out, groups=pending.groups, eps=pending.eps, pending=pending)
             return
@@ -152,11 +191,13 @@ class EmulatedKernels:
     # ---- block-diagonal products
     BLOCK_LINEAR_MAX_ROWS = 128
 
-    def block_linear(self, a, w, bias, out) -> None:
+    def block_linear(self, a, w, bias, out, gate=None) -> None:
         B, n_out, n_in = w.shape
         y = torch.einsum("tbi,boi->tbo", a.float().view(a.shape[0], B, n_in), w.float()).reshape(a.shape[0], B * n_out)
         if bias is not None:
             y = y + bias
+        if gate is not None:
+            y = y * torch.sigmoid(gate.float())
         out.copy_(y.to(out.dtype))
 
     # ---- the recurrent branch
@@ -232,12 +273,12 @@ class EmulatedKernels:
         return None
 
     # ---- rotation, rotate-half layout
-    def rotary_half(self, x, n_heads, head_stride, offset, freqs, positions) -> None:
+    def rotary_half(self, x, n_heads, head_stride, offset, freqs, positions, magnitude=1.0) -> None:
         n = freqs.numel()
         if n == 0:
             return
         a = positions.float()[:, None] * freqs[None, :]
-        cos, sin = torch.cos(a)[:, None, :], torch.sin(a)[:, None, :]
+        cos, sin = (torch.cos(a) * magnitude)[:, None, :], (torch.sin(a) * magnitude)[:, None, :]
         v = x[:, :n_heads * head_stride].view(x.shape[0], n_heads, head_stride)
         lo, hi = v[:, :, offset:offset + n].float().clone(), v[:, :, offset + n:offset + 2 * n].float().clone()
         v[:, :, offset:offset + n] = (lo * cos - hi * sin).to(x.dtype)
@@ -340,7 +381,7 @@ class EmulatedKernels:
         out.copy_((F.gelu(z.float(), approximate="tanh") * table[tokens.long()].float()).to(out.dtype))
 
     def projection_norm_rotate(self, q, k, n_heads, n_kv_heads, head_dim, eps, q_weight, k_weight, q_norm_dim=None, k_norm_dim=None, freqs=None, positions=None,
-                               half=False, v=None, value_dim=0, k_pages=None, v_pages=None, dest=None, page_size=0) -> None:
+                               half=False, v=None, value_dim=0, k_pages=None, v_pages=None, dest=None, page_size=0, temperature=None) -> None:
         kk = k.clone() if k_pages is not None else k
         for t, n, w in ((q, q_norm_dim, q_weight), (kk, k_norm_dim, k_weight)):
             self.head_prepare(t, 1, t.shape[1], eps, norm_dim=n, norm_weight=w)
@@ -350,6 +391,9 @@ class EmulatedKernels:
                 self.rotary_half(kk, n_kv_heads, head_dim, 0, freqs, positions)
             else:
                 self.rotary_pairs(q, kk, head_dim, freqs, positions)
+        if temperature is not None:
+            coef, every = temperature
+            q.copy_((q.float() * (1.0 + coef * torch.log(torch.floor((positions.float() + 1.0) / every) + 1.0))[:, None]).to(q.dtype))
         if k_pages is not None:
             self.kv_write(kk, v, k_pages, v_pages, dest, n_kv_heads, head_dim, page_size, value_dim=value_dim)
 
@@ -361,10 +405,10 @@ class EmulatedKernels:
         y.copy_(y + s if accumulate else s)
 
     # ---- mixture of experts
-    def moe_route(self, z, correction, chosen, weights, *, n_groups=1, keep=1, group_top=2, renormalize=False, softmax=False) -> None:
+    def moe_route(self, z, correction, chosen, weights, *, n_groups=1, keep=1, group_top=2, renormalize=False, scoring="sigmoid") -> None:
         T, E = z.shape
         top = chosen.shape[1]
-        s = torch.softmax(z.float(), -1) if softmax else torch.sigmoid(z.float())
+        s = z.float() if scoring == "softmax_chosen" else torch.softmax(z.float(), -1) if scoring == "softmax" else torch.sigmoid(z.float())
         c = s if correction is None else s + correction
         per = E // n_groups
         for t in range(T):
@@ -377,7 +421,7 @@ class EmulatedKernels:
             order = sorted(range(E), key=lambda e: (-float(ct[e]), e))[:top]
             chosen[t] = torch.tensor(order, dtype=torch.int32)
             wt = s[t][order]
-            weights[t] = wt / wt.sum() if renormalize else wt
+            weights[t] = torch.softmax(wt, -1) if scoring == "softmax_chosen" else wt / wt.sum() if renormalize else wt
 
     @staticmethod
     def moe_tile_rows(pairs, n_experts) -> int:
@@ -415,6 +459,8 @@ class EmulatedKernels:
                 if limit > 0:
                     gt, up = gt.clamp(max=limit), up.clamp(-limit, limit)
                 y = _act(activation)(gt) * (up + up_shift)
+            else:
+                y = _act(activation)(y)
             out[pos] = y.to(out.dtype)
 
     def moe_combine(self, expert_out, pos_of, weights, y, accumulate=False, chosen=None, n_real=0, identity_in=None) -> None:
@@ -540,13 +586,13 @@ class EmulatedKernels:
         self.kv_write(c, c, k_pages, v_pages, dest, 1, c.shape[1], page_size)
 
     def latent_rope_write(self, kv, latent_dim, weight, eps, norm_dim, q, n_heads, q_head, q_offset, freqs, positions, k_pages, v_pages, dest,
-                          page_size) -> None:
+                          page_size, magnitude=1.0) -> None:
         KD = kv.shape[1]
         self.head_prepare(kv, 1, latent_dim, eps, norm_dim=norm_dim, norm_weight=weight)
         if freqs is not None and freqs.numel():
-            self.rotary_half(kv, 1, KD, latent_dim, freqs, positions)
+            self.rotary_half(kv, 1, KD, latent_dim, freqs, positions, magnitude)
             if q is not None:
-                self.rotary_half(q, n_heads, q_head, q_offset, freqs, positions)
+                self.rotary_half(q, n_heads, q_head, q_offset, freqs, positions, magnitude)
         self.kv_write(kv, kv[:, :latent_dim], k_pages, v_pages, dest, 1, KD, page_size, value_dim=latent_dim)
 
     def recurrent_tokens(self, x, y, taps, conv_bias, gate_weight, gate_bias, decay, state, token_slots, out, out_scale=1.0) -> None:

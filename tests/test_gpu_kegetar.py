@@ -317,7 +317,7 @@ def test_the_router_with_softmax_scores_and_groups_scored_by_their_best(T, N, G,
     z[0] = 0.0  # equal scores: the correction alone decides
     chosen = torch.empty(T, top, dtype=torch.int32, device=DEV)
     weights = torch.empty(T, top, device=DEV)
-    K().moe_route(dev(z), dev(corr), chosen, weights, n_groups=G, keep=keep, group_top=1, softmax=True)
+    K().moe_route(dev(z), dev(corr), chosen, weights, n_groups=G, keep=keep, group_top=1, scoring="softmax")
     want_c, want_w, margin = P.route(z.double(), corr.double(), top, G, keep)
     clear = margin > 1e-5
     assert clear.sum() >= T // 2
