@@ -55,7 +55,7 @@ def main() -> int:
     ap.add_argument("--shape", default="7b", choices=["7b", "xl", "20b"],
                     help="layer sizes of the decode workload: 7b is the headline's; xl and 20b measure the same step at the other "
                          "sizes of the reference's configurations (use --no-points: the prefill point is 2,048 tokens)")
-    ap.add_argument("--workload", default="decode", choices=["decode", "xl_mix", "20b", "zederax", "nakurax", "tativik", "kegetar", "lelatar"],
+    ap.add_argument("--workload", default="decode", choices=["decode", "xl_mix", "20b", "zederax", "nakurax", "tativik", "kegetar", "lelatar", "kelasun"],
                     help="decode: the workload described above. xl_mix / 20b: continuous-batching workloads at the gpt2_xl and gpt2_20b sizes "
                          "through InferenceEngine.generate; they print their own line. zederax: prefill and decode rates of Zederax "
                          "layers at a few sizes beside GPT-2 layers of the same width, heads and inner width; its own line. nakurax: the same for "
@@ -64,11 +64,12 @@ def main() -> int:
                          "kegetar: Kegetar layers (windowed attention that keeps the first positions beside gated linear attention, and attention whose "
                          "keys are its values, in turn; dense and routed feed-forwards in turn) beside Tativik layers. lelatar: Lelatar layers (attention with sinks "
                          "beside a gated delta rule with a dense feed-forward, and state-space duality, in turn, two layers looped, a token input a layer) beside "
-                         "Kegetar layers")
+                         "Kegetar layers. kelasun: Kelasun layers (attention with a distance term and sinks, and latent attention with a rotated key "
+                         "part, in turn, routed experts without gates beside a shared one, a norm behind every sum) beside Tativik and Kegetar layers")
     ap.add_argument("--sizes", default="1k,2k,4k", help="with --workload zederax / nakurax: which of the sizes 1k, 2k, 4k to run")
     ap.add_argument("--batches", default="1,8,64", help="with --workload zederax: decode batch sizes to time ('' for none)")
     ap.add_argument("--no-prefill", action="store_true", help="with --workload zederax: skip the 2,048-token prompt")
-    ap.add_argument("--arch", default="both", choices=["both", "zederax", "gpt2", "nakurax", "tativik", "kegetar", "lelatar"],
+    ap.add_argument("--arch", default="both", choices=["both", "zederax", "gpt2", "nakurax", "tativik", "kegetar", "lelatar", "kelasun"],
                     help="with --workload zederax / nakurax: one architecture only (for profiling)")
     args = ap.parse_args()
     if args.gpus != 1:
@@ -80,7 +81,7 @@ def main() -> int:
     from levanter_amd.config import InferenceEngineConfig, LmConfig
     from levanter_amd.engine import InferenceEngine, Request
 
-    if args.workload in ("zederax", "nakurax", "tativik", "kegetar", "lelatar"):
+    if args.workload in ("zederax", "nakurax", "tativik", "kegetar", "lelatar", "kelasun"):
         return zederax_workload(args)
     if args.workload != "decode":
         return serving_workload(args)
@@ -409,6 +410,24 @@ def lelatar_config(z):
             "loop": {"start": start, "stop": start + 2, "times": 2}, "token_side": {"dim": z["width"] // 16}}
 
 
+def kelasun_config(z):
+    """Layers of attention with a distance term, sinks and a temperature and layers of latent attention (queries through a latent, a rotated
+    key part of 32 with stretched frequencies, a gate per element), in turn; the heads, head sizes and layer count of the size, the latents
+    of Tativik's layers above (three key heads' size, at most 224; half the width for the queries). The feed-forward has 32 experts of a
+    quarter of the size's inner width, 4 a token, and a shared one of the same width."""
+    import math
+
+    rot = 32
+    attention = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["vdim"], "scale": 1.0 / math.sqrt(z["dim"]), "q_temp": {"coef": 0.1, "every": 2048}}
+    latent = {"heads": z["heads"], "dim": z["dim"], "rot_dim": rot, "vdim": z["vdim"], "kv_rank": min(224, 3 * z["dim"]), "q_rank": z["width"] // 2,
+              "scale": 1.0 / math.sqrt(z["dim"] + rot),
+              "rot": {"dims": rot, "base": 500000.0, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    mlp = {"kind": "moe", "expert": {"ff": z["ff"] // 4}, "router": {"experts": 32, "top": 4}, "shared": {"ff": z["ff"] // 4}}
+    layers = [json.loads(json.dumps({"type": "attention" if i % 2 == 0 else "latent_attention", "mixer": attention if i % 2 == 0 else latent, "mlp": mlp}))
+              for i in range(z["layers"])]
+    return {"architecture": "Kelasun", "vocab": ZEDERAX_VOCAB, "width": z["width"], "norm": {"eps": 1e-6}, "postln_alpha": 2.0, "logit_scale": 0.5, "layers": layers}
+
+
 def zederax_workload(args) -> int:
     """Prefill (one 2,048-token prompt) and decode (batch 1, 8, 64 after 512-token prompts) through the engine, for Zederax
     (or, with --workload nakurax, Nakurax and Zederax) and for GPT-2 at equal sizes. One JSON line."""
@@ -486,11 +505,14 @@ def zederax_workload(args) -> int:
             archs = [("kegetar", kegetar_config(z)), ("tativik", tativik_config(z))]
         if args.workload == "lelatar":  # beside the closest model: Kegetar's attention beside a recurrence with a matrix state, gated feed-forwards
             archs = [("lelatar", lelatar_config(z)), ("kegetar", kegetar_config(z))]
+        if args.workload == "kelasun":  # beside the closest models: Tativik's latent attention and experts, Kegetar's attention with a distance term
+            archs = [("kelasun", kelasun_config(z)), ("tativik", tativik_config(z)), ("kegetar", kegetar_config(z))]
         for arch, raw in archs:
             if args.arch in ("both", arch):
                 print(f"[bench] {arch} at size {name} ...", file=sys.stderr, flush=True)
                 results[name][arch] = measure(raw)
-    print(json.dumps({"metric": ("prefill and decode tok/s of Lelatar layers beside Kegetar layers of equal width, heads and head sizes" if args.workload == "lelatar" else
+    print(json.dumps({"metric": ("prefill and decode tok/s of Kelasun layers beside Tativik and Kegetar layers of equal width, heads and head sizes" if args.workload == "kelasun" else
+                                 "prefill and decode tok/s of Lelatar layers beside Kegetar layers of equal width, heads and head sizes" if args.workload == "lelatar" else
                                  "prefill and decode tok/s of Kegetar layers beside Tativik layers of equal width, heads and head sizes" if args.workload == "kegetar" else
                                  f"prefill and decode tok/s of Tativik layers beside Nakurax layers of equal width, heads and (per token) inner width" if args.workload == "tativik" else
                                  f"prefill and decode tok/s of {args.workload.capitalize()} layers beside {'Zederax and ' if args.workload == 'nakurax' else ''}GPT-2 layers of equal width, heads and inner width"),

@@ -27,6 +27,21 @@ def rounded_products():
         _ROUND = was
 
 
+_MARGINS: Optional[List[torch.Tensor]] = None
+
+
+@contextlib.contextmanager
+def close_calls():
+    """Collects, router by router, how far apart the last chosen and the first left-out logit of every token are (infinitely far where
+    every expert is chosen): where they nearly tie, another rounding chooses another expert and gets another result."""
+    global _MARGINS
+    was, _MARGINS = _MARGINS, []
+    try:
+        yield _MARGINS
+    finally:
+        _MARGINS = was
+
+
 def lin(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     """w x for every row of x (weights are stored [out, in])."""
     return _ROUND(_ROUND(x) @ w.T)
@@ -157,6 +172,9 @@ def expert(h: torch.Tensor, W: Dict[str, torch.Tensor], p: str) -> torch.Tensor:
 
 def route(z: torch.Tensor, top: int) -> Tuple[torch.Tensor, torch.Tensor]:
     """Router logits ``[T, E]`` -> the ``top`` experts of each token and their weights, the softmax of the chosen logits alone."""
+    if _MARGINS is not None:
+        order = z.sort(-1, descending=True).values
+        _MARGINS.append(order[:, top - 1] - order[:, top] if top < z.shape[1] else torch.full((z.shape[0],), math.inf, dtype=F64))
     best = z.topk(top, dim=-1)
     return best.indices, torch.softmax(best.values, -1)
 
