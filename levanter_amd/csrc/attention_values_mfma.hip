@@ -249,6 +249,7 @@ attention_values_mfma_kernel(const bf16_t* __restrict__ q, long q_stride, float*
 // (requested two blocks ahead, while the blocks before are computed) -> LDS, keys as [HD/8][64][8], values transposed as
 // [value head][VD][64 + 8] with everything beyond the last written key made zero on the way.
 #define VS_STRIDE 72
+#define RUN_MAX_LDS (80 * 1024)  // bytes a workgroup may take: two workgroups a CU
 #define RUN_PAGES 2048  // page ids of a tile's key range that are kept in LDS
 #define K_STAGE ((HD * 8 + PF_THREADS - 1) / PF_THREADS)        // 16-byte chunks of a key block per thread
 #define V_STAGE ((NVC * VD * 8 + PF_THREADS - 1) / PF_THREADS)  // and of the value blocks
@@ -524,11 +525,16 @@ extern "C" int lev_attention_values_mfma(const void* q, long q_stride, float* ou
     long reach = window > 0 && window < max_keys ? window : max_keys;
     if (chunk > 0 && chunk < reach) reach = chunk;
     reach += PF_ROWS + 64 + (keep > 0 ? keep + 64 + PS : 0);
-    if (lds + RUN_PAGES * sizeof(int) <= 64 * 1024 && reach / PS + 2 <= RUN_PAGES)
+    const size_t all_lds = lds + RUN_PAGES * sizeof(int);
+    if (all_lds > 64 * 1024 && all_lds <= RUN_MAX_LDS) {  // more than a kernel gets unasked
+      hipError_t e = hipFuncSetAttribute((const void*)attention_values_mfma_runs_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      LEV_REQUIRE(e == hipSuccess, "attention: %zu bytes of LDS a workgroup: %s", all_lds, hipGetErrorString(e));
+    }
+    if (all_lds <= RUN_MAX_LDS && reach / PS + 2 <= RUN_PAGES)
       attention_values_mfma_runs_kernel<<<grid, PF_THREADS, lds, stream>>>((const bf16_t*)q, q_stride, out, (const bf16_t*)k_pages,
                                                                          (const bf16_t*)v_pages, positions, token_seq, block_tables,
                                                                          bt_stride, tiles, H, KVH, NV, PS, scale, window, chunk, keep, softcap, slopes, sinks);
-    else  // the largest head sizes, the longest ranges: every wave by itself, operands straight from the pages
+    else  // the longest ranges: every wave by itself, operands straight from the pages
       attention_values_mfma_kernel<false><<<dim3(n_tiles * SUB_TILES, H, chunks), 64, 0, stream>>>(
           (const bf16_t*)q, q_stride, out, (const bf16_t*)k_pages, (const bf16_t*)v_pages, positions, token_seq, block_tables, bt_stride,
           tiles, H, KVH, NV, PS, scale, window, chunk, keep, softcap, slopes, 1, nullptr, nullptr, sinks);

@@ -8,13 +8,12 @@
 //             lower index); the weights are the winners' s (times 1 / their sum if `renormalize`), in the order of falling c.
 //   sort      the T * top (token, choice) pairs by expert: sorted[pos] = pair, pos_of[pair] = pos, and a list of row tiles
 //             (expert, first position, rows <= tile_rows) that covers every expert's stretch; n_tiles on the device.
-//             tile_rows is 16, or 64 for steps with many rows an expert (a wave then runs four row tiles on every weight
-//             fragment it loads).
+//             tile_rows is 16, or 128 for steps with many rows an expert.
 //   linear    for every tile: out[pos][o] = sum_k w[expert][o][k] a[row(pos)][k], row(pos) = the pair's token (gather) or pos
 //             itself, through the activation (none for the second product); with glu the expert's matrix is [gate ; up] (2F rows) and
 //             out[pos][f] = act(gate_f) * up_f.
 //             bfloat16 on the matrix cores (16x16x32): few tiles of 16 rows with K split over a workgroup's waves, many with a
-//             wave per tile, tiles of 64 rows with both operands staged through LDS; float32 in plain arithmetic. Workgroups
+//             wave per tile, tiles of 128 rows with both operands staged through LDS; float32 in plain arithmetic. Workgroups
 //             beyond n_tiles return at once.
 //             with limit > 0 the gate sum is capped at limit and the up sum clamped to +-limit first, and up_shift is added to
 //             the up sum: act(min(gate, limit)) * (clamp(up) + up_shift).
@@ -23,32 +22,41 @@
 //             places but no tiles (the products never see them), and combine takes the token's own row of `identity_in` for them.
 #include "common.h"
 
-#define MOE_TM 16          // rows of a matrix-core row tile; a tile of the list has tile_rows = MOE_TM or 4 * MOE_TM rows
+#define MOE_TM 16          // rows of a matrix-core row tile, and of a tile of the list in steps of few tokens
+#define MOE_BIG 128        // rows of a tile of the list in the others
 #define MOE_MAX_E 1024     // experts
 #define MOE_MAX_TOP 32
 
 // ---- route ------------------------------------------------------------------------------------
-__global__ void __launch_bounds__(64)
-moe_route_kernel(const float* __restrict__ z, long z_stride, const float* __restrict__ correction, int E, int G, int keep, int group_top, int top,
-                 int renormalize, int scoring, int* __restrict__ chosen, float* __restrict__ weights) {
-  __shared__ float s_s[MOE_MAX_E], c_s[MOE_MAX_E], g_s[MOE_MAX_E];
-  __shared__ int sel[MOE_MAX_TOP];
-  const int t = blockIdx.x, lane = threadIdx.x;
+// One wave routes one token; s_s, c_s (and g_s with groups) are E (G) numbers, sel MOE_MAX_TOP numbers of its own in LDS. Every wave of
+// the workgroup passes the same barriers. `extra`: a further choice behind the `top` ones, expert E with weight 1 (an expert that runs for
+// every token). store: the wave's token is one of the step's.
+struct MoeRouteArgs {
+  const float* z;
+  long z_stride;
+  const float* correction;
+  int E, G, keep, group_top, top, renormalize, scoring, extra;
+  int* chosen;
+  float* weights;
+};
+__device__ __forceinline__ void moe_route_token(const MoeRouteArgs& a, int t, bool store, float* s_s, float* c_s, float* g_s, int* sel) {
+  const int lane = threadIdx.x & 63, E = a.E, G = a.G, top = a.top;
   const int per = E / G;
+  const float* zt = a.z + (size_t)t * a.z_stride;
   float z_max = 0.f, inv_sum = 1.0f;
-  if (scoring == 1) {
+  if (a.scoring == 1) {
     float mx = -INFINITY;
-    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[(size_t)t * z_stride + e]);
+    for (int e = lane; e < E; e += 64) mx = fmaxf(mx, zt[e]);
     z_max = wave_max(mx);
     float sum = 0.f;
-    for (int e = lane; e < E; e += 64) sum += expf(z[(size_t)t * z_stride + e] - z_max);
+    for (int e = lane; e < E; e += 64) sum += expf(zt[e] - z_max);
     inv_sum = 1.0f / wave_sum(sum);
   }
   for (int e = lane; e < E; e += 64) {
-    const float ze = z[(size_t)t * z_stride + e];
-    const float s = scoring == 2 ? ze : scoring == 1 ? expf(ze - z_max) * inv_sum : 1.0f / (1.0f + expf(-ze));
+    const float ze = zt[e];
+    const float s = a.scoring == 2 ? ze : a.scoring == 1 ? expf(ze - z_max) * inv_sum : 1.0f / (1.0f + expf(-ze));
     s_s[e] = s;
-    c_s[e] = s + (correction ? correction[e] : 0.f);
+    c_s[e] = s + (a.correction ? a.correction[e] : 0.f);
   }
   __syncthreads();
   if (G > 1) {
@@ -56,7 +64,7 @@ moe_route_kernel(const float* __restrict__ z, long z_stride, const float* __rest
       float sum = 0.f;
       float last = INFINITY;
       int last_i = -1;
-      for (int n = 0; n < min(group_top, per); ++n) {  // the next largest: below (last, last_i) in the order (value falling, index rising)
+      for (int n = 0; n < min(a.group_top, per); ++n) {  // the next largest: below (last, last_i) in the order (value falling, index rising)
         float best = -INFINITY;
         int best_i = -1;
         for (int i = 0; i < per; ++i) {
@@ -75,7 +83,7 @@ moe_route_kernel(const float* __restrict__ z, long z_stride, const float* __rest
       const float mine = g_s[g];
       int ahead = 0;  // groups that come before this one
       for (int o = 0; o < G; ++o) ahead += (g_s[o] > mine || (g_s[o] == mine && o < g)) ? 1 : 0;
-      if (ahead >= keep) c_s[e] = -INFINITY;
+      if (ahead >= a.keep) c_s[e] = -INFINITY;
     }
     __syncthreads();
   }
@@ -100,87 +108,154 @@ moe_route_kernel(const float* __restrict__ z, long z_stride, const float* __rest
     wsum += s_s[best_e];
     __syncthreads();
   }
-  if (scoring == 2) {  // every lane sums the same few numbers
-    float mx = -INFINITY, sum = 0.f;
+  const size_t at = (size_t)t * (top + a.extra);
+  float mx = 0.f;
+  if (a.scoring == 2) {  // every lane sums the same few numbers
+    mx = -INFINITY, wsum = 0.f;
     for (int n = 0; n < top; ++n) mx = fmaxf(mx, s_s[sel[n]]);
-    for (int n = 0; n < top; ++n) sum += expf(s_s[sel[n]] - mx);
-    if (lane < top) {
-      const int e = sel[lane];
-      chosen[(size_t)t * top + lane] = e;
-      weights[(size_t)t * top + lane] = expf(s_s[e] - mx) / sum;
-    }
-    return;
+    for (int n = 0; n < top; ++n) wsum += expf(s_s[sel[n]] - mx);
   }
+  if (!store) return;
   if (lane < top) {
     const int e = sel[lane];
-    chosen[(size_t)t * top + lane] = e;
-    weights[(size_t)t * top + lane] = renormalize ? s_s[e] / wsum : s_s[e];
+    a.chosen[at + lane] = e;
+    a.weights[at + lane] = a.scoring == 2 ? expf(s_s[e] - mx) / wsum : a.renormalize ? s_s[e] / wsum : s_s[e];
+  } else if (lane == top && a.extra) {
+    a.chosen[at + top] = E;
+    a.weights[at + top] = 1.0f;
   }
 }
 
-extern "C" int lev_moe_route(const float* z, long z_stride, const float* correction, int T, int E, int G, int keep, int group_top, int top,
-                             int renormalize, int scoring, int* chosen, float* weights, hipStream_t stream) {
-  LEV_REQUIRE(scoring >= 0 && scoring <= 2, "experts: unknown scoring %d", scoring);
-  LEV_REQUIRE(T >= 0 && E > 0 && E <= MOE_MAX_E, "experts: %d experts (at most %d)", E, MOE_MAX_E);
-  LEV_REQUIRE(G > 0 && E % G == 0 && keep > 0 && keep <= G && group_top > 0, "experts: %d groups of %d experts, %d kept", G, E, keep);
-  LEV_REQUIRE(top > 0 && top <= MOE_MAX_TOP && top <= keep * (E / G), "experts: %d experts a token out of %d that can be chosen (at most %d)", top, keep * (E / G), MOE_MAX_TOP);
-  LEV_REQUIRE(z && chosen && weights && z_stride >= E, "experts: a tensor is missing");
-  if (T == 0) return 0;
-  moe_route_kernel<<<T, 64, 0, stream>>>(z, z_stride, correction, E, G, keep, group_top, top, renormalize, scoring, chosen, weights);
-  return lev_check_launch("moe_route");
+__global__ void __launch_bounds__(64)
+moe_route_kernel(const MoeRouteArgs a) {
+  __shared__ float s_s[MOE_MAX_E], c_s[MOE_MAX_E], g_s[MOE_MAX_E];
+  __shared__ int sel[MOE_MAX_TOP];
+  moe_route_token(a, blockIdx.x, true, s_s, c_s, g_s, sel);
 }
 
 // ---- sort --------------------------------------------------------------------------------------
 // One workgroup. meta: [0] = n_tiles; tiles: (expert, first position, rows) per tile. The order of an expert's pairs among
 // themselves is whatever the atomic counters give: a pair's results do not depend on its place in a tile.
 #define MOE_SORT_NT 1024
-__global__ void __launch_bounds__(MOE_SORT_NT)
-moe_sort_kernel(const int* __restrict__ chosen, int P, int E, int n_real, int tile_rows, int* __restrict__ sorted, int* __restrict__ pos_of,
-                int* __restrict__ tiles, int* __restrict__ meta) {
-  __shared__ int count[MOE_MAX_E], start[MOE_MAX_E], tile_start[MOE_MAX_E + 1], cursor[MOE_MAX_E];
+struct MoeSortLds {
+  int count[MOE_MAX_E + 1], start[MOE_MAX_E + 1], tile_start[MOE_MAX_E + 2], cursor[MOE_MAX_E + 1];
+};
+__device__ __forceinline__ void moe_sort_pairs(MoeSortLds& l, const int* chosen, int P, int E, int n_real, int tile_rows, int* __restrict__ sorted,
+                                               int* __restrict__ pos_of, int* __restrict__ tiles, int* __restrict__ meta) {
   const int tid = threadIdx.x;
-  for (int e = tid; e < E; e += MOE_SORT_NT) count[e] = 0, cursor[e] = 0;
+  for (int e = tid; e < E; e += MOE_SORT_NT) l.count[e] = 0, l.cursor[e] = 0;
   __syncthreads();
-  for (int p = tid; p < P; p += MOE_SORT_NT) atomicAdd(&count[chosen[p]], 1);
+  for (int p = tid; p < P; p += MOE_SORT_NT) atomicAdd(&l.count[chosen[p]], 1);
   __syncthreads();
-  if (tid == 0) {
-    int at = 0, tile = 0;
-    for (int e = 0; e < E; ++e) {
-      start[e] = at;
-      tile_start[e] = tile;
-      at += count[e];
-      if (e < n_real) tile += (count[e] + tile_rows - 1) / tile_rows;  // experts without weights get places and no tiles
+  if (tid < 64) {  // running sums over the experts: each lane a stretch of neighbours, then across the lanes
+    const int c = (E + 63) / 64, lo = min(E, tid * c), hi = min(E, lo + c);
+    int n = 0, nt = 0;
+    for (int e = lo; e < hi; ++e) {
+      n += l.count[e];
+      if (e < n_real) nt += (l.count[e] + tile_rows - 1) / tile_rows;  // experts without weights get places and no tiles
     }
-    tile_start[E] = tile;
-    meta[0] = tile;
+    int at = n, tile = nt;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const int a = __shfl_up(at, o, 64), b = __shfl_up(tile, o, 64);
+      if (tid >= o) at += a, tile += b;
+    }
+    if (tid == 63) l.tile_start[E] = tile, meta[0] = tile;
+    at -= n, tile -= nt;
+    for (int e = lo; e < hi; ++e) {
+      l.start[e] = at;
+      l.tile_start[e] = tile;
+      at += l.count[e];
+      if (e < n_real) tile += (l.count[e] + tile_rows - 1) / tile_rows;
+    }
   }
   __syncthreads();
   for (int p = tid; p < P; p += MOE_SORT_NT) {
     const int e = chosen[p];
-    const int pos = start[e] + atomicAdd(&cursor[e], 1);
+    const int pos = l.start[e] + atomicAdd(&l.cursor[e], 1);
     sorted[pos] = p;
     pos_of[p] = pos;
   }
   for (int e = tid; e < E; e += MOE_SORT_NT) {
-    const int n = tile_start[e + 1] - tile_start[e];
+    const int n = l.tile_start[e + 1] - l.tile_start[e];
     for (int i = 0; i < n; ++i) {
-      int* tl = tiles + 3 * (size_t)(tile_start[e] + i);
+      int* tl = tiles + 3 * (size_t)(l.tile_start[e] + i);
       tl[0] = e;
-      tl[1] = start[e] + i * tile_rows;
-      tl[2] = min(tile_rows, count[e] - i * tile_rows);
+      tl[1] = l.start[e] + i * tile_rows;
+      tl[2] = min(tile_rows, l.count[e] - i * tile_rows);
     }
   }
 }
 
+__global__ void __launch_bounds__(MOE_SORT_NT)
+moe_sort_kernel(const int* __restrict__ chosen, int P, int E, int n_real, int tile_rows, int* __restrict__ sorted, int* __restrict__ pos_of,
+                int* __restrict__ tiles, int* __restrict__ meta) {
+  __shared__ MoeSortLds l;
+  moe_sort_pairs(l, chosen, P, E, n_real, tile_rows, sorted, pos_of, tiles, meta);
+}
+
+// Both for a step of few tokens, in one workgroup: a wave routes a token, then all of them sort.
+#define MOE_SMALL_T (MOE_SORT_NT / 64)
+#define MOE_SMALL_E 256
+__global__ void __launch_bounds__(MOE_SORT_NT)
+moe_route_sort_kernel(const MoeRouteArgs a, int T, int n_real, int tile_rows, int* __restrict__ sorted, int* __restrict__ pos_of, int* __restrict__ tiles,
+                      int* __restrict__ meta) {
+  __shared__ MoeSortLds l;
+  __shared__ float s_s[MOE_SMALL_T][MOE_SMALL_E], c_s[MOE_SMALL_T][MOE_SMALL_E];
+  __shared__ int sel[MOE_SMALL_T][MOE_MAX_TOP];
+  const int wave = threadIdx.x >> 6;
+  // the groups' scores take the place of the sort's counters, which nobody needs before the routing is done
+  float* g_s = reinterpret_cast<float*>(l.count) + (size_t)wave * MOE_SMALL_E / 4;
+  moe_route_token(a, min(wave, T - 1), wave < T, s_s[wave], c_s[wave], g_s, sel[wave]);
+  __syncthreads();  // the choices, in global memory, are the whole workgroup's
+  moe_sort_pairs(l, a.chosen, T * (a.top + a.extra), a.E + a.extra, n_real, tile_rows, sorted, pos_of, tiles, meta);
+}
+
+static int moe_route_check(const MoeRouteArgs& a, int T) {
+  LEV_REQUIRE(a.scoring >= 0 && a.scoring <= 2, "experts: unknown scoring %d", a.scoring);
+  LEV_REQUIRE(T >= 0 && a.E > 0 && a.E <= MOE_MAX_E, "experts: %d experts (at most %d)", a.E, MOE_MAX_E);
+  LEV_REQUIRE(a.G > 0 && a.E % a.G == 0 && a.keep > 0 && a.keep <= a.G && a.group_top > 0, "experts: %d groups of %d experts, %d kept", a.G, a.E, a.keep);
+  LEV_REQUIRE(a.top > 0 && a.top <= MOE_MAX_TOP && a.top <= a.keep * (a.E / a.G), "experts: %d experts a token out of %d that can be chosen (at most %d)", a.top,
+              a.keep * (a.E / a.G), MOE_MAX_TOP);
+  LEV_REQUIRE(a.extra == 0 || a.extra == 1, "experts: one further choice at most");
+  LEV_REQUIRE(a.z && a.chosen && a.weights && a.z_stride >= a.E, "experts: a tensor is missing");
+  return 0;
+}
+
+extern "C" int lev_moe_route(const float* z, long z_stride, const float* correction, int T, int E, int G, int keep, int group_top, int top,
+                             int renormalize, int scoring, int extra, int* chosen, float* weights, hipStream_t stream) {
+  const MoeRouteArgs a{z, z_stride, correction, E, G, keep, group_top, top, renormalize, scoring, extra, chosen, weights};
+  if (moe_route_check(a, T)) return -1;
+  if (T == 0) return 0;
+  moe_route_kernel<<<T, 64, 0, stream>>>(a);
+  return lev_check_launch("moe_route");
+}
+
 extern "C" int lev_moe_max_tiles(int P, int E, int tile_rows) { return P / tile_rows + E + 1; }
 
-extern "C" int lev_moe_sort(const int* chosen, int P, int E, int n_real, int tile_rows, int* sorted, int* pos_of, int* tiles, int* meta, hipStream_t stream) {
-  LEV_REQUIRE(P >= 0 && E > 0 && E <= MOE_MAX_E, "experts: %d experts (at most %d)", E, MOE_MAX_E);
-  LEV_REQUIRE(tile_rows == MOE_TM || tile_rows == 4 * MOE_TM, "experts: tiles of %d rows (%d or %d)", tile_rows, MOE_TM, 4 * MOE_TM);
+static int moe_sort_check(const void* chosen, int P, int E, int n_real, int tile_rows, const void* sorted, const void* pos_of, const void* tiles, const void* meta) {
+  LEV_REQUIRE(P >= 0 && E > 0 && E <= MOE_MAX_E + 1, "experts: %d experts (at most %d)", E, MOE_MAX_E + 1);
+  LEV_REQUIRE(tile_rows == MOE_TM || tile_rows == MOE_BIG, "experts: tiles of %d rows (%d or %d)", tile_rows, MOE_TM, MOE_BIG);
   LEV_REQUIRE(chosen && sorted && pos_of && tiles && meta, "experts: a tensor is missing");
   LEV_REQUIRE(n_real >= 0 && n_real <= E, "experts: %d of %d experts have weights", n_real, E);
+  return 0;
+}
+
+extern "C" int lev_moe_sort(const int* chosen, int P, int E, int n_real, int tile_rows, int* sorted, int* pos_of, int* tiles, int* meta, hipStream_t stream) {
+  if (moe_sort_check(chosen, P, E, n_real, tile_rows, sorted, pos_of, tiles, meta)) return -1;
   moe_sort_kernel<<<1, MOE_SORT_NT, 0, stream>>>(chosen, P, E, n_real, tile_rows, sorted, pos_of, tiles, meta);
   return lev_check_launch("moe_sort");
+}
+
+// 1: not for these sizes (nothing has been launched); else as the two above, one after the other
+extern "C" int lev_moe_route_sort(const float* z, long z_stride, const float* correction, int T, int E, int G, int keep, int group_top, int top,
+                                  int renormalize, int scoring, int extra, int* chosen, float* weights, int n_real, int tile_rows, int* sorted, int* pos_of,
+                                  int* tiles, int* meta, hipStream_t stream) {
+  const MoeRouteArgs a{z, z_stride, correction, E, G, keep, group_top, top, renormalize, scoring, extra, chosen, weights};
+  if (moe_route_check(a, T) || moe_sort_check(chosen, T * (top + extra), E + extra, n_real, tile_rows, sorted, pos_of, tiles, meta)) return -1;
+  if (T == 0 || T > MOE_SMALL_T || E > MOE_SMALL_E || G > MOE_SMALL_E / 4) return 1;
+  moe_route_sort_kernel<<<1, MOE_SORT_NT, 0, stream>>>(a, T, n_real, tile_rows, sorted, pos_of, tiles, meta);
+  return lev_check_launch("moe_route_sort");
 }
 
 // ---- the experts' products ------------------------------------------------------------------------
@@ -347,92 +422,134 @@ moe_linear_splitk_kernel(const bf16_t* __restrict__ a, long a_stride, const bf16
   }
 }
 
-// Tiles of 64 rows (prompts): a workgroup of four waves owns a tile's 64 rows and 128 outputs (with glu: 128 of gate and the same
-// 128 of up); the rows' and the weights' k-steps of 32 go from global memory into registers one step ahead and from there into
-// LDS (two buffers, rows 40 elements apart so that the fragments' 16-byte reads spread over the banks), and every wave takes
-// its fragments from there: a weight or activation byte is fetched once a workgroup instead of once a wave.
-#define MOE_BN 128
-#define MOE_LD 40
-template <typename TO, bool GLU>
-__global__ void __launch_bounds__(256)
-moe_linear_tile_kernel(const bf16_t* __restrict__ a, long a_stride, const bf16_t* __restrict__ w, TO* __restrict__ out, long o_stride,
-                       const int* __restrict__ tiles, const int* __restrict__ meta, const int* __restrict__ sorted, int top, int gather,
-                       int K, int N, int F, int act, float limit, float up_shift) {
-  constexpr int WR = GLU ? 2 * MOE_BN : MOE_BN, WL = WR / 64;  // weight rows of a workgroup, loads of them per thread and k-step
-  __shared__ __attribute__((aligned(16))) bf16_t sa[2][64][MOE_LD];
-  __shared__ __attribute__((aligned(16))) bf16_t sw[2][WR][MOE_LD];
-  const int tile = blockIdx.x;
-  if (tile >= meta[0]) return;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
-  const int o0 = blockIdx.y * MOE_BN;
-  const int e = tiles[3 * tile], first = tiles[3 * tile + 1], rows = tiles[3 * tile + 2];
-  // what this thread fetches: 8 elements of one activation row and of WL weight rows per k-step
-  const int lrow = tid >> 2, lk = (tid & 3) * 8;
-  const int pos = first + min(lrow, rows - 1);  // rows beyond the tile: read again, never stored
-  const bf16_t* ap = a + (size_t)(gather ? sorted[pos] / top : pos) * a_stride;
-  const bf16_t* wp[WL];
+// Tiles of 128 rows (prompts, large batches): a workgroup of four waves owns 128 rows and 128 weight rows (with glu: 64 outputs' gate
+// rows and the same outputs' up rows), a wave 64 x 64 of them, so that a fragment from LDS feeds four products. K goes by in steps of 64,
+// two steps on their way in registers and two buffers in LDS (rows 72 elements apart), one barrier a step. Rows beyond the tile are
+// read again and never stored; a wave whose 64 rows all lie beyond it does not compute. The workgroups of a tile and of its neighbours
+// in the list (an expert's rows, its weights) follow each other on one of the eight chiplets (workgroups are dealt to them in turn).
+#define MOE_BIG_K 64
+#define MOE_BIG_LD (MOE_BIG_K + 8)
+#define MOE_BIG_LDS (2 * 2 * MOE_BIG * MOE_BIG_LD * (int)sizeof(bf16_t))
+template <typename TO>
+__device__ __forceinline__ void moe_store4(TO* p, const float (&v)[4], int n, bool vec);
+template <>
+__device__ __forceinline__ void moe_store4<float>(float* p, const float (&v)[4], int n, bool vec) {
+  if (vec && n >= 4) *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+  else
 #pragma unroll
-  for (int i = 0; i < WL; ++i) {
-    const int r = lrow + 64 * i;  // row of the workgroup's weight tile: gate rows, then (glu) up rows
-    const int o = min(o0 + (r % MOE_BN), F - 1) + (r >= MOE_BN ? F : 0);
-    wp[i] = w + (size_t)e * N * K + (size_t)o * K;
+    for (int r = 0; r < 4; ++r)
+      if (r < n) p[r] = v[r];
+}
+template <>
+__device__ __forceinline__ void moe_store4<bf16_t>(bf16_t* p, const float (&v)[4], int n, bool vec) {
+  if (vec && n >= 4) *reinterpret_cast<uint2*>(p) = make_uint2(float2_to_bf16x2(v[0], v[1]), float2_to_bf16x2(v[2], v[3]));
+  else
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (r < n) p[r] = float_to_bf16(v[r]);
+}
+
+template <typename TO, bool GLU>
+__global__ void __launch_bounds__(256, 2)
+moe_linear_big_kernel(const bf16_t* __restrict__ a, long a_stride, const bf16_t* __restrict__ w, TO* __restrict__ out, long o_stride,
+                      const int* __restrict__ tiles, const int* __restrict__ meta, const int* __restrict__ sorted, int top, int gather,
+                      int K, int N, int F, int act, float limit, float up_shift, int n_cols, int vec) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char moe_smem[];
+  bf16_t* sa = reinterpret_cast<bf16_t*>(moe_smem);    // [2][128][72]
+  bf16_t* sw = sa + 2 * MOE_BIG * MOE_BIG_LD;          // [2][128][72]
+  constexpr int BN = GLU ? MOE_BIG / 2 : MOE_BIG;      // outputs of a workgroup
+  const int n_tiles = meta[0], per = (n_tiles + 7) / 8;
+  if (per == 0) return;
+  const int slot = blockIdx.x >> 3, tile = (blockIdx.x & 7) * per + slot % per, ycol = slot / per;
+  if (ycol >= n_cols || tile >= n_tiles) return;  // the whole workgroup
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, col = lane & 15, g = lane >> 4;
+  const int wr = wave >> 1, wc = wave & 1;
+  const int o0 = ycol * BN;
+  const int e = tiles[3 * tile], first = tiles[3 * tile + 1], rows = tiles[3 * tile + 2];
+  // what this thread fetches: a chunk of 8 elements of four activation rows and of four weight rows per step
+  const int lrow = tid >> 3, lk = (tid & 7) * 8;
+  const bf16_t *ap[4], *wp[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int r = lrow + 32 * i;
+    const int pos = first + min(r, rows - 1);
+    ap[i] = a + (size_t)(gather ? sorted[pos] / top : pos) * a_stride;
+    const int o = min(o0 + (r % BN), F - 1) + (r >= BN ? F : 0);
+    wp[i] = w + ((size_t)e * N + o) * K;
   }
-  moe_f32x4 acc[4][2], acc_up[4][2];
+  moe_f32x4 acc[4][4];
 #pragma unroll
   for (int rt = 0; rt < 4; ++rt)
 #pragma unroll
-    for (int nt = 0; nt < 2; ++nt) acc[rt][nt] = acc_up[rt][nt] = moe_f32x4{0.f, 0.f, 0.f, 0.f};
-  moe_u32x4 ra, rw[WL];
-  auto fetch = [&](int k0) {
+    for (int nt = 0; nt < 4; ++nt) acc[rt][nt] = moe_f32x4{0.f, 0.f, 0.f, 0.f};
+  moe_u32x4 ra0[4], rw0[4], ra1[4], rw1[4];
+  auto fetch = [&](int k0, moe_u32x4 (&ra)[4], moe_u32x4 (&rw)[4]) {
     const int kk = k0 + lk, kc = min(kk, K - 8);  // loads stand under no condition; a chunk beyond the row counts as zeros
     const uint32_t keep = kk < K ? 0xffffffffu : 0u;
-    const moe_u32x4 x = *reinterpret_cast<const moe_u32x4*>(ap + kc);
-    ra = moe_u32x4{x[0] & keep, x[1] & keep, x[2] & keep, x[3] & keep};
 #pragma unroll
-    for (int i = 0; i < WL; ++i) rw[i] = *reinterpret_cast<const moe_u32x4*>(wp[i] + kc);
-  };
-  auto stage = [&](int buf) {
-    *reinterpret_cast<moe_u32x4*>(&sa[buf][lrow][lk]) = ra;
-#pragma unroll
-    for (int i = 0; i < WL; ++i) *reinterpret_cast<moe_u32x4*>(&sw[buf][lrow + 64 * i][lk]) = rw[i];
-  };
-  fetch(0);
-  stage(0);
-  __syncthreads();
-  int buf = 0;
-  for (int k0 = 0; k0 < K; k0 += 32) {
-    const bool more = k0 + 32 < K;
-    if (more) fetch(k0 + 32);
-    moe_u32x4 av[4], wv[2], wu[2];
-#pragma unroll
-    for (int rt = 0; rt < 4; ++rt) av[rt] = *reinterpret_cast<const moe_u32x4*>(&sa[buf][16 * rt + col][8 * g]);
-#pragma unroll
-    for (int nt = 0; nt < 2; ++nt) {
-      wv[nt] = *reinterpret_cast<const moe_u32x4*>(&sw[buf][wave * 32 + 16 * nt + col][8 * g]);
-      if (GLU) wu[nt] = *reinterpret_cast<const moe_u32x4*>(&sw[buf][MOE_BN + wave * 32 + 16 * nt + col][8 * g]);
+    for (int i = 0; i < 4; ++i) {
+      const moe_u32x4 x = *reinterpret_cast<const moe_u32x4*>(ap[i] + kc);
+      ra[i] = moe_u32x4{x[0] & keep, x[1] & keep, x[2] & keep, x[3] & keep};
+      rw[i] = *reinterpret_cast<const moe_u32x4*>(wp[i] + kc);
     }
+  };
+  auto stage = [&](int buf, const moe_u32x4 (&ra)[4], const moe_u32x4 (&rw)[4]) {
 #pragma unroll
-    for (int rt = 0; rt < 4; ++rt)
+    for (int i = 0; i < 4; ++i) {
+      *reinterpret_cast<moe_u32x4*>(sa + ((size_t)buf * MOE_BIG + lrow + 32 * i) * MOE_BIG_LD + lk) = ra[i];
+      *reinterpret_cast<moe_u32x4*>(sw + ((size_t)buf * MOE_BIG + lrow + 32 * i) * MOE_BIG_LD + lk) = rw[i];
+    }
+  };
+  const bool active = wr * 64 < rows;
+  auto multiply = [&](int buf) {
+    if (!active) return;  // the whole wave
 #pragma unroll
-      for (int nt = 0; nt < 2; ++nt) {
-        acc[rt][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(moe_as_bf16x8(wv[nt]), moe_as_bf16x8(av[rt]), acc[rt][nt], 0, 0, 0);
-        if (GLU) acc_up[rt][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(moe_as_bf16x8(wu[nt]), moe_as_bf16x8(av[rt]), acc_up[rt][nt], 0, 0, 0);
+    for (int ks = 0; ks < MOE_BIG_K; ks += 32) {
+      moe_u32x4 av[4], wv[4];
+#pragma unroll
+      for (int rt = 0; rt < 4; ++rt)
+        av[rt] = *reinterpret_cast<const moe_u32x4*>(sa + ((size_t)buf * MOE_BIG + wr * 64 + 16 * rt + col) * MOE_BIG_LD + ks + 8 * g);
+#pragma unroll
+      for (int nt = 0; nt < 4; ++nt) {
+        const int r = GLU ? (nt < 2 ? wc * 32 + 16 * nt : BN + wc * 32 + 16 * (nt - 2)) : wc * 64 + 16 * nt;
+        wv[nt] = *reinterpret_cast<const moe_u32x4*>(sw + ((size_t)buf * MOE_BIG + r + col) * MOE_BIG_LD + ks + 8 * g);
       }
-    if (more) stage(buf ^ 1);  // nobody reads that buffer: every wave has passed the barrier behind the step that did
-    __syncthreads();
-    buf ^= 1;
+#pragma unroll
+      for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+        for (int nt = 0; nt < 4; ++nt)
+          acc[rt][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(moe_as_bf16x8(wv[nt]), moe_as_bf16x8(av[rt]), acc[rt][nt], 0, 0, 0);
+    }
+  };
+  const int steps = (K + MOE_BIG_K - 1) / MOE_BIG_K;
+  fetch(0, ra0, rw0);
+  fetch(MOE_BIG_K, ra1, rw1);  // beyond K: clamped and zero
+  stage(0, ra0, rw0);
+  lds_barrier();
+  for (int st = 0; st < steps; st += 2) {  // the buffers and the register sets take turns; conditions are uniform over the workgroup
+    if (st + 2 < steps) fetch((st + 2) * MOE_BIG_K, ra0, rw0);
+    multiply(0);
+    if (st + 1 >= steps) break;
+    stage(1, ra1, rw1);  // nobody reads that buffer: every wave has passed the barrier behind the step that did
+    lds_barrier();
+    if (st + 3 < steps) fetch((st + 3) * MOE_BIG_K, ra1, rw1);
+    multiply(1);
+    if (st + 2 < steps) stage(0, ra0, rw0);
+    lds_barrier();
   }
 #pragma unroll
   for (int rt = 0; rt < 4; ++rt) {
-    if (16 * rt + col >= rows) continue;
+    const int row = wr * 64 + 16 * rt + col;
+    if (row >= rows) continue;
 #pragma unroll
-    for (int nt = 0; nt < 2; ++nt)
+    for (int nt = 0; nt < (GLU ? 2 : 4); ++nt) {
+      const int o = o0 + wc * (GLU ? 32 : 64) + 16 * nt + 4 * g;
+      if (o >= F) continue;
+      float v[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int o = o0 + wave * 32 + 16 * nt + 4 * g + r;
-        if (o < F)
-          out[(size_t)(first + 16 * rt + col) * o_stride + o] = from_float<TO>(GLU ? moe_act(acc[rt][nt][r], acc_up[rt][nt][r], act, limit, up_shift) : lev_activate(acc[rt][nt][r], act));
-      }
+      for (int r = 0; r < 4; ++r) v[r] = GLU ? moe_act(acc[rt][nt][r], acc[rt][(nt + 2) & 3][r], act, limit, up_shift) : lev_activate(acc[rt][nt][r], act);
+      moe_store4<TO>(out + (size_t)(first + row) * o_stride + o, v, F - o, vec);
+    }
   }
 }
 
@@ -443,7 +560,7 @@ extern "C" int lev_moe_linear(const void* a, long a_stride, const void* w, void*
   LEV_REQUIRE(a && w && out && tiles && meta && sorted, "experts: a tensor is missing");
   LEV_REQUIRE(K > 0 && N > 0 && (!glu || N % 2 == 0) && top > 0 && max_tiles >= 0, "experts: bad sizes K=%d N=%d", K, N);
   LEV_REQUIRE(act >= 0 && act <= LEV_ACT_LAST, "experts: unknown activation %d", act);
-  LEV_REQUIRE(tile_rows == MOE_TM || tile_rows == 4 * MOE_TM, "experts: tiles of %d rows (%d or %d)", tile_rows, MOE_TM, 4 * MOE_TM);
+  LEV_REQUIRE(tile_rows == MOE_TM || tile_rows == MOE_BIG, "experts: tiles of %d rows (%d or %d)", tile_rows, MOE_TM, MOE_BIG);
   LEV_REQUIRE(dtype == LEV_F32 || dtype == LEV_BF16, "experts: unknown dtype %d", dtype);
   LEV_REQUIRE(dtype == LEV_BF16 || out_dtype == LEV_F32, "experts: float32 inputs give float32 outputs");
   const int F = glu ? N / 2 : N;
@@ -465,20 +582,25 @@ extern "C" int lev_moe_linear(const void* a, long a_stride, const void* w, void*
 #undef MOE_SPLITK
       return lev_check_launch("moe_linear (matrix cores, K split)");
     }
-    if (tile_rows != MOE_TM) {  // tiles of 64 rows: operands through LDS
-      dim3 grid_t(max_tiles, (F + MOE_BN - 1) / MOE_BN);
-#define MOE_TILE(TO)                                                                                                                             \
-  do {                                                                                                                                           \
-    if (glu)                                                                                                                                     \
-      moe_linear_tile_kernel<TO, true><<<grid_t, 256, 0, stream>>>((const bf16_t*)a, a_stride, (const bf16_t*)w, (TO*)out, o_stride, tiles, meta,   \
-                                                                  sorted, top, gather, K, N, F, act, limit, up_shift);                                            \
-    else                                                                                                                                         \
-      moe_linear_tile_kernel<TO, false><<<grid_t, 256, 0, stream>>>((const bf16_t*)a, a_stride, (const bf16_t*)w, (TO*)out, o_stride, tiles, meta,  \
-                                                                   sorted, top, gather, K, N, F, act, limit, up_shift);                                           \
+    if (tile_rows == MOE_BIG) {
+      const int bn = glu ? MOE_BIG / 2 : MOE_BIG, n_cols = (F + bn - 1) / bn;
+      const long blocks = (long)((max_tiles + 7) / 8) * 8 * n_cols;
+      LEV_REQUIRE(blocks <= 0x7fffffffL, "experts: too many tiles (%ld)", blocks);
+      const int vec = o_stride % 4 == 0 && ((uintptr_t)out & (out_dtype == LEV_F32 ? 15 : 7)) == 0;
+#define MOE_BIG_CASE(TO, G)                                                                                                                       \
+  do {                                                                                                                                            \
+    hipError_t e = hipFuncSetAttribute((const void*)moe_linear_big_kernel<TO, G>, hipFuncAttributeMaxDynamicSharedMemorySize, MOE_BIG_LDS);        \
+    LEV_REQUIRE(e == hipSuccess, "experts: %d bytes of LDS a workgroup: %s", MOE_BIG_LDS, hipGetErrorString(e));                                   \
+    moe_linear_big_kernel<TO, G><<<(unsigned)blocks, 256, MOE_BIG_LDS, stream>>>((const bf16_t*)a, a_stride, (const bf16_t*)w, (TO*)out, o_stride, tiles, \
+                                                                                meta, sorted, top, gather, K, N, F, act, limit, up_shift, n_cols, vec); \
   } while (0)
-      if (out_dtype == LEV_F32) MOE_TILE(float); else MOE_TILE(bf16_t);
-#undef MOE_TILE
-      return lev_check_launch("moe_linear (matrix cores, tiles through LDS)");
+      if (out_dtype == LEV_F32) {
+        if (glu) MOE_BIG_CASE(float, true); else MOE_BIG_CASE(float, false);
+      } else {
+        if (glu) MOE_BIG_CASE(bf16_t, true); else MOE_BIG_CASE(bf16_t, false);
+      }
+#undef MOE_BIG_CASE
+      return lev_check_launch("moe_linear (matrix cores, tiles of 128 rows)");
     }
     // many tiles of 16 rows: a wave per tile and 32 outputs, both operands straight from global memory
     const int nt = 2;

@@ -284,7 +284,8 @@ register_unit("core", ["errors.hip", "elementwise.hip", "layer_ops.hip", "gemm_s
     "lev_delta_rule": [_P] * 5 + [_L, _P, _L, _P, _P, _P, _P, _L, _I, _I, _I, _F, _F, _F, _I, _P],
     "lev_delta_rule_scan": [_P] * 5 + [_L, _P, _L, _P, _P, _P, _P, _L, _P, _I, _I, _I, _I, _F, _F, _F, _I, _P],
     "lev_delta_rule_scan_workspace": [_I, _I, _I],
-    "lev_moe_route": [_P, _L, _P] + [_I] * 8 + [_P, _P, _P],
+    "lev_moe_route": [_P, _L, _P] + [_I] * 9 + [_P, _P, _P],
+    "lev_moe_route_sort": [_P, _L, _P] + [_I] * 9 + [_P, _P, _I, _I] + [_P] * 5,
     "lev_moe_max_tiles": [_I, _I, _I],
     "lev_moe_sort": [_P, _I, _I, _I, _I, _P, _P, _P, _P, _P],
     "lev_moe_linear": [_P, _L, _P, _P, _L, _P, _P, _P] + [_I] * 8 + [_F, _F, _I, _I, _I, _P],

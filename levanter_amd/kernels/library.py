@@ -1171,25 +1171,45 @@ class HipKernels:
 
     # ---- mixture of experts --------------------------------------------------------------------
     def moe_route(self, z, correction, chosen, weights, *, n_groups: int = 1, keep: int = 1, group_top: int = 2, renormalize: bool = False,
-                  scoring: str = "sigmoid") -> None:
+                  scoring: str = "sigmoid", extra: bool = False) -> None:
         """Per token: ``s = sigmoid(z)`` (``z`` float32 ``[T, E]``), with ``scoring`` "softmax" the softmax of ``z`` over all E, with "softmax_chosen"
         ``z`` itself, the weights then being the softmax over the winners' ``s``; the choice goes by ``s + correction``; only experts of the
         ``keep`` groups (of ``n_groups`` equal groups of neighbours) whose ``group_top`` largest choice scores sum highest can be
         chosen; ``chosen`` int32 ``[T, top]`` the winners in the order of falling choice score (ties: lower index first),
-        ``weights`` float32 ``[T, top]`` their ``s`` (divided by their sum with ``renormalize``)."""
+        ``weights`` float32 ``[T, top]`` their ``s`` (divided by their sum with ``renormalize``). ``extra``: one column more, expert E with
+        weight 1 for every token."""
+        self._check(self.lib.lev_moe_route(*self._route_args(z, correction, chosen, weights, n_groups, keep, group_top, renormalize, scoring, extra), self._s()))
+
+    def _route_args(self, z, correction, chosen, weights, n_groups, keep, group_top, renormalize, scoring, extra):
         _dev(z, correction, chosen, weights)
         T, E = z.shape
-        top = chosen.shape[1]
+        cols = chosen.shape[1]
         _req(z.dtype == torch.float32 and chosen.dtype == torch.int32 and weights.dtype == torch.float32, "experts: logits and weights float32, choices int32")
-        _req(tuple(chosen.shape) == tuple(weights.shape) == (T, top) and chosen.is_contiguous() and weights.is_contiguous(), "experts: choices and weights must be [T, top]")
+        _req(tuple(chosen.shape) == tuple(weights.shape) == (T, cols) and chosen.is_contiguous() and weights.is_contiguous(), "experts: choices and weights must be [T, top]")
         _req(correction is None or (correction.dtype == torch.float32 and correction.numel() == E and correction.is_contiguous()), "experts: the correction must be float32 [E]")
-        self._check(self.lib.lev_moe_route(_ptr(z), _rows(z, "experts: z"), _ptr(correction), T, E, int(n_groups), int(keep), int(group_top), top,
-                                           int(renormalize), self.MOE_SCORING[scoring], _ptr(chosen), _ptr(weights), self._s()))
+        return (_ptr(z), _rows(z, "experts: z"), _ptr(correction), T, E, int(n_groups), int(keep), int(group_top), cols - int(bool(extra)), int(renormalize),
+                self.MOE_SCORING[scoring], int(bool(extra)), _ptr(chosen), _ptr(weights))
+
+    def moe_route_sort(self, z, correction, chosen, weights, sorted_pairs, pos_of, tiles, meta, *, n_groups: int = 1, keep: int = 1, group_top: int = 2,
+                       renormalize: bool = False, scoring: str = "sigmoid", extra: bool = False, tile_rows: int = 16, n_real: Optional[int] = None) -> None:
+        """``moe_route`` and ``moe_sort`` (of E experts, E + 1 with ``extra``), for a few tokens in one kernel."""
+        n_experts = z.shape[1] + int(bool(extra))
+        args = self._route_args(z, correction, chosen, weights, n_groups, keep, group_top, renormalize, scoring, extra)
+        self._sort_check(chosen, n_experts, sorted_pairs, pos_of, tiles, meta, tile_rows)
+        rc = self.lib.lev_moe_route_sort(*args, int(n_experts if n_real is None else n_real), int(tile_rows), _ptr(sorted_pairs), _ptr(pos_of), _ptr(tiles),
+                                         _ptr(meta), self._s())
+        if rc < 0:
+            self._check(rc)
+        if rc > 0:
+            self._check(self.lib.lev_moe_route(*args, self._s()))
+            self.moe_sort(chosen, n_experts, sorted_pairs, pos_of, tiles, meta, tile_rows=tile_rows, n_real=n_real)
 
     @staticmethod
     def moe_tile_rows(pairs: int, n_experts: int) -> int:
-        """Rows of a tile of the experts' products: 64 where an expert has 32 rows or more on average, else 16."""
-        return 64 if pairs >= 32 * n_experts else 16
+        """Rows of a tile of the experts' products: 128 where an expert has 12 rows or more on average, else 16 (32 experts of 2048 x 2048,
+        4 a token, microseconds of the two products, 16 / 128: 64 tokens 56 + 57 / 51 + 50 (gated 126 / 135 for the first), 128 tokens 96 + 89 /
+        53 + 51, 256 tokens 137 + 140 / 55 + 55)."""
+        return 128 if pairs >= 12 * n_experts else 16
 
     def moe_max_tiles(self, pairs: int, n_experts: int, tile_rows: int = 16) -> int:
         return int(self.lib.lev_moe_max_tiles(int(pairs), int(n_experts), int(tile_rows)))
@@ -1199,12 +1219,16 @@ class HipKernels:
         inverse, ``tiles`` int32 ``[max_tiles, 3]`` (expert, first place, rows <= ``tile_rows``) covering every expert's stretch,
         ``meta[0]`` their number. Everything stays on the device. ``n_real``: only the experts below it have weights; the pairs of the others
         get places and no tiles (``moe_combine`` gives them the token's own input)."""
+        P = self._sort_check(chosen, n_experts, sorted_pairs, pos_of, tiles, meta, tile_rows)
+        self._check(self.lib.lev_moe_sort(_ptr(chosen), P, int(n_experts), int(n_experts if n_real is None else n_real), int(tile_rows), _ptr(sorted_pairs), _ptr(pos_of), _ptr(tiles), _ptr(meta), self._s()))
+
+    def _sort_check(self, chosen, n_experts, sorted_pairs, pos_of, tiles, meta, tile_rows) -> int:
         _dev(chosen, sorted_pairs, pos_of, tiles, meta)
         P = chosen.numel()
         for t in (chosen, sorted_pairs, pos_of, tiles, meta):
             _req(t.dtype == torch.int32 and t.is_contiguous(), "experts: int32 tables")
         _req(sorted_pairs.numel() >= P and pos_of.numel() >= P and tiles.numel() >= 3 * self.moe_max_tiles(P, n_experts, tile_rows) and meta.numel() >= 1, "experts: tables too small")
-        self._check(self.lib.lev_moe_sort(_ptr(chosen), P, int(n_experts), int(n_experts if n_real is None else n_real), int(tile_rows), _ptr(sorted_pairs), _ptr(pos_of), _ptr(tiles), _ptr(meta), self._s()))
+        return P
 
     def moe_linear(self, a, w, out, tiles, meta, sorted_pairs, *, top: int, gather: bool, glu: bool = False, activation: str = "none",
                    tile_rows: int = 16, limit: float = 0.0, up_shift: float = 0.0) -> None:

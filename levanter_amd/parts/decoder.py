@@ -114,9 +114,9 @@ class DecoderLm:
     def weight_bytes(self) -> int:
         seen, total = set(), 0
         for obj in self._walk(self):
-            if isinstance(obj, torch.Tensor) and obj.data_ptr() not in seen:
-                seen.add(obj.data_ptr())
-                total += obj.numel() * obj.element_size()
+            if isinstance(obj, torch.Tensor) and obj.untyped_storage().data_ptr() not in seen:  # parts may hold pieces of one tensor
+                seen.add(obj.untyped_storage().data_ptr())
+                total += obj.untyped_storage().nbytes()
         return total
 
     def _walk(self, obj, depth=0):

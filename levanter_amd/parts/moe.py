@@ -26,6 +26,7 @@ import torch
 
 from levanter_amd.kernels.library import ACTIVATIONS, PendingExperts
 from .base import BuildEnv, FeedForward, StepContext
+from .feed_forward import GatedMlp
 from .linear import Linear
 from .embedding import tensors_of_nested
 from .registry import FEED_FORWARDS, part_class
@@ -87,8 +88,22 @@ class RoutedExperts(FeedForward):
                 w_in[e, :F] = f32(f"experts.{e}.gate.weight", (F, D))
             w_in[e, -Fp:][:F] = f32(f"experts.{e}.up.weight", (F, D))
             w_down[e, :, :F] = f32(f"experts.{e}.down.weight", (D, F))
+        # A shared expert of the experts' own form stands behind them as one more expert: in a step of few tokens it is a choice that every
+        # token makes (no products of its own); in others its own products are the faster ones. Both read the same memory.
+        self.joined = False
+        sh = self.shared
+        if sh is not None and not self.n_identity and all(hasattr(sh, a) for a in ("up", "down", "activation")):
+            same = (tuple(sh.up.weight.shape) == tuple(w_in.shape[1:]) and tuple(sh.down.weight.shape) == (D, Fp) and sh.up.bias is None and sh.down.bias is None
+                    and ACTIVATIONS[sh.activation] == ACTIVATIONS[self.activation] and isinstance(sh, GatedMlp) == self.gated
+                    and getattr(sh, "limit", 0.0) == self.limit and getattr(sh, "up_shift", 0.0) == self.up_shift)
+            if same:
+                w_in = torch.cat([w_in, sh.up.weight.to(torch.float32).cpu()[None]], 0)
+                w_down = torch.cat([w_down, sh.down.weight.to(torch.float32).cpu()[None]], 0)
+                self.joined = True
         self.w_in = w_in.to(env.device, env.dtype).contiguous()
         self.w_down = w_down.to(env.device, env.dtype).contiguous()
+        if self.joined:
+            sh.up.weight, sh.down.weight = self.w_in[E], self.w_down[E]
 
     def forward(self, h: torch.Tensor, x: torch.Tensor, ctx: StepContext) -> None:
         self._run(h, x, ctx, True)
@@ -107,35 +122,38 @@ class RoutedExperts(FeedForward):
         if self.n_identity:
             self.compute(h, y, ctx)
             return None
-        expert_out, pos_of, weights, _ = self._experts(h, ctx)
-        if self.shared is not None:
+        expert_out, pos_of, weights, _, whole = self._experts(h, ctx)
+        if not whole:
             self.shared.compute(h, y, ctx)
-        return PendingExperts(expert_out, pos_of, weights, alone=self.shared is None)
+        return PendingExperts(expert_out, pos_of, weights, alone=whole)
 
     def _experts(self, h: torch.Tensor, ctx: StepContext, z=None):
         """Routing and the chosen experts' products: their outputs (float32 ``[T * top, dim]``, in the order of the experts), every pair's place
-        among them, the weights and the choices ``[T, top]``."""
+        among them, the weights and the choices ``[T, top]``, and whether that is the whole result (no shared expert, or one that is the last
+        of the choices, which are top + 1 then)."""
         K = ctx.kernels
         T, E, top = h.shape[0], self.n_outputs, self.top
         dev = h.device
         if z is None:
             z = self.router(h, ctx, out_dtype=torch.float32)
+        joined = self.joined and K.moe_tile_rows(T * (top + 1), E + 1) == 16
+        if joined:
+            E, top = E + 1, top + 1
         chosen = torch.empty((T, top), dtype=torch.int32, device=dev)
         weights = torch.empty((T, top), dtype=torch.float32, device=dev)
-        more = {"scoring": self.score} if self.score != "sigmoid" else {}
-        K.moe_route(z, self.correction, chosen, weights, n_groups=self.n_groups, keep=self.keep, group_top=self.group_top, renormalize=self.renormalize, **more)
         P = T * top
-        rows = K.moe_tile_rows(P, E)  # prompts: four row tiles on every weight fragment a wave loads
+        rows = K.moe_tile_rows(P, E)
         tables = torch.empty(2 * P + 3 * K.moe_max_tiles(P, E, rows) + 1, dtype=torch.int32, device=dev)
         sorted_pairs, pos_of, meta, tiles = tables[:P], tables[P:2 * P], tables[2 * P:2 * P + 1], tables[2 * P + 1:]
         own = {"n_real": self.n_experts} if self.n_identity else {}
-        K.moe_sort(chosen, E, sorted_pairs, pos_of, tiles, meta, tile_rows=rows, **own)
+        K.moe_route_sort(z, self.correction, chosen, weights, sorted_pairs, pos_of, tiles, meta, n_groups=self.n_groups, keep=self.keep, group_top=self.group_top,
+                         renormalize=self.renormalize, scoring=self.score, extra=joined, tile_rows=rows, **own)
         inner = ctx.empty(P, self.inner_padded)
         clamp = {"limit": self.limit, "up_shift": self.up_shift} if self.limit or self.up_shift else {}
         K.moe_linear(h, self.w_in, inner, tiles, meta, sorted_pairs, top=top, gather=True, glu=self.gated, activation=self.activation, tile_rows=rows, **clamp)
         expert_out = ctx.empty(P, self.dim, torch.float32)
         K.moe_linear(inner, self.w_down, expert_out, tiles, meta, sorted_pairs, top=top, gather=False, tile_rows=rows)
-        return expert_out, pos_of, weights, chosen
+        return expert_out, pos_of, weights, chosen, joined or self.shared is None
 
     def _run(self, h: torch.Tensor, y: torch.Tensor, ctx: StepContext, accumulate: bool, z=None) -> None:
         K = ctx.kernels
@@ -143,12 +161,12 @@ class RoutedExperts(FeedForward):
             z = self.router(h, ctx, out_dtype=torch.float32)
         if accumulate:
             ctx.settle()  # the sum below reads the residual stream itself
-        expert_out, pos_of, weights, chosen = self._experts(h, ctx, z)
+        expert_out, pos_of, weights, chosen, whole = self._experts(h, ctx, z)
         if self.n_identity:
             K.moe_combine(expert_out, pos_of, weights, y, accumulate=accumulate, chosen=chosen, n_real=self.n_experts, identity_in=h)
         else:
             K.moe_combine(expert_out, pos_of, weights, y, accumulate=accumulate)
-        if self.shared is not None:
+        if not whole:
             may_defer, ctx.may_defer = ctx.may_defer, False  # y is not the residual stream: its sum is finished here
             self.shared.forward(h, y, ctx)  # added to the experts' sum
             ctx.may_defer = may_defer

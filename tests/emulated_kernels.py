@@ -405,8 +405,11 @@ class EmulatedKernels:
         y.copy_(y + s if accumulate else s)
 
     # ---- mixture of experts
-    def moe_route(self, z, correction, chosen, weights, *, n_groups=1, keep=1, group_top=2, renormalize=False, scoring="sigmoid") -> None:
+    def moe_route(self, z, correction, chosen, weights, *, n_groups=1, keep=1, group_top=2, renormalize=False, scoring="sigmoid", extra=False) -> None:
         T, E = z.shape
+        if extra:
+            chosen[:, -1], weights[:, -1] = E, 1.0
+            chosen, weights = chosen[:, :-1], weights[:, :-1]
         top = chosen.shape[1]
         s = z.float() if scoring == "softmax_chosen" else torch.softmax(z.float(), -1) if scoring == "softmax" else torch.sigmoid(z.float())
         c = s if correction is None else s + correction
@@ -423,9 +426,13 @@ class EmulatedKernels:
             wt = s[t][order]
             weights[t] = torch.softmax(wt, -1) if scoring == "softmax_chosen" else wt / wt.sum() if renormalize else wt
 
+    def moe_route_sort(self, z, correction, chosen, weights, sorted_pairs, pos_of, tiles, meta, *, tile_rows=16, n_real=None, extra=False, **kw) -> None:
+        self.moe_route(z, correction, chosen, weights, extra=extra, **kw)
+        self.moe_sort(chosen, z.shape[1] + int(extra), sorted_pairs, pos_of, tiles, meta, tile_rows=tile_rows, n_real=n_real)
+
     @staticmethod
     def moe_tile_rows(pairs, n_experts) -> int:
-        return 64 if pairs >= 32 * n_experts else 16
+        return 128 if pairs >= 12 * n_experts else 16
 
     def moe_max_tiles(self, pairs, n_experts, tile_rows=16) -> int:
         return pairs // tile_rows + n_experts + 1

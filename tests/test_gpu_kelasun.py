@@ -228,8 +228,39 @@ def test_the_router_that_weights_by_a_softmax_over_the_chosen(T, E, top):
     torch.testing.assert_close(weights.cpu().double(), want_w, rtol=2e-5, atol=1e-6)
 
 
+@pytest.mark.parametrize("T,E,G,keep,top,scoring,extra", [(1, 8, 1, 1, 2, "softmax_chosen", True), (16, 32, 1, 1, 4, "softmax_chosen", True), (7, 18, 3, 2, 4, "sigmoid", False),
+                                                           (13, 256, 64, 5, 8, "softmax", False), (5, 12, 6, 6, 12, "sigmoid", True), (17, 8, 1, 1, 2, "softmax_chosen", True),
+                                                           (9, 300, 1, 1, 3, "softmax", True), (200, 1024, 1, 1, 32, "softmax_chosen", True), (3, 1, 1, 1, 1, "softmax_chosen", True)])
+def test_routing_and_sorting_in_one_kernel(T, E, G, keep, top, scoring, extra):
+    """The choices and weights of the routing kernel, bit for bit, with one choice more if asked for; every pair has one place, experts lie
+    in rising order, and the tiles cover them (also beyond the sizes of the one kernel, where two run)."""
+    kern = K()
+    g = torch.Generator().manual_seed(E + T)
+    z, corr = dev(torch.randn(T, E, generator=g) * 2), dev(torch.randn(E, generator=g) * 0.1)
+    n, cols = E + int(extra), top + int(extra)
+    Pn = T * cols
+    rows = kern.moe_tile_rows(Pn, n)
+    want_c, want_w = torch.empty(T, top, dtype=torch.int32, device=DEV), torch.empty(T, top, device=DEV)
+    kw = dict(n_groups=G, keep=keep, group_top=2, scoring=scoring, renormalize=scoring == "sigmoid")
+    kern.moe_route(z, corr, want_c, want_w, **kw)
+    chosen, weights = torch.full((T, cols), -1, dtype=torch.int32, device=DEV), torch.full((T, cols), -1.0, device=DEV)
+    tables = torch.full((2 * Pn + 3 * kern.moe_max_tiles(Pn, n, rows) + 1,), -7, dtype=torch.int32, device=DEV)
+    sorted_pairs, pos_of, meta, tiles = tables[:Pn], tables[Pn:2 * Pn], tables[2 * Pn:2 * Pn + 1], tables[2 * Pn + 1:]
+    n_real = n if extra else max(1, E - 2)
+    kern.moe_route_sort(z, corr, chosen, weights, sorted_pairs, pos_of, tiles, meta, extra=extra, tile_rows=rows, n_real=n_real, **kw)
+    assert torch.equal(chosen[:, :top], want_c) and torch.equal(weights[:, :top], want_w)
+    if extra:
+        assert bool((chosen[:, top] == E).all()) and bool((weights[:, top] == 1.0).all())
+    sp, po, flat = sorted_pairs.cpu().long(), pos_of.cpu().long(), chosen.cpu().reshape(-1).long()
+    assert torch.equal(sp[po], torch.arange(Pn)) and torch.equal(flat[sp], flat.sort().values)
+    tl = tiles.cpu().view(-1, 3)[:int(meta[0])]
+    covered = torch.cat([torch.arange(int(f), int(f) + int(m)) for _, f, m in tl])
+    assert torch.equal(covered, torch.arange(int((flat < n_real).sum())))
+    assert all(bool((flat[sp][int(f):int(f) + int(m)] == int(e)).all()) and 0 < int(m) <= rows for e, f, m in tl)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("T,D,F,E,top,shared", [(37, 64, 24, 6, 3, 24), (1, 32, 8, 2, 2, None), (300, 96, 48, 4, 2, 40), (5, 40, 13, 9, 1, 16), (700, 64, 24, 30, 4, 64), (400, 64, 160, 5, 2, None)])
+@pytest.mark.parametrize("T,D,F,E,top,shared", [(37, 64, 24, 6, 3, 24), (1, 32, 8, 2, 2, None), (300, 96, 48, 4, 2, 40), (5, 40, 13, 9, 1, 16), (5, 40, 16, 9, 2, 16), (16, 64, 32, 7, 1, 32), (20, 64, 32, 16, 3, 32), (700, 64, 24, 30, 4, 64), (400, 64, 160, 5, 2, None)])
 def test_experts_without_gates_beside_a_shared_one(dtype, T, D, F, E, top, shared):
     """Few tokens, tiles of 16 rows and of 64: the part's own result, the result added to a stream, and the sum left to the pass that reads it."""
     from levanter_amd.parts import BuildEnv, PartSpec, TensorSpec, part_class
@@ -263,7 +294,8 @@ def test_experts_without_gates_beside_a_shared_one(dtype, T, D, F, E, top, share
     torch.testing.assert_close(x.cpu().double()[clear], (x0.double() + want)[clear], **limits)
     y = torch.full((T, D), float("nan"), device=DEV)
     left = part.compute_unsummed(dev(h, dtype), y, ctx)
-    assert left.alone == (shared is None)
+    # a shared expert of the experts' size (filled up to a multiple of 8) is the last choice of every token where the experts have few rows each
+    assert left.alone == (shared is None or (shared == (F + 7) // 8 * 8 and T * (top + 1) < 12 * (E + 1)))
     product = ctx.take_product_pending(y)
     x, nw = dev(x0), torch.ones(D, device=DEV)
     K().finish(K().sum_norm_step(x, alpha=2.0, y=None if left.alone or product is not None else y, product=product, experts=left, write_norm=(nw, None, 1e-5, False), defer=True))
