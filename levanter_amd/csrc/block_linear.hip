@@ -111,6 +111,7 @@ block_linear_mfma_kernel(const TA* __restrict__ a, long a_stride, const bf16_t* 
   blm_f32x4 acc[BLM_NT];
 #pragma unroll
   for (int nt = 0; nt < BLM_NT; ++nt) acc[nt] = blm_f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
   for (int k0 = 0; k0 < n_in; k0 += 32) {
     const int kk = k0 + 8 * g, kc = min(kk, n_in - 8);  // loads stand under no condition; a chunk beyond the row counts as zeros
     blm_u32x4 av = blm_load8(arow + kc);

@@ -24,11 +24,11 @@
 
 #define MOE_TM 16          // rows of a matrix-core row tile, and of a tile of the list in steps of few tokens
 #define MOE_BIG 128        // rows of a tile of the list in the others
-#define MOE_MAX_E 1024     // experts
+#define MOE_MAX_E 1024     // experts (at most 32 a lane)
 #define MOE_MAX_TOP 32
 
 // ---- route ------------------------------------------------------------------------------------
-// One wave routes one token; s_s, c_s (and g_s with groups) are E (G) numbers, sel MOE_MAX_TOP numbers of its own in LDS. Every wave of
+// One wave routes one token; s_s, c_s (and g_s with groups) are E (G) numbers of its own in LDS. Every wave of
 // the workgroup passes the same barriers. `extra`: a further choice behind the `top` ones, expert E with weight 1 (an expert that runs for
 // every token). store: the wave's token is one of the step's.
 struct MoeRouteArgs {
@@ -39,7 +39,7 @@ struct MoeRouteArgs {
   int* chosen;
   float* weights;
 };
-__device__ __forceinline__ void moe_route_token(const MoeRouteArgs& a, int t, bool store, float* s_s, float* c_s, float* g_s, int* sel) {
+__device__ __forceinline__ void moe_route_token(const MoeRouteArgs& a, int t, bool store, float* s_s, float* c_s, float* g_s) {
   const int lane = threadIdx.x & 63, E = a.E, G = a.G, top = a.top;
   const int per = E / G;
   const float* zt = a.z + (size_t)t * a.z_stride;
@@ -87,15 +87,16 @@ __device__ __forceinline__ void moe_route_token(const MoeRouteArgs& a, int t, bo
     }
     __syncthreads();
   }
+  // the next largest, `top` times: every lane looks through its own experts (e % 64 == lane), the lanes compare; lane n keeps the n-th
   float wsum = 0.f;
+  int mine = 0;
+  uint32_t taken = 0;  // of this lane's experts: bit e / 64
   for (int n = 0; n < top; ++n) {
     float best = -INFINITY;
     int best_e = 0x7fffffff;
-    for (int e = lane; e < E; e += 64) {
-      bool taken = false;
-      for (int p = 0; p < n; ++p) taken = taken || sel[p] == e;
+    for (int e = lane, i = 0; e < E; e += 64, ++i) {
       const float c = c_s[e];
-      if (!taken && (c > best || (c == best && e < best_e))) best = c, best_e = e;
+      if (!(taken >> i & 1u) && (c > best || (c == best && e < best_e))) best = c, best_e = e;
     }
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) {
@@ -104,22 +105,23 @@ __device__ __forceinline__ void moe_route_token(const MoeRouteArgs& a, int t, bo
       if (ob > best || (ob == best && oe < best_e)) best = ob, best_e = oe;
     }
     if (best_e >= E) best_e = 0;  // nothing left to choose from (a configuration that keeps fewer experts than it uses)
-    if (lane == 0) sel[n] = best_e;
+    if ((best_e & 63) == lane) taken |= 1u << (best_e >> 6);
+    if (lane == n) mine = best_e;
     wsum += s_s[best_e];
-    __syncthreads();
   }
   const size_t at = (size_t)t * (top + a.extra);
-  float mx = 0.f;
-  if (a.scoring == 2) {  // every lane sums the same few numbers
-    mx = -INFINITY, wsum = 0.f;
-    for (int n = 0; n < top; ++n) mx = fmaxf(mx, s_s[sel[n]]);
-    for (int n = 0; n < top; ++n) wsum += expf(s_s[sel[n]] - mx);
+  float weight = s_s[mine];
+  if (a.scoring == 2) {
+    const float mx = wave_max(lane < top ? weight : -INFINITY);
+    weight = lane < top ? expf(weight - mx) : 0.f;
+    weight /= wave_sum(weight);
+  } else if (a.renormalize) {
+    weight /= wsum;
   }
   if (!store) return;
   if (lane < top) {
-    const int e = sel[lane];
-    a.chosen[at + lane] = e;
-    a.weights[at + lane] = a.scoring == 2 ? expf(s_s[e] - mx) / wsum : a.renormalize ? s_s[e] / wsum : s_s[e];
+    a.chosen[at + lane] = mine;
+    a.weights[at + lane] = weight;
   } else if (lane == top && a.extra) {
     a.chosen[at + top] = E;
     a.weights[at + top] = 1.0f;
@@ -129,8 +131,7 @@ __device__ __forceinline__ void moe_route_token(const MoeRouteArgs& a, int t, bo
 __global__ void __launch_bounds__(64)
 moe_route_kernel(const MoeRouteArgs a) {
   __shared__ float s_s[MOE_MAX_E], c_s[MOE_MAX_E], g_s[MOE_MAX_E];
-  __shared__ int sel[MOE_MAX_TOP];
-  moe_route_token(a, blockIdx.x, true, s_s, c_s, g_s, sel);
+  moe_route_token(a, blockIdx.x, true, s_s, c_s, g_s);
 }
 
 // ---- sort --------------------------------------------------------------------------------------
@@ -202,11 +203,10 @@ moe_route_sort_kernel(const MoeRouteArgs a, int T, int n_real, int tile_rows, in
                       int* __restrict__ meta) {
   __shared__ MoeSortLds l;
   __shared__ float s_s[MOE_SMALL_T][MOE_SMALL_E], c_s[MOE_SMALL_T][MOE_SMALL_E];
-  __shared__ int sel[MOE_SMALL_T][MOE_MAX_TOP];
   const int wave = threadIdx.x >> 6;
   // the groups' scores take the place of the sort's counters, which nobody needs before the routing is done
   float* g_s = reinterpret_cast<float*>(l.count) + (size_t)wave * MOE_SMALL_E / 4;
-  moe_route_token(a, min(wave, T - 1), wave < T, s_s[wave], c_s[wave], g_s, sel[wave]);
+  moe_route_token(a, min(wave, T - 1), wave < T, s_s[wave], c_s[wave], g_s);
   __syncthreads();  // the choices, in global memory, are the whole workgroup's
   moe_sort_pairs(l, a.chosen, T * (a.top + a.extra), a.E + a.extra, n_real, tile_rows, sorted, pos_of, tiles, meta);
 }

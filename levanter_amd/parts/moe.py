@@ -42,6 +42,10 @@ class RoutedExperts(FeedForward):
     (if gated), ``experts.<e>.up.weight`` ``[inner, dim]``, ``experts.<e>.down.weight`` ``[dim, inner]``."""
 
     graph_safe = True
+    JOIN_MAX = 1 << 23
+    """A shared expert with larger matrices than this keeps products of its own in every step (decode of 8 layers, one token / 8, with the
+    shared expert joined and not: matrices of 1024 x 1024 0.63 / 0.80 and 0.68 / 0.86 ms, 2048 x 2048 0.87 / 1.34 and 0.93 / 1.36 ms,
+    4 layers of 4096 x 4096 0.86 / 1.75 and 0.82 / 1.67 ms: there the plain product streams its weight faster)."""
 
     def __init__(self, spec: PartSpec, tensors: Dict[str, torch.Tensor], env: BuildEnv):
         super().__init__(spec, tensors, env)
@@ -93,7 +97,7 @@ class RoutedExperts(FeedForward):
         self.joined = False
         sh = self.shared
         if sh is not None and not self.n_identity and all(hasattr(sh, a) for a in ("up", "down", "activation")):
-            same = (tuple(sh.up.weight.shape) == tuple(w_in.shape[1:]) and tuple(sh.down.weight.shape) == (D, Fp) and sh.up.bias is None and sh.down.bias is None
+            same = (F * D <= self.JOIN_MAX and tuple(sh.up.weight.shape) == tuple(w_in.shape[1:]) and tuple(sh.down.weight.shape) == (D, Fp) and sh.up.bias is None and sh.down.bias is None
                     and ACTIVATIONS[sh.activation] == ACTIVATIONS[self.activation] and isinstance(sh, GatedMlp) == self.gated
                     and getattr(sh, "limit", 0.0) == self.limit and getattr(sh, "up_shift", 0.0) == self.up_shift)
             if same:
