@@ -95,10 +95,16 @@ __device__ __forceinline__ blm_u32x4 blm_load8(const float* p) {
   return blm_u32x4{float2_to_bf16x2(lo.x, lo.y), float2_to_bf16x2(lo.z, lo.w), float2_to_bf16x2(hi.x, hi.y), float2_to_bf16x2(hi.z, hi.w)};
 }
 
+__device__ __forceinline__ void blm_store4(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+__device__ __forceinline__ void blm_store4(bf16_t* p, const float (&v)[4]) {
+  *reinterpret_cast<uint2*>(p) = make_uint2(float2_to_bf16x2(v[0], v[1]), float2_to_bf16x2(v[2], v[3]));
+}
+
 template <typename TA, typename TO, int BLM_NT>
 __global__ void __launch_bounds__(256)
 block_linear_mfma_kernel(const TA* __restrict__ a, long a_stride, const bf16_t* __restrict__ w, const float* __restrict__ bias,
-                         TO* __restrict__ out, long o_stride, const bf16_t* __restrict__ gate, long g_stride, int T, int n_in, int n_out, int col_sets) {
+                         TO* __restrict__ out, long o_stride, const bf16_t* __restrict__ gate, long g_stride, int T, int n_in, int n_out, int col_sets,
+                         int vec, int vec_gate) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 15, g = lane >> 4;
   const int t0 = (blockIdx.x * 4 + wave) * 16;
   if (t0 >= T) return;  // the whole wave
@@ -127,16 +133,38 @@ block_linear_mfma_kernel(const TA* __restrict__ a, long a_stride, const bf16_t* 
   const int t = t0 + col;
   if (t >= T) return;
 #pragma unroll
-  for (int nt = 0; nt < BLM_NT; ++nt)
+  for (int nt = 0; nt < BLM_NT; ++nt) {
+    const int o = o0 + 16 * nt + 4 * g;
+    if (o >= n_out) continue;
+    const size_t c = (size_t)b * n_out + o;
+    const int n = min(4, n_out - o);
+    float v[4], gv[4] = {0.f, 0.f, 0.f, 0.f};
+    if (gate != nullptr) {
+      const bf16_t* gp = gate + (size_t)t * g_stride + c;
+      if (vec_gate) {
+        const uint2 x = *reinterpret_cast<const uint2*>(gp);
+        gv[0] = __uint_as_float(x.x << 16), gv[1] = __uint_as_float(x.x & 0xffff0000u);
+        gv[2] = __uint_as_float(x.y << 16), gv[3] = __uint_as_float(x.y & 0xffff0000u);
+      } else {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int o = o0 + 16 * nt + 4 * g + r;
-      if (o < n_out) {
-        const size_t c = (size_t)b * n_out + o;
-        const float gv = gate ? 1.0f / (1.0f + expf(-bf16_to_float(gate[(size_t)t * g_stride + c]))) : 1.0f;
-        out[(size_t)t * o_stride + c] = from_float<TO>((acc[nt][r] + (bias ? bias[c] : 0.f)) * gv);
+        for (int r = 0; r < 4; ++r)
+          if (r < n) gv[r] = bf16_to_float(gp[r]);
       }
     }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      v[r] = acc[nt][r] + (bias && r < n ? bias[c + r] : 0.f);
+      if (gate != nullptr) v[r] *= 1.0f / (1.0f + expf(-gv[r]));
+    }
+    TO* op = out + (size_t)t * o_stride + c;
+    if (vec) {  // blocks, rows and the tensor at multiples of four numbers
+      blm_store4(op, v);
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (r < n) op[r] = from_float<TO>(v[r]);
+    }
+  }
 }
 
 extern "C" int lev_block_linear_mfma(const void* a, long a_stride, const void* w, const float* bias, void* out, long o_stride, const void* gate,
@@ -151,14 +179,16 @@ extern "C" int lev_block_linear_mfma(const void* a, long a_stride, const void* w
   const int col_sets = (n_out + 16 * nt - 1) / (16 * nt);
   LEV_REQUIRE((long)B * col_sets <= 65535, "block_linear: too many column tiles (%ld)", (long)B * col_sets);
   dim3 grid((T + 63) / 64, B * col_sets);
+  const int vec = n_out % 4 == 0 && o_stride % 4 == 0 && ((uintptr_t)out & (out_dtype == LEV_F32 ? 15 : 7)) == 0;
+  const int vec_gate = n_out % 4 == 0 && g_stride % 4 == 0 && ((uintptr_t)gate & 7) == 0;
 #define BLM_CASE(A, O, TA, TO)                                                                                                     \
   if (a_dtype == A && out_dtype == O) {                                                                                            \
     if (nt == 1)                                                                                                                   \
       block_linear_mfma_kernel<TA, TO, 1><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, (const bf16_t*)w, bias, (TO*)out, o_stride, (const bf16_t*)gate, g_stride, T, n_in, \
-                                                                   n_out, col_sets);                                               \
+                                                                   n_out, col_sets, vec, vec_gate);                                               \
     else                                                                                                                           \
       block_linear_mfma_kernel<TA, TO, 4><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, (const bf16_t*)w, bias, (TO*)out, o_stride, (const bf16_t*)gate, g_stride, T, n_in, \
-                                                                   n_out, col_sets);                                               \
+                                                                   n_out, col_sets, vec, vec_gate);                                               \
     return lev_check_launch("block_linear (matrix cores)");                                                                       \
   }
   BLM_CASE(LEV_BF16, LEV_BF16, bf16_t, bf16_t)
